@@ -41,7 +41,8 @@ typedef enum {
     A81W41_ERR_INVALID_ARG = 1, /* shape / alignment / null pointer: what the reference asserts on */
     A81W41_ERR_HIP = 2,         /* a HIP runtime call failed */
     A81W41_ERR_IO = 3,          /* weight file missing or short (reference: std::runtime_error) */
-    A81W41_ERR_NO_DEVICE = 4    /* no gfx950 device visible */
+    A81W41_ERR_NO_DEVICE = 4,   /* no gfx950 device visible */
+    A81W41_ERR_UNSUPPORTED = 5  /* the model has no such path or class */
 } a81w41_status;
 
 const char *a81w41_status_string(int status);

@@ -1,6 +1,6 @@
-"""ctypes binding of ``csrc/liba81w41.so`` (the C ABI in ``include/a81w41.h``).
+"""ctypes binding of the libraries in ``csrc/`` (the C ABI in ``include/a81w41.h`` and ``include/a81w41_model.h``).
 
-The library is loaded from the source tree; if it has not been built the call
+``lib()`` is the A81W41 layer with the Qwen3 model, ``core()`` what all models share.  A library is loaded from the source tree; if it has not been built the call
 fails with instructions -- there is no fallback path.
 """
 from __future__ import annotations
@@ -9,9 +9,12 @@ import ctypes as C
 import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
-LIB_PATH = os.path.join(_HERE, "csrc", "liba81w41.so")
+CSRC = os.path.join(_HERE, "csrc")
+LIB_PATH = os.path.join(CSRC, "liba81w41.so")
+CORE_PATH = os.path.join(CSRC, "liba81w41_core.so")
 
 OK = 0
+ERR_UNSUPPORTED = 5
 _vp, _i, _i64, _sz = C.c_void_p, C.c_int, C.c_int64, C.c_size_t
 
 # name -> (restype, argtypes): every symbol include/a81w41.h declares
@@ -80,13 +83,31 @@ SIGNATURES = {
     "a81w41_qwen3_generate_greedy": (_i, [_vp, _vp, _i, _i, _vp, C.POINTER(C.c_double), C.POINTER(C.c_double)]),
 }
 
+# every symbol include/a81w41_model.h declares, and the status functions
+CORE_SIGNATURES = {
+    "a81w41_status_string": (C.c_char_p, [_i]),
+    "a81w41_last_error": (C.c_char_p, []),
+    "a81w41_model_load": (_i, [C.c_char_p, C.c_char_p, _i, C.POINTER(_vp)]),
+    "a81w41_model_create_random": (_i, [C.c_char_p, C.c_char_p, _i, C.c_uint64, C.POINTER(_vp)]),
+    "a81w41_model_destroy": (None, [_vp]),
+    "a81w41_model_vocab": (_i, [_vp]),
+    "a81w41_model_max_seq": (_i, [_vp]),
+    "a81w41_model_position": (_i, [_vp]),
+    "a81w41_model_reset": (_i, [_vp]),
+    "a81w41_model_forward": (_i, [_vp, _vp, _i, _vp, _i, _vp]),
+    "a81w41_model_generate_greedy": (_i, [_vp, _vp, _i, _i, _vp, C.POINTER(C.c_double), C.POINTER(C.c_double)]),
+    "a81w41_model_set_option": (_i, [_vp, C.c_char_p, _i]),
+    "a81w41_model_read_buffer": (_i, [_vp, C.c_char_p, _vp, _sz]),
+    "a81w41_model_resident_bytes": (_sz, [_vp, C.POINTER(_sz), C.POINTER(_sz)]),
+}
+
 
 class Qwen3Config(C.Structure):
     """a81w41_qwen3_config"""
     _fields_ = [("n_layers", _i), ("hidden", _i), ("n_q_heads", _i), ("n_kv_heads", _i), ("intermediate", _i),
                 ("vocab", _i), ("max_seq", _i), ("rope_theta", C.c_float), ("rms_eps", C.c_float)]
 
-_lib = None
+_libs = {}
 
 
 class A81W41Error(RuntimeError):
@@ -95,23 +116,32 @@ class A81W41Error(RuntimeError):
         self.status = status
 
 
-def lib():
-    """Load the HIP library (once) and bind every exported symbol."""
-    global _lib
-    if _lib is None:
-        if not os.path.exists(LIB_PATH):
+def load(path: str, signatures: dict):
+    """Load a library of ``csrc/`` (once) and bind the named symbols."""
+    if path not in _libs:
+        if not os.path.exists(path):
             raise ImportError(
-                f"{LIB_PATH} is missing: build it with `make -C {os.path.dirname(LIB_PATH)}` "
+                f"{path} is missing: build it with `make -C {CSRC}` "
                 "(or __graft_entry__.build()); this package has no CPU fallback")
-        L = C.CDLL(LIB_PATH)
-        for name, (res, args) in SIGNATURES.items():
+        L = C.CDLL(path)
+        for name, (res, args) in signatures.items():
             fn = getattr(L, name)  # AttributeError if the library lacks a declared symbol
             fn.restype = res
             fn.argtypes = args
-        _lib = L
-    return _lib
+        _libs[path] = L
+    return _libs[path]
+
+
+def lib():
+    """The A81W41 layer and the Qwen3 model, every exported symbol bound."""
+    return load(LIB_PATH, SIGNATURES)
+
+
+def core():
+    """The model interface; a model's own library registers with it when it is loaded."""
+    return load(CORE_PATH, CORE_SIGNATURES)
 
 
 def check(status: int) -> None:
     if status != OK:
-        raise A81W41Error(status, lib().a81w41_last_error().decode())
+        raise A81W41Error(status, core().a81w41_last_error().decode())

@@ -197,14 +197,13 @@ namespace a81w41 {
 const void* linear_w6(const a81w41_linear* layer);  // null if the layer has no fp32-parameter blob
 bool linear_block_scaled(const a81w41_linear* layer, int M);  // an M-row call of this layer contracts on the block-scaled kernel
 
-// Records `message` as the calling thread's last error and returns `status` (capi.cpp).
+// Records `message` as the calling thread's last error and returns `status` (status.cpp).
 int report_failure(int status, const char* message);
 // IEEE binary32 -> binary16, round to nearest even (host, capi.cpp).
 uint16_t float_to_half_bits(float f);
 
 // ---- operators around the linears in the Qwen3 forward pass (qwen3_ops.hip) ----------------
 // head_dim is 128; positions are read from device memory (pos_dev[0] = tokens already cached).
-hipError_t launch_embed_rows(const int* ids, const void* table_fp16, float* out, int M, int hidden, int vocab, hipStream_t s);
 hipError_t launch_add_rmsnorm(const float* x, const float* res_in, const float* w, float* res_out, float* norm_out, int M,
                               int hidden, float eps, hipStream_t s);
 // Same, with the normalised rows written as 80 B activation blocks (what the fp32-parameter
@@ -247,8 +246,4 @@ hipError_t launch_attention_one_token_split(const float* qkv, int n_q, int n_kv,
 hipError_t launch_silu_mul(const float* gate_up, float* out, int M, int inter, hipStream_t s);
 // silu(gate) * up as 80 B activation blocks of the [M][inter] result.  inter % 64 == 0, gate_up 16-byte aligned.
 hipError_t launch_silu_mul_quant(const float* gate_up, void* q_out, int M, int inter, hipStream_t s);
-hipError_t launch_argmax_token(const float* logits, int n, int* next_id, int* history, int history_len, int* step_dev,
-                               hipStream_t s);
-hipError_t launch_advance(int* pos_dev, int by, hipStream_t s);
-
 }  // namespace a81w41

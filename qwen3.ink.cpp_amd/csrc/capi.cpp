@@ -22,14 +22,13 @@
 
 namespace {
 
-thread_local char g_err[512] = "";
-
 int fail(int status, const char* fmt, ...) {
     va_list ap;
     va_start(ap, fmt);
-    vsnprintf(g_err, sizeof(g_err), fmt, ap);
+    char buf[512];
+    vsnprintf(buf, sizeof(buf), fmt, ap);
     va_end(ap);
-    return status;
+    return a81w41::report_failure(status, buf);
 }
 
 int hip_fail(hipError_t e, const char* what) {
@@ -169,25 +168,10 @@ bool linear_block_scaled(const a81w41_linear* l, int M) {
     if (!l->w6 || M < kGemmFp6MinRows || l->kernel_choice == A81W41_KERNEL_INT8) return false;
     return l->kernel_choice == A81W41_KERNEL_BLOCK_SCALED || gemm_fp6_preferred(M, l->N, l->K);
 }
-// Lets the other translation units of the library leave their message where a81w41_last_error() finds it.
-int report_failure(int status, const char* message) { return fail(status, "%s", message); }
 uint16_t float_to_half_bits(float f) { return f32_to_f16(f); }
 }  // namespace a81w41
 
 extern "C" {
-
-const char* a81w41_status_string(int status) {
-    switch (status) {
-        case A81W41_OK: return "ok";
-        case A81W41_ERR_INVALID_ARG: return "invalid argument";
-        case A81W41_ERR_HIP: return "HIP runtime error";
-        case A81W41_ERR_IO: return "weight file error";
-        case A81W41_ERR_NO_DEVICE: return "no gfx950 device";
-        default: return "unknown status";
-    }
-}
-
-const char* a81w41_last_error(void) { return g_err; }
 
 size_t a81w41_weight_blob_bytes(int K, int N, int fp32) {
     if (!shape_ok(N, K)) return 0;

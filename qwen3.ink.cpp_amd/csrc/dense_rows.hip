@@ -1,0 +1,162 @@
+// Row kernels around the dense matrix products: norms in groups, the residual step between two norms with an
+// optional weighted mean over depth, and the routing of tokens to experts by a table.  One workgroup per row; the
+// row sits in LDS as fp32.
+#include "dense_common.h"
+
+namespace a81w41 {
+namespace {
+
+constexpr int kThreads = 256;
+
+template <typename T>
+__global__ __launch_bounds__(kThreads) void group_norm_kernel(const float* __restrict__ x, int width, GroupNorm norm, T* __restrict__ out,
+                                                             int ld_out) {
+    extern __shared__ float smem[];
+    float* inv = smem;
+    float* red = inv + norm.groups;
+    const float* row = x + (size_t)blockIdx.x * width;
+    group_inverse_rms<kThreads>([&](int i) { return row[i]; }, width, norm.groups, norm.eps, inv, red);
+    const int size = width / norm.groups;
+    T* dst = out + (size_t)blockIdx.x * ld_out;
+    for (int i = threadIdx.x; i < width; i += kThreads) dst[i] = (T)(row[i] * inv[i / size] * norm.w[i]);
+}
+
+template <typename T>
+__global__ __launch_bounds__(kThreads) void residual_norm_kernel(const float* x, SublayerOut y, GroupNorm norm_y, DepthAverage depth,
+                                                                float* x_out, GroupNorm norm_h, T* __restrict__ h, int ld_h,
+                                                                int width) {
+    extern __shared__ float smem[];
+    float* v = smem;
+    float* inv = v + width;
+    float* red = inv + max(norm_y.groups, norm_h.groups);
+    const size_t m = blockIdx.x, base = m * width;
+    const int t = threadIdx.x;
+    if (y.y) {
+        const float share = y.slot_rows ? 1.0f / (float)y.top : 0.f;
+        for (int i = t; i < width; i += kThreads) {
+            float s;
+            if (y.slot_rows) {
+                s = 0.f;
+                for (int k = 0; k < y.top; k++) s += y.y[(size_t)y.slot_rows[m * y.top + k] * width + i];
+                s *= share;
+                if (y.shared) s += y.shared[base + i];
+            } else {
+                s = y.y[base + i];
+            }
+            v[i] = s;
+        }
+        __syncthreads();
+        group_inverse_rms<kThreads>([&](int i) { return v[i]; }, width, norm_y.groups, norm_y.eps, inv, red);
+    }
+    const int size_y = width / max(norm_y.groups, 1);
+    for (int i = t; i < width; i += kThreads) {  // every element of v is read and written by the same thread from here on
+        float r = x[base + i];
+        if (y.y) r += v[i] * inv[i / size_y] * norm_y.w[i];
+        if (depth.states) {
+            depth.states[depth.n * depth.state_step + base + i] = r;
+            float s = 0.f;
+            for (int j = 0; j < depth.n; j++) s = fmaf(depth.coef[j], depth.states[j * depth.state_step + base + i], s);
+            r = fmaf(depth.coef[depth.n], r, s);
+        }
+        x_out[base + i] = r;
+        v[i] = r;
+    }
+    __syncthreads();
+    group_inverse_rms<kThreads>([&](int i) { return v[i]; }, width, norm_h.groups, norm_h.eps, inv, red);
+    const int size_h = width / norm_h.groups;
+    T* dst = h + m * ld_h;
+    for (int i = t; i < width; i += kThreads) dst[i] = (T)(v[i] * inv[i / size_h] * norm_h.w[i]);
+}
+
+// Exclusive prefix sum of a[0..n) in place, total returned to every thread; 1024 threads.
+__device__ int block_exclusive_scan(int* a, int n, int* tmp) {
+    const int t = threadIdx.x;
+    int carry = 0;
+    for (int base = 0; base < n; base += 1024) {
+        const int own = base + t < n ? a[base + t] : 0;
+        tmp[t] = own;
+        __syncthreads();
+        for (int off = 1; off < 1024; off <<= 1) {
+            const int add = t >= off ? tmp[t - off] : 0;
+            __syncthreads();
+            tmp[t] += add;
+            __syncthreads();
+        }
+        if (base + t < n) a[base + t] = carry + tmp[t] - own;
+        carry += tmp[1023];
+        __syncthreads();
+    }
+    return carry;
+}
+
+__global__ __launch_bounds__(1024) void table_route_kernel(const int* __restrict__ ids, const int* __restrict__ table, int vocab,
+                                                         int top, int experts, int M, int* __restrict__ src_rows,
+                                                         int* __restrict__ slot_rows, GroupTile* __restrict__ tiles,
+                                                         int* __restrict__ n_tiles) {
+    extern __shared__ int cnt[];  // [experts] counts, [experts] first rows, [experts] first tiles, [1024]
+    int *first = cnt + experts, *tile0 = first + experts, *tmp = tile0 + experts;
+    const int t = threadIdx.x, total = M * top;
+    for (int e = t; e < experts; e += 1024) cnt[e] = 0;
+    __syncthreads();
+    auto expert_of = [&](int i) {
+        const int id = min(max(ids[i / top], 0), vocab - 1);
+        return min(max(table[(size_t)id * top + i % top], 0), experts - 1);
+    };
+    for (int i = t; i < total; i += 1024) atomicAdd(&cnt[expert_of(i)], 1);
+    __syncthreads();
+    for (int e = t; e < experts; e += 1024) {
+        first[e] = cnt[e];
+        tile0[e] = (cnt[e] + kGroupTileRows - 1) / kGroupTileRows;
+    }
+    __syncthreads();
+    block_exclusive_scan(first, experts, tmp);
+    const int all_tiles = block_exclusive_scan(tile0, experts, tmp);
+    if (t == 0) *n_tiles = all_tiles;
+    for (int e = t; e < experts; e += 1024) {
+        const int n = cnt[e];
+        for (int k = 0; k * kGroupTileRows < n; k++)
+            tiles[tile0[e] + k] = GroupTile{e, first[e] + k * kGroupTileRows, min(kGroupTileRows, n - k * kGroupTileRows)};
+    }
+    __syncthreads();
+    // where a token's row lands among its expert's rows does not matter: a row's result does not depend on its place
+    for (int i = t; i < total; i += 1024) {
+        const int r = atomicAdd(&first[expert_of(i)], 1);
+        src_rows[r] = i / top;
+        slot_rows[i] = r;
+    }
+}
+
+}  // namespace
+
+template <typename T>
+hipError_t launch_group_norm(const float* x, int M, int width, const GroupNorm& norm, T* out, int ld_out, hipStream_t s) {
+    const size_t lds = (norm.groups + kThreads / 64) * sizeof(float);
+    hipLaunchKernelGGL(group_norm_kernel<T>, dim3(M), dim3(kThreads), lds, s, x, width, norm, out, ld_out);
+    return hipGetLastError();
+}
+
+template <typename T>
+hipError_t launch_residual_norm(const float* x, const SublayerOut& y, const GroupNorm& norm_y, const DepthAverage& depth, float* x_out,
+                                const GroupNorm& norm_h, T* h, int ld_h, int M, int width, hipStream_t s) {
+    const int groups = norm_y.groups > norm_h.groups ? norm_y.groups : norm_h.groups;
+    const size_t lds = (width + groups + kThreads / 64) * sizeof(float);
+    hipLaunchKernelGGL(residual_norm_kernel<T>, dim3(M), dim3(kThreads), lds, s, x, y, norm_y, depth, x_out, norm_h, h, ld_h, width);
+    return hipGetLastError();
+}
+
+hipError_t launch_table_route(const int* ids, const int* table, int vocab, int top, int experts, int M, int* src_rows,
+                              int* slot_rows, GroupTile* tiles, int* n_tiles, hipStream_t s) {
+    const size_t lds = (3 * (size_t)experts + 1024) * sizeof(int);
+    hipLaunchKernelGGL(table_route_kernel, dim3(1), dim3(1024), lds, s, ids, table, vocab, top, experts, M, src_rows, slot_rows,
+                       tiles, n_tiles);
+    return hipGetLastError();
+}
+
+#define INSTANTIATE(T)                                                                                                          \
+    template hipError_t launch_group_norm<T>(const float*, int, int, const GroupNorm&, T*, int, hipStream_t);                     \
+    template hipError_t launch_residual_norm<T>(const float*, const SublayerOut&, const GroupNorm&, const DepthAverage&, float*, \
+                                                const GroupNorm&, T*, int, int, int, hipStream_t);
+INSTANTIATE(bf16)
+INSTANTIATE(float)
+
+}  // namespace a81w41

@@ -13,28 +13,15 @@
 
 #include "../../include/a81w41.h"
 #include "a81w41_kernels.h"
+#include "decoder_session.h"
+#include "json.h"
 
 namespace {
 
-int fail(int status, const char* fmt, ...) {
-    char buf[400];
-    va_list ap;
-    va_start(ap, fmt);
-    vsnprintf(buf, sizeof(buf), fmt, ap);
-    va_end(ap);
-    return a81w41::report_failure(status, buf);
-}
+using a81w41::failf;
 
-#define Q_HIP(expr)                                                                  \
-    do {                                                                             \
-        hipError_t _e = (expr);                                                      \
-        if (_e != hipSuccess) return fail(A81W41_ERR_HIP, "%s: %s", #expr, hipGetErrorString(_e)); \
-    } while (0)
-#define Q_TRY(expr)              \
-    do {                         \
-        int _st = (expr);        \
-        if (_st) return _st;     \
-    } while (0)
+#define Q_HIP A81W41_HIP_TRY
+#define Q_TRY A81W41_TRY
 
 constexpr int kHeadDim = 128;
 
@@ -47,7 +34,7 @@ struct LayerWeights {
 
 }  // namespace
 
-struct a81w41_qwen3 {
+struct a81w41_qwen3 : a81w41_model {
     a81w41_qwen3_config cfg{};
     a81w41_context* ctx = nullptr;
     std::vector<LayerWeights> layers;
@@ -57,15 +44,9 @@ struct a81w41_qwen3 {
     float *cos_t = nullptr, *sin_t = nullptr;
     // activations, sized for max_seq rows
     float *x = nullptr, *x2 = nullptr, *h = nullptr, *qkv = nullptr, *attn = nullptr, *o = nullptr, *gate_up = nullptr, *act = nullptr;
-    float* logits = nullptr;
-    int *ids = nullptr, *pos = nullptr, *step = nullptr, *history = nullptr;
-    int history_len = 0;
-    int host_pos = 0;
-    int plan_ctx = 0;              // longest context the passes being enqueued will see (picks the attention's key split)
     float* attn_part = nullptr;    // split attention: n_q * kAttentionMaxSplits * 132 floats
     unsigned* attn_arrive = nullptr;  // ... and n_q arrival counters, zero between launches
     float attn_scale = 0.f;  // 1/sqrt(128) unless a scaling.bin said otherwise
-    hipStream_t stream = nullptr;
     int cu_count = 0;  // of the device the model lives on
     // Switches of a81w41_qwen3_set_option: each keeps a fusion off (or fixes the attention's key split) so
     // that tests can compare the fused pass with the separate kernels bit for bit.
@@ -73,6 +54,15 @@ struct a81w41_qwen3 {
     unsigned opt_spin_limit = 0;  // 0: the chain's default
     int opt_attention_split = 0;
     int qkv_dim() const { return (cfg.n_q_heads + 2 * cfg.n_kv_heads) * kHeadDim; }
+
+    ~a81w41_qwen3() override;
+    int create();  // buffers and cache of cfg
+    size_t weight_bytes() const override;
+
+   protected:
+    int ready() const override;
+    int enqueue_pass(int M, const int* want, int n_want, hipStream_t s) override;
+    int check_passes() override;
 };
 
 namespace {
@@ -85,7 +75,7 @@ int linear_dims(const a81w41_qwen3* m, int layer, int which, int& N, int& K) {
         return 0;
     }
     if (layer < 0 || layer >= c.n_layers || which < 0 || which > 3)
-        return fail(A81W41_ERR_INVALID_ARG, "no linear %d in layer %d", which, layer);
+        return failf(A81W41_ERR_INVALID_ARG, "no linear %d in layer %d", which, layer);
     switch (which) {
         case 0: N = m->qkv_dim(); K = c.hidden; break;
         case 1: N = c.hidden; K = c.n_q_heads * kHeadDim; break;
@@ -99,27 +89,34 @@ a81w41_linear** linear_slot(a81w41_qwen3* m, int layer, int which) {
     return layer == -1 ? &m->lm_head : &m->layers[layer].lin[which];
 }
 
-int ready(const a81w41_qwen3* m) {
-    if (!m->lm_head || !m->final_norm || !m->embedding) return fail(A81W41_ERR_INVALID_ARG, "lm_head, final norm or embedding not set");
+}  // namespace
+
+int a81w41_qwen3::ready() const {
+    const a81w41_qwen3* m = this;
+    if (!m->lm_head || !m->final_norm || !m->embedding) return failf(A81W41_ERR_INVALID_ARG, "lm_head, final norm or embedding not set");
     for (size_t l = 0; l < m->layers.size(); l++)
         for (int w = 0; w < 4; w++)
             if (!m->layers[l].lin[w] || !m->layers[l].norm[w])
-                return fail(A81W41_ERR_INVALID_ARG, "layer %zu: linear or norm %d not set", l, w);
+                return failf(A81W41_ERR_INVALID_ARG, "layer %zu: linear or norm %d not set", l, w);
     return 0;
 }
 
-// One pass over M new tokens whose ids are in m->ids; leaves the last token's logits in
-// m->logits and advances the device position by M.  Enqueues only.
+namespace {
 int enqueue_pass_one_token(a81w41_qwen3* m, hipStream_t s);
 bool one_token_pass_usable(const a81w41_qwen3* m);
 bool prefill_fusion_usable(const a81w41_qwen3* m);
 
-int enqueue_pass(a81w41_qwen3* m, int M, hipStream_t s) {
+}  // namespace
+
+// One pass over M new tokens whose ids are in m->ids; leaves the wanted tokens' logits in
+// m->logits and advances the device position by M.  Enqueues only.
+int a81w41_qwen3::enqueue_pass(int M, const int* want, int n_want, hipStream_t s) {
+    a81w41_qwen3* m = this;
     if (M == 1 && one_token_pass_usable(m)) return enqueue_pass_one_token(m, s);
     const a81w41_qwen3_config& c = m->cfg;
     const int qkv_dim = m->qkv_dim(), q_dim = c.n_q_heads * kHeadDim;
     const float scale = m->attn_scale;  // scaling.bin, QwenAttention.cc:44-46
-    Q_HIP(a81w41::launch_embed_rows(m->ids, m->embedding, m->x, M, c.hidden, c.vocab, s));
+    Q_HIP(a81w41::launch_embed_rows(m->ids, m->embedding, a81w41::TableType::kFp16, c.hidden, m->x, M, c.hidden, c.vocab, s));
     const float* pending = nullptr;  // output of the previous sub-block, not yet added to the residual stream x
     // Several rows: the norms and SiLU*mul write the quantised blocks of their result straight into the
     // context's scratch, and the matrix-core contraction reads them from there -- the same blocks the
@@ -175,11 +172,14 @@ int enqueue_pass(a81w41_qwen3* m, int M, hipStream_t s) {
     }
     Q_HIP(a81w41::launch_add_rmsnorm(pending ? pending : m->x, pending ? m->x : nullptr, m->final_norm, m->x, m->h, M,
                                      c.hidden, c.rms_eps, s));
-    // lm_head on the last token only (QwenForCausalLM.cc:43-46)
-    Q_TRY(a81w41_linear_forward(m->lm_head, m->h + (size_t)(M - 1) * c.hidden, 1, m->logits, s));
+    // lm_head on the wanted tokens only: in generation the last one (QwenForCausalLM.cc:43-46)
+    for (int i = 0; i < n_want; i++)
+        Q_TRY(a81w41_linear_forward(m->lm_head, m->h + (size_t)want[i] * c.hidden, 1, m->logits + (size_t)i * c.vocab, s));
     Q_HIP(a81w41::launch_advance(m->pos, M, s));
     return 0;
 }
+
+namespace {
 
 // The same pass for one token with the elementwise work folded into the neighbouring kernels, five
 // launches per layer: every add + RMSNorm runs inside the GEMV that consumes it (qkv, gate_up,
@@ -221,7 +221,7 @@ int enqueue_pass_one_token(a81w41_qwen3* m, hipStream_t s) {
     if (splits > fit) splits = fit;
     if (env_split > 0) splits = env_split;
     splits = splits < 1 ? 1 : (splits > a81w41::kAttentionMaxSplits ? a81w41::kAttentionMaxSplits : splits);
-    Q_HIP(a81w41::launch_embed_rows(m->ids, m->embedding, m->o, 1, c.hidden, c.vocab, s));  // pending = the embedding
+    Q_HIP(a81w41::launch_embed_rows(m->ids, m->embedding, a81w41::TableType::kFp16, c.hidden, m->o, 1, c.hidden, c.vocab, s));  // pending = the embedding
     // The linears and the attention of the pass are one dependent chain (QwenDecoderLayer.cc:39-105).  As links of
     // an overlapping chain each of them starts while its predecessor runs and requests its first weight blocks
     // (or cache rows) before it waits for it; same kernels' arithmetic, same bits.
@@ -347,16 +347,21 @@ bool one_token_pass_usable(const a81w41_qwen3* m) {
 }
 
 // After a synchronisation: did an in-kernel wait of a chained pass give up?  (Clears the condition.)
-int check_chain(a81w41_qwen3* m) {
+}  // namespace
+
+int a81w41_qwen3::check_passes() {
+    a81w41_qwen3* m = this;
     a81w41::ChainState* chain = a81w41::context_chain(m->ctx);
     if (!chain || chain->open) return 0;
     bool gave_up = false;
     Q_HIP(a81w41::chain_status(chain, &gave_up));
     if (gave_up)
-        return fail(A81W41_ERR_HIP, "a wait inside the chained one-token pass gave up: the results of that pass are invalid "
+        return failf(A81W41_ERR_HIP, "a wait inside the chained one-token pass gave up: the results of that pass are invalid "
                                     "(is the GPU shared with other work?)");
     return 0;
 }
+
+namespace {
 
 template <typename T>
 int dev_alloc(T** p, size_t count) {
@@ -369,24 +374,34 @@ int dev_alloc(T** p, size_t count) {
 extern "C" {
 
 int a81w41_qwen3_create(const a81w41_qwen3_config* cfg, a81w41_qwen3** out) {
-    if (!cfg || !out) return fail(A81W41_ERR_INVALID_ARG, "null argument");
+    if (!cfg || !out) return failf(A81W41_ERR_INVALID_ARG, "null argument");
     *out = nullptr;
     const a81w41_qwen3_config& c = *cfg;
     if (c.n_layers < 1 || c.n_q_heads < 1 || c.n_kv_heads < 1 || c.n_q_heads % c.n_kv_heads || c.hidden < 64 ||
         c.hidden % 64 || c.intermediate < 64 || c.intermediate % 64 || c.vocab < 8 || c.vocab % 8 || c.max_seq < 1 ||
         c.max_seq > 8192 || !(c.rope_theta > 0.f) || !(c.rms_eps >= 0.f))
-        return fail(A81W41_ERR_INVALID_ARG, "bad model configuration (hidden, intermediate multiples of 64; vocab of 8; "
+        return failf(A81W41_ERR_INVALID_ARG, "bad model configuration (hidden, intermediate multiples of 64; vocab of 8; "
                                             "max_seq <= 8192; n_q_heads a multiple of n_kv_heads)");
-    // on any failure below the half-built model is torn down by its regular destructor
-    std::unique_ptr<a81w41_qwen3, void (*)(a81w41_qwen3*)> m(new (std::nothrow) a81w41_qwen3, a81w41_qwen3_destroy);
-    if (!m) return fail(A81W41_ERR_HIP, "out of host memory");
+    // on any failure below the half-built model is torn down by its destructor
+    std::unique_ptr<a81w41_qwen3> m(new (std::nothrow) a81w41_qwen3);
+    if (!m) return failf(A81W41_ERR_HIP, "out of host memory");
     m->cfg = c;
+    Q_TRY(m->create());
+    *out = m.release();
+    return A81W41_OK;
+}
+
+}  // extern "C"
+
+int a81w41_qwen3::create() {
+    a81w41_qwen3* m = this;
+    const a81w41_qwen3_config& c = cfg;
     m->attn_scale = 1.0f / std::sqrt((float)kHeadDim);
     {
         int dev = 0;
         Q_HIP(hipGetDevice(&dev));
         Q_HIP(hipDeviceGetAttribute(&m->cu_count, hipDeviceAttributeMultiprocessorCount, dev));
-        if (m->cu_count < 1) return fail(A81W41_ERR_HIP, "device reports no compute units");
+        if (m->cu_count < 1) return failf(A81W41_ERR_HIP, "device reports no compute units");
     }
     const int max_cols = c.hidden > c.intermediate ? c.hidden : c.intermediate;
     const int q_dim = c.n_q_heads * kHeadDim;
@@ -394,10 +409,8 @@ int a81w41_qwen3_create(const a81w41_qwen3_config* cfg, a81w41_qwen3** out) {
     m->layers.resize(c.n_layers);
     const size_t cache_elems = (size_t)c.n_kv_heads * c.max_seq * kHeadDim;
     for (auto& L : m->layers) {
-        Q_HIP(hipMalloc(&L.k_cache, cache_elems * 2));
-        Q_HIP(hipMalloc(&L.v_cache, cache_elems * 2));
-        Q_HIP(hipMemset(L.k_cache, 0, cache_elems * 2));
-        Q_HIP(hipMemset(L.v_cache, 0, cache_elems * 2));
+        Q_TRY(m->cache.add(cache_elems * 2, &L.k_cache));
+        Q_TRY(m->cache.add(cache_elems * 2, &L.v_cache));
     }
     const size_t rows = c.max_seq;
     Q_TRY(dev_alloc(&m->x, rows * c.hidden));
@@ -408,18 +421,10 @@ int a81w41_qwen3_create(const a81w41_qwen3_config* cfg, a81w41_qwen3** out) {
     Q_TRY(dev_alloc(&m->o, rows * c.hidden));
     Q_TRY(dev_alloc(&m->gate_up, rows * 2 * c.intermediate));
     Q_TRY(dev_alloc(&m->act, rows * c.intermediate));
-    Q_TRY(dev_alloc(&m->logits, (size_t)c.vocab));
+    Q_TRY(m->init_session(c.max_seq, c.vocab, c.max_seq));
     Q_TRY(dev_alloc(&m->attn_part, (size_t)c.n_q_heads * a81w41::kAttentionMaxSplits * 132));
     Q_TRY(dev_alloc(&m->attn_arrive, (size_t)c.n_q_heads));
     Q_HIP(hipMemset(m->attn_arrive, 0, (size_t)c.n_q_heads * sizeof(unsigned)));
-    Q_TRY(dev_alloc(&m->ids, rows));
-    Q_TRY(dev_alloc(&m->pos, 1));
-    Q_TRY(dev_alloc(&m->step, 1));
-    m->history_len = 8192;
-    Q_TRY(dev_alloc(&m->history, (size_t)m->history_len));
-    Q_HIP(hipMemset(m->pos, 0, sizeof(int)));
-    Q_HIP(hipMemset(m->step, 0, sizeof(int)));
-    Q_HIP(hipMemset(m->ids, 0, rows * sizeof(int)));
     // rotate-half tables: angle(pos, j) = pos * theta^(-2 (j mod 64) / 128), both halves alike
     std::vector<float> cs((size_t)c.max_seq * kHeadDim), sn(cs.size());
     for (int p = 0; p < c.max_seq; p++)
@@ -433,34 +438,32 @@ int a81w41_qwen3_create(const a81w41_qwen3_config* cfg, a81w41_qwen3** out) {
     Q_TRY(dev_alloc(&m->sin_t, sn.size()));
     Q_HIP(hipMemcpy(m->cos_t, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
     Q_HIP(hipMemcpy(m->sin_t, sn.data(), sn.size() * 4, hipMemcpyHostToDevice));
-    Q_HIP(hipStreamCreate(&m->stream));
-    *out = m.release();
     return A81W41_OK;
 }
 
-void a81w41_qwen3_destroy(a81w41_qwen3* m) {
-    if (!m) return;
+a81w41_qwen3::~a81w41_qwen3() {
+    a81w41_qwen3* m = this;
     if (m->stream) (void)hipStreamSynchronize(m->stream);
     for (auto& L : m->layers) {
         for (int w = 0; w < 4; w++) {
             a81w41_linear_destroy(L.lin[w]);
             (void)hipFree(L.norm[w]);
         }
-        (void)hipFree(L.k_cache);
-        (void)hipFree(L.v_cache);
     }
     a81w41_linear_destroy(m->lm_head);
     void* bufs[] = {m->final_norm, m->embedding, m->cos_t, m->sin_t, m->x, m->x2, m->h, m->qkv, m->attn, m->o,
-                    m->gate_up, m->act, m->logits, m->ids, m->pos, m->step, m->history, m->attn_part, m->attn_arrive};
+                    m->gate_up, m->act, m->attn_part, m->attn_arrive};
     for (void* b : bufs) (void)hipFree(b);
-    if (m->stream) (void)hipStreamDestroy(m->stream);
     a81w41_context_destroy(m->ctx);
-    delete m;
 }
+
+extern "C" {
+
+void a81w41_qwen3_destroy(a81w41_qwen3* m) { delete m; }
 
 int a81w41_qwen3_set_linear(a81w41_qwen3* m, int layer, int which, const uint8_t* weight_int4, const float* scale,
                             const float* offset) {
-    if (!m) return fail(A81W41_ERR_INVALID_ARG, "null model");
+    if (!m) return failf(A81W41_ERR_INVALID_ARG, "null model");
     int N, K;
     Q_TRY(linear_dims(m, layer, which, N, K));
     a81w41_linear** slot = linear_slot(m, layer, which);
@@ -472,7 +475,7 @@ int a81w41_qwen3_set_linear(a81w41_qwen3* m, int layer, int which, const uint8_t
 }
 
 int a81w41_qwen3_set_linear_blobs(a81w41_qwen3* m, int layer, int which, const void* blob_fp16, const void* blob_fp32) {
-    if (!m) return fail(A81W41_ERR_INVALID_ARG, "null model");
+    if (!m) return failf(A81W41_ERR_INVALID_ARG, "null model");
     int N, K;
     Q_TRY(linear_dims(m, layer, which, N, K));
     a81w41_linear** slot = linear_slot(m, layer, which);
@@ -484,7 +487,7 @@ int a81w41_qwen3_set_linear_blobs(a81w41_qwen3* m, int layer, int which, const v
 }
 
 int a81w41_qwen3_set_norm(a81w41_qwen3* m, int layer, int which, const float* weight) {
-    if (!m || !weight) return fail(A81W41_ERR_INVALID_ARG, "null argument");
+    if (!m || !weight) return failf(A81W41_ERR_INVALID_ARG, "null argument");
     float** slot;
     size_t n;
     if (layer == -1) {
@@ -492,7 +495,7 @@ int a81w41_qwen3_set_norm(a81w41_qwen3* m, int layer, int which, const float* we
         n = m->cfg.hidden;
     } else {
         if (layer < 0 || layer >= m->cfg.n_layers || which < 0 || which > 3)
-            return fail(A81W41_ERR_INVALID_ARG, "no norm %d in layer %d", which, layer);
+            return failf(A81W41_ERR_INVALID_ARG, "no norm %d in layer %d", which, layer);
         slot = &m->layers[layer].norm[which];
         n = which < 2 ? (size_t)m->cfg.hidden : (size_t)kHeadDim;
     }
@@ -502,7 +505,7 @@ int a81w41_qwen3_set_norm(a81w41_qwen3* m, int layer, int which, const float* we
 }
 
 int a81w41_qwen3_set_embedding(a81w41_qwen3* m, const uint16_t* table_fp16) {
-    if (!m || !table_fp16) return fail(A81W41_ERR_INVALID_ARG, "null argument");
+    if (!m || !table_fp16) return failf(A81W41_ERR_INVALID_ARG, "null argument");
     const size_t bytes = (size_t)m->cfg.vocab * m->cfg.hidden * 2;
     if (!m->embedding) Q_HIP(hipMalloc(&m->embedding, bytes));
     Q_HIP(hipMemcpy(m->embedding, table_fp16, bytes, hipMemcpyHostToDevice));
@@ -510,7 +513,7 @@ int a81w41_qwen3_set_embedding(a81w41_qwen3* m, const uint16_t* table_fp16) {
 }
 
 int a81w41_qwen3_set_option(a81w41_qwen3* m, int option, int value) {
-    if (!m) return fail(A81W41_ERR_INVALID_ARG, "null model");
+    if (!m) return failf(A81W41_ERR_INVALID_ARG, "null model");
     switch (option) {
         case A81W41_QWEN3_OPT_UNFUSED: m->opt_unfused = value != 0; break;
         case A81W41_QWEN3_OPT_ATTN_FP32: m->opt_attn_fp32 = value != 0; break;
@@ -518,18 +521,28 @@ int a81w41_qwen3_set_option(a81w41_qwen3* m, int option, int value) {
         case A81W41_QWEN3_OPT_VECTOR_ATTENTION: m->opt_vector_attention = value != 0; break;
         case A81W41_QWEN3_OPT_CHAIN: m->opt_chain = value != 0; break;
         case A81W41_QWEN3_OPT_CHAIN_SPIN_LIMIT:
-            if (value < 0) return fail(A81W41_ERR_INVALID_ARG, "spin limit must be >= 0 (0: default)");
+            if (value < 0) return failf(A81W41_ERR_INVALID_ARG, "spin limit must be >= 0 (0: default)");
             m->opt_spin_limit = (unsigned)value;
             break;
         case A81W41_QWEN3_OPT_ATTENTION_SPLIT:
             if (value < 0 || value > a81w41::kAttentionMaxSplits)
-                return fail(A81W41_ERR_INVALID_ARG, "attention split must be 0 (automatic) .. %d", a81w41::kAttentionMaxSplits);
+                return failf(A81W41_ERR_INVALID_ARG, "attention split must be 0 (automatic) .. %d", a81w41::kAttentionMaxSplits);
             m->opt_attention_split = value;
             break;
-        default: return fail(A81W41_ERR_INVALID_ARG, "unknown option %d", option);
+        default: return failf(A81W41_ERR_INVALID_ARG, "unknown option %d", option);
     }
     return A81W41_OK;
 }
+
+}  // extern "C"
+
+size_t a81w41_qwen3::weight_bytes() const {
+    size_t lin = 0, other = 0;
+    a81w41_qwen3_resident_bytes(this, &lin, &other, nullptr, nullptr);
+    return lin + other;
+}
+
+extern "C" {
 
 size_t a81w41_qwen3_resident_bytes(const a81w41_qwen3* m, size_t* linear_weights, size_t* other_weights, size_t* kv_cache,
                                    size_t* buffers) {
@@ -561,13 +574,13 @@ size_t a81w41_qwen3_resident_bytes(const a81w41_qwen3* m, size_t* linear_weights
 }
 
 int a81w41_qwen3_chain_status(a81w41_qwen3* m, int* gave_up) {
-    if (!m || !gave_up) return fail(A81W41_ERR_INVALID_ARG, "null argument");
+    if (!m || !gave_up) return failf(A81W41_ERR_INVALID_ARG, "null argument");
     Q_HIP(hipStreamSynchronize(m->stream));
     return a81w41_context_chain_status(m->ctx, gave_up);
 }
 
 int a81w41_qwen3_read_buffer(a81w41_qwen3* m, int which, float* host_out, size_t count) {
-    if (!m || !host_out) return fail(A81W41_ERR_INVALID_ARG, "null argument");
+    if (!m || !host_out) return failf(A81W41_ERR_INVALID_ARG, "null argument");
     const a81w41_qwen3_config& c = m->cfg;
     const size_t rows = c.max_seq;
     const float* src = nullptr;
@@ -581,53 +594,40 @@ int a81w41_qwen3_read_buffer(a81w41_qwen3* m, int which, float* host_out, size_t
         case A81W41_QWEN3_BUF_GATE_UP: src = m->gate_up; have = rows * 2 * c.intermediate; break;
         case A81W41_QWEN3_BUF_ACT: src = m->act; have = rows * c.intermediate; break;
         case A81W41_QWEN3_BUF_LOGITS: src = m->logits; have = c.vocab; break;
-        default: return fail(A81W41_ERR_INVALID_ARG, "unknown buffer %d", which);
+        default: return failf(A81W41_ERR_INVALID_ARG, "unknown buffer %d", which);
     }
-    if (count > have) return fail(A81W41_ERR_INVALID_ARG, "buffer %d holds %zu floats, %zu asked for", which, have, count);
+    if (count > have) return failf(A81W41_ERR_INVALID_ARG, "buffer %d holds %zu floats, %zu asked for", which, have, count);
     Q_HIP(hipStreamSynchronize(m->stream));
     Q_HIP(hipMemcpy(host_out, src, count * sizeof(float), hipMemcpyDeviceToHost));
     return A81W41_OK;
 }
 
 int a81w41_qwen3_reset(a81w41_qwen3* m) {
-    if (!m) return fail(A81W41_ERR_INVALID_ARG, "null model");
-    Q_HIP(hipStreamSynchronize(m->stream));
-    Q_HIP(hipMemset(m->pos, 0, sizeof(int)));
-    Q_HIP(hipMemset(m->step, 0, sizeof(int)));
-    m->host_pos = 0;
-    return A81W41_OK;
+    if (!m) return failf(A81W41_ERR_INVALID_ARG, "null model");
+    return m->reset();
 }
 
 int a81w41_qwen3_forward(a81w41_qwen3* m, const int* token_ids, int n_tokens, float* logits_host) {
-    if (!m || !token_ids) return fail(A81W41_ERR_INVALID_ARG, "null argument");
-    Q_TRY(ready(m));
-    if (n_tokens < 1 || m->host_pos + n_tokens > m->cfg.max_seq)
-        return fail(A81W41_ERR_INVALID_ARG, "%d tokens on top of %d do not fit max_seq %d", n_tokens, m->host_pos, m->cfg.max_seq);
-    Q_HIP(hipMemcpy(m->ids, token_ids, (size_t)n_tokens * sizeof(int), hipMemcpyHostToDevice));
-    m->plan_ctx = m->host_pos + n_tokens;
-    Q_TRY(enqueue_pass(m, n_tokens, m->stream));
-    Q_HIP(hipStreamSynchronize(m->stream));
-    m->host_pos += n_tokens;
-    Q_TRY(check_chain(m));
-    if (logits_host) Q_HIP(hipMemcpy(logits_host, m->logits, (size_t)m->cfg.vocab * 4, hipMemcpyDeviceToHost));
-    return A81W41_OK;
+    if (!m || !token_ids) return failf(A81W41_ERR_INVALID_ARG, "null argument");
+    const int last = n_tokens - 1;
+    return m->forward(token_ids, n_tokens, &last, n_tokens > 0 ? 1 : 0, logits_host);
 }
 
 int a81w41_qwen3_attention(const float* q_dev, int q_row_stride, const void* k_cache_dev, const void* v_cache_dev,
                            const int* pos_dev, float* out_dev, int out_row_stride, int M, int n_q, int n_kv, int max_seq,
                            float scale, int variant, void* stream) {
-    if (!q_dev || !k_cache_dev || !v_cache_dev || !pos_dev || !out_dev) return fail(A81W41_ERR_INVALID_ARG, "null argument");
+    if (!q_dev || !k_cache_dev || !v_cache_dev || !pos_dev || !out_dev) return failf(A81W41_ERR_INVALID_ARG, "null argument");
     if (M < 1 || n_kv < 1 || n_q < n_kv || n_q % n_kv || max_seq < 1 || max_seq > 8192 || q_row_stride < n_q * kHeadDim ||
         out_row_stride < n_q * kHeadDim || q_row_stride % 4 || out_row_stride % 4 || variant < 0 || variant > 6)
-        return fail(A81W41_ERR_INVALID_ARG, "bad attention shape");
+        return failf(A81W41_ERR_INVALID_ARG, "bad attention shape");
     if ((reinterpret_cast<uintptr_t>(q_dev) | reinterpret_cast<uintptr_t>(out_dev) | reinterpret_cast<uintptr_t>(k_cache_dev) |
          reinterpret_cast<uintptr_t>(v_cache_dev)) & 15)
-        return fail(A81W41_ERR_INVALID_ARG, "attention buffers must be 16-byte aligned");
+        return failf(A81W41_ERR_INVALID_ARG, "attention buffers must be 16-byte aligned");
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (variant >= 2) {
         const int heads = variant == 2 ? 0 : 1 << (variant - 3);  // 3..6: 1, 2, 4, 8 heads per workgroup
         if (!a81w41::attention_prefill_fits(M, n_q, n_kv) || (heads && (n_q / n_kv) % heads))
-            return fail(A81W41_ERR_INVALID_ARG,
+            return failf(A81W41_ERR_INVALID_ARG,
                         "the matrix-core attention needs M > 8, n_q / n_kv in {1, 2, 4, 8} and a divisor of it as heads per workgroup");
         Q_HIP(a81w41::launch_attention_prefill(q_dev, q_row_stride, k_cache_dev, v_cache_dev, pos_dev, out_dev, out_row_stride, M,
                                                n_q, n_kv, max_seq, scale, s, nullptr, heads));
@@ -643,10 +643,10 @@ int a81w41_qwen3_attention_one_token(const float* qkv_dev, int n_q, int n_kv, co
                                      void* v_cache_dev, float* out_dev, int max_seq, float eps, float scale, int splits,
                                      void* stream) {
     if (!qkv_dev || !q_w_dev || !k_w_dev || !cos_dev || !sin_dev || !pos_dev || !k_cache_dev || !v_cache_dev || !out_dev)
-        return fail(A81W41_ERR_INVALID_ARG, "null argument");
+        return failf(A81W41_ERR_INVALID_ARG, "null argument");
     if (n_kv < 1 || n_q < n_kv || n_q % n_kv || max_seq < 1 || max_seq > 8192 || splits < 1 ||
         splits > a81w41::kAttentionMaxSplits)
-        return fail(A81W41_ERR_INVALID_ARG, "bad attention shape");
+        return failf(A81W41_ERR_INVALID_ARG, "bad attention shape");
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (splits == 1) {
         Q_HIP(a81w41::launch_attention_one_token(qkv_dev, n_q, n_kv, q_w_dev, k_w_dev, cos_dev, sin_dev, pos_dev, k_cache_dev,
@@ -670,76 +670,8 @@ int a81w41_qwen3_attention_one_token(const float* qkv_dev, int n_q, int n_kv, co
 
 int a81w41_qwen3_generate_greedy(a81w41_qwen3* m, const int* prompt, int n_prompt, int n_new, int* out_tokens,
                                  double* prefill_ms, double* decode_ms) {
-    if (!m || !prompt || !out_tokens) return fail(A81W41_ERR_INVALID_ARG, "null argument");
-    Q_TRY(ready(m));
-    if (n_prompt < 1 || n_new < 1 || n_new > m->history_len || m->host_pos + n_prompt + n_new - 1 > m->cfg.max_seq)
-        return fail(A81W41_ERR_INVALID_ARG, "prompt of %d and %d new tokens on top of %d do not fit max_seq %d", n_prompt,
-                    n_new, m->host_pos, m->cfg.max_seq);
-    hipStream_t s = m->stream;
-    // events and graph objects are released on every way out of this function
-    struct Scoped {
-        hipEvent_t ev[4] = {nullptr, nullptr, nullptr, nullptr};
-        hipGraph_t graph = nullptr;
-        hipGraphExec_t exec = nullptr;
-        ~Scoped() {
-            for (hipEvent_t e : ev)
-                if (e) (void)hipEventDestroy(e);
-            if (exec) (void)hipGraphExecDestroy(exec);
-            if (graph) (void)hipGraphDestroy(graph);
-        }
-    } own;
-    for (hipEvent_t& e : own.ev) Q_HIP(hipEventCreate(&e));
-    const hipEvent_t e0 = own.ev[0], e1 = own.ev[1], e2 = own.ev[2], e3 = own.ev[3];
-    Q_HIP(hipMemcpy(m->ids, prompt, (size_t)n_prompt * sizeof(int), hipMemcpyHostToDevice));
-    Q_HIP(hipMemset(m->step, 0, sizeof(int)));
-    Q_HIP(hipEventRecord(e0, s));
-    m->plan_ctx = m->host_pos + n_prompt + n_new - 1;  // also what the decode steps captured below will reach
-    Q_TRY(enqueue_pass(m, n_prompt, s));
-    // first new token: argmax of the prompt's logits; it becomes the next pass's input id
-    Q_HIP(a81w41::launch_argmax_token(m->logits, m->cfg.vocab, m->ids, m->history, m->history_len, m->step, s));
-    Q_HIP(hipEventRecord(e1, s));
-    Q_HIP(hipStreamSynchronize(s));
-    m->host_pos += n_prompt;
-
-    const int n_steps = n_new - 1;
-    if (n_steps > 0) {
-        // one decode step = a pass over the single id in ids[0] + argmax; captured once, replayed
-        hipGraph_t& graph = own.graph;
-        hipGraphExec_t& exec = own.exec;
-        bool captured = false;
-        if (hipStreamBeginCapture(s, hipStreamCaptureModeThreadLocal) == hipSuccess) {
-            int st = enqueue_pass(m, 1, s);
-            if (st == 0 && a81w41::launch_argmax_token(m->logits, m->cfg.vocab, m->ids, m->history, m->history_len, m->step, s) != hipSuccess)
-                st = 1;
-            const hipError_t ee = hipStreamEndCapture(s, &graph);
-            if (st == 0 && ee == hipSuccess && graph && hipGraphInstantiate(&exec, graph, nullptr, nullptr, 0) == hipSuccess)
-                captured = true;
-        }
-        (void)hipGetLastError();
-        Q_HIP(hipEventRecord(e3, s));
-        for (int i = 0; i < n_steps; i++) {
-            if (captured) {
-                Q_HIP(hipGraphLaunch(exec, s));
-            } else {
-                Q_TRY(enqueue_pass(m, 1, s));
-                Q_HIP(a81w41::launch_argmax_token(m->logits, m->cfg.vocab, m->ids, m->history, m->history_len, m->step, s));
-            }
-        }
-        Q_HIP(hipEventRecord(e2, s));
-        Q_HIP(hipStreamSynchronize(s));
-        m->host_pos += n_steps;
-    } else {
-        Q_HIP(hipEventRecord(e2, s));
-        Q_HIP(hipStreamSynchronize(s));
-    }
-    float ms01 = 0.f, ms12 = 0.f;
-    Q_HIP(hipEventElapsedTime(&ms01, e0, e1));
-    if (n_steps > 0) Q_HIP(hipEventElapsedTime(&ms12, e3, e2));
-    if (prefill_ms) *prefill_ms = ms01;
-    if (decode_ms) *decode_ms = ms12;
-    Q_TRY(check_chain(m));
-    Q_HIP(hipMemcpy(out_tokens, m->history, (size_t)n_new * sizeof(int), hipMemcpyDeviceToHost));
-    return A81W41_OK;
+    if (!m) return failf(A81W41_ERR_INVALID_ARG, "null argument");
+    return m->generate_greedy(prompt, n_prompt, n_new, out_tokens, prefill_ms, decode_ms);
 }
 
 }  // extern "C"
@@ -748,10 +680,10 @@ namespace {
 
 int read_exact(const std::string& name, void* dst, size_t bytes) {
     FILE* f = fopen(name.c_str(), "rb");
-    if (!f) return fail(A81W41_ERR_IO, "cannot open %s", name.c_str());
+    if (!f) return failf(A81W41_ERR_IO, "cannot open %s", name.c_str());
     const size_t got = fread(dst, 1, bytes, f);
     fclose(f);
-    if (got != bytes) return fail(A81W41_ERR_IO, "%s: expected %zu bytes, read %zu", name.c_str(), bytes, got);
+    if (got != bytes) return failf(A81W41_ERR_IO, "%s: expected %zu bytes, read %zu", name.c_str(), bytes, got);
     return A81W41_OK;
 }
 
@@ -847,7 +779,7 @@ int load_into(a81w41_qwen3* m, const std::string& root) {
 }  // namespace
 
 extern "C" int a81w41_qwen3_load(const char* root, const a81w41_qwen3_config* cfg, a81w41_qwen3** out) {
-    if (!root || !out) return fail(A81W41_ERR_INVALID_ARG, "null argument");
+    if (!root || !out) return failf(A81W41_ERR_INVALID_ARG, "null argument");
     *out = nullptr;
     a81w41_qwen3* m = nullptr;
     Q_TRY(a81w41_qwen3_create(cfg, &m));
@@ -859,3 +791,30 @@ extern "C" int a81w41_qwen3_load(const char* root, const a81w41_qwen3_config* cf
     *out = m;
     return A81W41_OK;
 }
+
+namespace {
+
+// Qwen3 through the registry: the reference's weight tree with a config.json of the sizes beside it.
+int load_registered(const a81w41::LoadRequest& req, a81w41_model** out) {
+    if (req.dtype != "bfloat16")
+        return failf(A81W41_ERR_UNSUPPORTED, "Qwen3 runs on its quantised weights only (served under the name bfloat16)");
+    if (req.random_weights) return failf(A81W41_ERR_UNSUPPORTED, "Qwen3 has no random weights of its own");
+    const a81w41::Json& j = *req.config;
+    a81w41_qwen3_config c{};
+    c.n_layers = j.size("num_hidden_layers");
+    c.hidden = j.size("hidden_size");
+    c.n_q_heads = j.size("num_attention_heads");
+    c.n_kv_heads = j.size("num_key_value_heads");
+    c.intermediate = j.size("intermediate_size");
+    c.vocab = j.size("vocab_size");
+    c.max_seq = req.max_seq;
+    c.rope_theta = (float)j.at("rope_theta").number();
+    c.rms_eps = (float)j.at("rms_norm_eps").number();
+    a81w41_qwen3* m = nullptr;
+    Q_TRY(a81w41_qwen3_load(req.dir.c_str(), &c, &m));
+    *out = m;
+    return A81W41_OK;
+}
+const a81w41::RegisterModel registered("Qwen3", load_registered);
+
+}  // namespace

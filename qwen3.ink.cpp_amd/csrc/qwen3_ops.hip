@@ -5,7 +5,6 @@
 // replayed unchanged.  Every index that depends on device data is clamped into its array.
 //
 // What each kernel restates:
-//   embed_rows              Embedding::forward                 src/ops/embedding.cc:13-26
 //   add_rmsnorm             add + Qwen3RMSNorm::forward        QwenOperator.cc:24-53, 715-722
 //   qk_norm_rope_cache      per-head RMSNorm, rotate-half RoPE, KV-cache append
 //                                                            QwenAttention.cc:78-122, ops/RotaryPosEmb.cc:6-78
@@ -15,7 +14,6 @@
 //                           activation quantiser of the linear that consumes the row
 //                           (quantize_row_q8_1_repack_fp32, quantized_gemx_kernels.cc:803-911), so the
 //                           fp32 row never goes to memory; the blocks are bit-identical to quantising it
-//   argmax_token            sample_token_greedy (first maximum)  Pipeline.cc:54-62
 #include "a81w41_kernels.h"
 #include "quantize_common.h"
 
@@ -63,22 +61,6 @@ __device__ __forceinline__ void store_quantized_float4(uint8_t* __restrict__ blo
         float* par = reinterpret_cast<float*>(blk);
         par[h] = qz.d;
         par[2 + h] = qz.ssum;
-    }
-}
-
-__global__ __launch_bounds__(256) void embed_rows_kernel(const int* __restrict__ ids, const __half* __restrict__ table,
-                                                       float* __restrict__ out, int hidden, int vocab) {
-    const int m = blockIdx.x;
-    const int id = min(max(ids[m], 0), vocab - 1);
-    // hidden is a multiple of 64 and the table 16-byte aligned: eight halves per load, two float4 per store
-    const uint4* row = reinterpret_cast<const uint4*>(table + (size_t)id * hidden);
-    float4* dst = reinterpret_cast<float4*>(out + (size_t)m * hidden);
-    for (int j = threadIdx.x; j < (hidden >> 3); j += 256) {
-        const uint4 u = row[j];
-        const __half2* h2 = reinterpret_cast<const __half2*>(&u);
-        const float2 a = __half22float2(h2[0]), b = __half22float2(h2[1]), c = __half22float2(h2[2]), d = __half22float2(h2[3]);
-        dst[2 * j] = make_float4(a.x, a.y, b.x, b.y);
-        dst[2 * j + 1] = make_float4(c.x, c.y, d.x, d.y);
     }
 }
 
@@ -760,70 +742,7 @@ __global__ __launch_bounds__(256) void silu_mul_quant_kernel(const float4* __res
     store_quantized_float4(q_out, i, v);
 }
 
-// First index of the maximum of logits[0..n); written to next_id[0] and to history[*step], then
-// the step counter and the position advance (the token just consumed is now in the cache).
-__global__ __launch_bounds__(1024) void argmax_token_kernel(const float* __restrict__ logits, int n, int* __restrict__ next_id,
-                                                          int* __restrict__ history, int history_len, int* __restrict__ step_dev) {
-    __shared__ float best_v[1024];
-    __shared__ int best_i[1024];
-    const int t = threadIdx.x;
-    float bv = -3.402823466e38f;
-    int bi = 0x7fffffff;
-    // n is a multiple of 8 and logits 16-byte aligned: scan float4s, four in flight
-    const float4* l4 = reinterpret_cast<const float4*>(logits);
-    const int n4 = n >> 2;
-    for (int j0 = t; j0 < n4; j0 += 4 * 1024) {
-        float4 v[4];
-#pragma unroll
-        for (int u = 0; u < 4; u++) {
-            const int j = j0 + u * 1024;
-            v[u] = j < n4 ? l4[j] : make_float4(-3.402823466e38f, -3.402823466e38f, -3.402823466e38f, -3.402823466e38f);
-        }
-#pragma unroll
-        for (int u = 0; u < 4; u++) {
-            const int i = 4 * (j0 + u * 1024);  // indices rise within a thread, so '>' keeps the first maximum
-            const float e[4] = {v[u].x, v[u].y, v[u].z, v[u].w};
-#pragma unroll
-            for (int k = 0; k < 4; k++)
-                if (e[k] > bv) {
-                    bv = e[k];
-                    bi = i + k;
-                }
-        }
-    }
-    best_v[t] = bv;
-    best_i[t] = bi;
-    __syncthreads();
-    for (int s = 512; s > 0; s >>= 1) {
-        if (t < s) {
-            const float ov = best_v[t + s];
-            const int oi = best_i[t + s];
-            if (ov > best_v[t] || (ov == best_v[t] && oi < best_i[t])) {
-                best_v[t] = ov;
-                best_i[t] = oi;
-            }
-        }
-        __syncthreads();
-    }
-    if (t == 0) {
-        const int id = best_i[0] == 0x7fffffff ? 0 : best_i[0];
-        next_id[0] = id;
-        const int st = step_dev[0];
-        if (st >= 0 && st < history_len) history[st] = id;
-        step_dev[0] = st + 1;
-    }
-}
-
-__global__ void advance_kernel(int* __restrict__ pos_dev, int by) {
-    if (threadIdx.x == 0 && blockIdx.x == 0) pos_dev[0] += by;
-}
-
 }  // namespace
-
-hipError_t launch_embed_rows(const int* ids, const void* table_fp16, float* out, int M, int hidden, int vocab, hipStream_t s) {
-    hipLaunchKernelGGL(embed_rows_kernel, dim3(M), dim3(256), 0, s, ids, static_cast<const __half*>(table_fp16), out, hidden, vocab);
-    return hipGetLastError();
-}
 
 hipError_t launch_add_rmsnorm(const float* x, const float* res_in, const float* w, float* res_out, float* norm_out, int M,
                               int hidden, float eps, hipStream_t s) {
@@ -922,17 +841,6 @@ hipError_t launch_silu_mul_quant(const float* gate_up, void* q_out, int M, int i
     const long long total4 = (long long)M * (inter / 4);
     hipLaunchKernelGGL(silu_mul_quant_kernel, dim3((unsigned)((total4 + 255) / 256)), dim3(256), 0, s,
                        reinterpret_cast<const float4*>(gate_up), static_cast<uint8_t*>(q_out), inter / 4, total4);
-    return hipGetLastError();
-}
-
-hipError_t launch_argmax_token(const float* logits, int n, int* next_id, int* history, int history_len, int* step_dev,
-                               hipStream_t s) {
-    hipLaunchKernelGGL(argmax_token_kernel, dim3(1), dim3(1024), 0, s, logits, n, next_id, history, history_len, step_dev);
-    return hipGetLastError();
-}
-
-hipError_t launch_advance(int* pos_dev, int by, hipStream_t s) {
-    hipLaunchKernelGGL(advance_kernel, dim3(1), dim3(64), 0, s, pos_dev, by);
     return hipGetLastError();
 }
 
