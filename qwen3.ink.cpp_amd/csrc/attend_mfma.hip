@@ -1,0 +1,284 @@
+// Causal attention on the matrix cores for bfloat16 rows, in the two forms latent attention needs:
+//   shared    every query row looks at the same key rows, whose first columns are also the values (attention in
+//             latent space: the key rows are the cache itself);
+//   expanded  keys and values of every head were formed beforehand: a key is [own part | part shared by all heads],
+//             values come transposed ([value column][key]).
+//
+// A wave owns 16 (or 2 x 16) query rows.  It forms the scores transposed, S^T = K Q^T (v_mfma_f32_16x16x32_bf16 with
+// the keys as rows), so that lane l holds scores of query l % 16 only: keys 16 t + 4 (l / 16) + i.  These registers
+// are, without any exchange, the B operand of O^T = V^T P^T if lane group l / 16 takes the keys
+// {4 g + i, 16 + 4 g + i} of a 32-key step as its eight k places; V^T is read from LDS in that order.  Running maximum
+// and sum are one value per lane.  Scores, softmax and sums are fp32.
+//
+// A tile of keys is copied global -> LDS by direct 16-byte loads.  Key rows: chunk c of row r at place c ^ (r & 7).
+// Query columns beyond the real width are zero, so whatever finite values sit there in the key rows do not count.
+#include "dense_common.h"
+
+namespace a81w41 {
+namespace {
+
+constexpr float kLog2e = 1.4426950408889634f;
+constexpr float kLowest = -1e30f;
+
+// DK, DV: capacities for key and value columns.  KT keys per tile, NBUF tiles in LDS.
+template <int DK, int DV, int WAVES, int QS, int KT, int NBUF, bool EXPANDED>
+__global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
+    constexpr int CK = DK / 8;                    // 16-byte chunks of a key row
+    constexpr int kKeyBytes = KT * DK * 2, kValueBytes = EXPANDED ? DV * KT * 2 : 0;
+    constexpr int CV = KT / 8;                    // chunks of a value row (transposed)
+    constexpr int kBuf = kKeyBytes + kValueBytes;
+    constexpr int KS = DK / 32, VF = DV / 16;
+    static_assert(DK % 64 == 0 && DV % 16 == 0 && KT % 32 == 0 && (!EXPANDED || CV == 8), "tile sizes");
+    __shared__ __attribute__((aligned(128))) uint8_t lds[NBUF * kBuf];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, g = lane >> 4;
+    const int z = blockIdx.y;
+    // the longest rows first
+    const int row0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * (16 * QS * WAVES);
+    const int pos = min(max(a.pos_dev[0], 0), a.max_seq - 1);
+    const int last_row = min(row0 + 16 * QS * WAVES, a.rows) - 1;
+    const int wg_keys = min(pos + last_row / a.rows_per_token, a.max_seq - 1) + 1;  // keys any row of the workgroup sees
+    int key_begin = 0, key_end = wg_keys;
+    if (a.splits > 1) {
+        const int all = min(pos + (a.rows - 1) / a.rows_per_token, a.max_seq - 1) + 1;
+        const int share = ((all + a.splits - 1) / a.splits + KT - 1) / KT * KT;
+        key_begin = min((int)blockIdx.z * share, wg_keys);
+        key_end = min(key_begin + share, wg_keys);
+    }
+    const bf16* k_own = a.k_own + z * a.k_own_head;
+    const bf16* v_t = EXPANDED ? a.v_t + (size_t)z * a.dv * a.ld_v : nullptr;
+    const int own_chunks = a.k_own_width >> 3, all_chunks = own_chunks + (EXPANDED ? a.k_shared_width >> 3 : 0);
+    auto copy_tile = [&](int key0, int buf) {
+        uint8_t* base = lds + buf * kBuf;
+        for (int n = wave; n < KT * CK / 64; n += WAVES) {
+            const int q = n * 64 + lane, r = q / CK, c = (q % CK) ^ (r & 7);
+            const size_t key = min(key0 + r, wg_keys - 1);
+            const bf16* src = k_own + key * a.ld_k_own;
+            if (c < own_chunks)
+                src += c * 8;
+            else if (EXPANDED && c < all_chunks)
+                src = a.k_shared + key * a.ld_k_shared + (c - own_chunks) * 8;
+            copy16_to_lds(src, base + n * 1024);
+        }
+        if constexpr (EXPANDED)
+            for (int n = wave; n < DV * CV / 64; n += WAVES) {
+                const int q = n * 64 + lane, r = q >> 3, c = (q & 7) ^ (r & 7);
+                copy16_to_lds(v_t + (size_t)min(r, a.dv - 1) * a.ld_v + key0 + c * 8, base + kKeyBytes + n * 1024);
+            }
+    };
+    // query operands
+    bf16x8 qf[QS][KS];
+    int limit[QS];  // last visible key of this lane's query
+#pragma unroll
+    for (int s = 0; s < QS; s++) {
+        const int r = row0 + (wave * QS + s) * 16 + l15, rc = min(r, a.rows - 1);
+        limit[s] = r < a.rows ? min(pos + rc / a.rows_per_token, a.max_seq - 1) : -1;
+        const bf16* src = a.q + z * a.q_head + (size_t)rc * a.ld_q;
+#pragma unroll
+        for (int k = 0; k < KS; k++) {
+            uint4 u = make_uint4(0, 0, 0, 0);
+            const int c = k * 4 + g;
+            if (c < all_chunks) u = *reinterpret_cast<const uint4*>(src + c * 8);
+            qf[s][k] = *reinterpret_cast<const bf16x8*>(&u);
+        }
+    }
+    f32x4 acc[QS][VF];
+    float mx[QS], sum[QS];
+#pragma unroll
+    for (int s = 0; s < QS; s++) {
+        mx[s] = kLowest;
+        sum[s] = 0.f;
+#pragma unroll
+        for (int f = 0; f < VF; f++) acc[s][f] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    // Values that are columns of the key rows: element (key row r, column 16 f + l15), r = 16 h + 4 g + j, sits at chunk
+    // (2 f + l15 / 8) ^ (r & 7); the exclusive or touches the low three bits only, so sixteen offsets serve all.
+    int value_at[4][4];
+    if constexpr (!EXPANDED) {
+#pragma unroll
+        for (int f = 0; f < 4; f++)
+#pragma unroll
+            for (int j = 0; j < 4; j++)
+                value_at[f][j] = (4 * g + j) * (DK * 2) + (((2 * f + (l15 >> 3)) ^ ((4 * g + j) & 7)) << 4) + (l15 & 7) * 2;
+    }
+    const float scale = a.scale * kLog2e;
+    const int n_tiles = (key_end - key_begin + KT - 1) / KT;
+    if (NBUF > 1 && n_tiles > 0) copy_tile(key_begin, 0);
+    for (int tile = 0; tile < n_tiles; tile++) {
+        const int key0 = key_begin + tile * KT;
+        if (NBUF == 1) {
+            if (tile) __syncthreads();  // nobody still reads the tile
+            copy_tile(key0, 0);
+        }
+        __builtin_amdgcn_s_waitcnt(0x0070);
+        __syncthreads();
+        if (NBUF > 1 && tile + 1 < n_tiles) copy_tile(key0 + KT, (tile + 1) % NBUF);
+        const uint8_t* kb = lds + (tile % NBUF) * kBuf;
+        const uint8_t* vb = kb + kKeyBytes;
+        f32x4 sc[QS][KT / 16];
+#pragma unroll
+        for (int t = 0; t < KT / 16; t++) {
+#pragma unroll
+            for (int s = 0; s < QS; s++) sc[s][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+            const uint8_t* row = kb + (t * 16 + l15) * (DK * 2);
+#pragma unroll
+            for (int k = 0; k < KS; k++) {
+                const bf16x8 kf = *reinterpret_cast<const bf16x8*>(row + (((k * 4 + g) ^ (l15 & 7)) << 4));
+#pragma unroll
+                for (int s = 0; s < QS; s++) sc[s][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s][k], sc[s][t], 0, 0, 0);
+            }
+        }
+        bf16x8 pf[QS][KT / 32];
+#pragma unroll
+        for (int s = 0; s < QS; s++) {
+            float m = mx[s];
+#pragma unroll
+            for (int t = 0; t < KT / 16; t++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const int key = key0 + t * 16 + 4 * g + i;
+                    const float v = sc[s][t][i] * scale;
+                    sc[s][t][i] = key <= limit[s] && key < key_end ? v : kLowest;
+                    m = fmaxf(m, sc[s][t][i]);
+                }
+            m = fmaxf(m, __shfl_xor(m, 16, 64));
+            m = fmaxf(m, __shfl_xor(m, 32, 64));
+            const float keep = exp2f(mx[s] - m);
+            float add = 0.f;
+#pragma unroll
+            for (int t = 0; t < KT / 16; t++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const float p = sc[s][t][i] > kLowest ? exp2f(sc[s][t][i] - m) : 0.f;
+                    add += p;
+                    pf[s][t >> 1][(t & 1) * 4 + i] = (bf16)p;
+                }
+            sum[s] = sum[s] * keep + add;
+            mx[s] = m;
+            if (__any(keep != 1.f)) {
+#pragma unroll
+                for (int f = 0; f < VF; f++) acc[s][f] *= keep;
+            }
+        }
+#pragma unroll
+        for (int u = 0; u < KT / 32; u++)
+#pragma unroll
+            for (int f = 0; f < VF; f++) {
+                bf16x8 vf;
+                if constexpr (EXPANDED) {
+                    const int r = f * 16 + l15;
+                    const uint8_t* row = vb + r * (KT * 2);
+                    const int c0 = u * 4 + (g >> 1);
+                    uint2 lo = *reinterpret_cast<const uint2*>(row + ((c0 ^ (r & 7)) << 4) + (g & 1) * 8);
+                    uint2 hi = *reinterpret_cast<const uint2*>(row + (((c0 + 2) ^ (r & 7)) << 4) + (g & 1) * 8);
+                    const uint4 w = make_uint4(lo.x, lo.y, hi.x, hi.y);
+                    vf = *reinterpret_cast<const bf16x8*>(&w);
+                } else {
+#pragma unroll
+                    for (int j = 0; j < 8; j++)
+                        vf[j] = *reinterpret_cast<const bf16*>(kb + value_at[f & 3][j & 3] + (f >> 2) * 128 +
+                                                               (u * 32 + (j >> 2) * 16) * (DK * 2));
+                }
+#pragma unroll
+                for (int s = 0; s < QS; s++) acc[s][f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[s][u], acc[s][f], 0, 0, 0);
+            }
+    }
+    // lane l holds value columns 16 f + 4 g + i of query l % 16
+#pragma unroll
+    for (int s = 0; s < QS; s++) {
+        float all = sum[s];
+        all += __shfl_xor(all, 16, 64);
+        all += __shfl_xor(all, 32, 64);
+        const int r = row0 + (wave * QS + s) * 16 + l15;
+        if (r >= a.rows) continue;
+        if (a.splits > 1) {
+            const size_t at = (size_t)blockIdx.z * a.rows + r;
+            if (g == 0) {
+                a.part_stats[2 * at] = mx[s];
+                a.part_stats[2 * at + 1] = all;
+            }
+            float* dst = a.part + at * a.ld_part;
+#pragma unroll
+            for (int f = 0; f < VF; f++)
+                if (f * 16 + 4 * g < a.ld_part) *reinterpret_cast<f32x4*>(dst + f * 16 + 4 * g) = acc[s][f];
+        } else {
+            float inv = 1.0f / all;
+            if (a.head_gate) inv *= sigmoid(a.head_gate[(size_t)r * a.ld_gate + z]);
+            bf16* dst = a.out + z * a.out_head + (size_t)r * a.ld_out;
+#pragma unroll
+            for (int f = 0; f < VF; f++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const int d = f * 16 + 4 * g + i;
+                    if (d < a.dv) dst[d] = (bf16)(acc[s][f][i] * inv);
+                }
+        }
+    }
+}
+
+// out[row] = sum_s w_s part_s / sum_s w_s sum_s with w_s = 2^(m_s - max m); one workgroup per row and 256 columns
+template <typename O>
+__global__ __launch_bounds__(256) void merge_shares_kernel(const float* __restrict__ part, int ld_part, const float* __restrict__ stats,
+                                                         int rows, int splits, int dv, O* __restrict__ out, int ld_out) {
+    __shared__ float w[kAttendMaxSplits];
+    __shared__ float norm;
+    const int r = blockIdx.x, t = threadIdx.x;
+    if (t < 64) {
+        float m = t < splits ? stats[2 * ((size_t)t * rows + r)] : kLowest;
+        const float l = t < splits ? stats[2 * ((size_t)t * rows + r) + 1] : 0.f;
+        const float top = dense_wave_max(m);
+        const float mine = exp2f(m - top);
+        if (t < splits) w[t] = mine;
+        const float total = dense_wave_sum(t < splits ? mine * l : 0.f);
+        if (t == 0) norm = 1.0f / total;
+    }
+    __syncthreads();
+    const int d = blockIdx.y * 256 + t;
+    if (d >= dv) return;
+    float s = 0.f;
+    for (int k = 0; k < splits; k++) s = fmaf(w[k], part[((size_t)k * rows + r) * ld_part + d], s);
+    out[(size_t)r * ld_out + d] = (O)(s * norm);
+}
+static_assert(kAttendMaxSplits <= 64, "the merge reads one share per lane");
+
+template <int DK, int DV, bool EXPANDED>
+hipError_t launch_sizes(const AttendArgs& a, int heads, hipStream_t s) {
+    if constexpr (EXPANDED) {
+        constexpr int rows = 16 * 2 * 4;
+        hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 2, 64, 2, true>), dim3((a.rows + rows - 1) / rows, heads, 1), dim3(256), 0, s, a);
+    } else if (a.rows <= 32) {
+        hipLaunchKernelGGL((attend_kernel<DK, DV, 1, 1, 32, 1, false>), dim3((a.rows + 15) / 16, 1, a.splits), dim3(64), 0, s, a);
+    } else {
+        hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 1, 32, 1, false>), dim3((a.rows + 63) / 64, 1, a.splits), dim3(256), 0, s, a);
+    }
+    return hipGetLastError();
+}
+
+}  // namespace
+
+bool attend_shared_fits(int dk, int dv) { return dk <= 576 && dv <= 512; }
+bool attend_expanded_fits(int own, int shared, int dv) { return own % 8 == 0 && shared % 8 == 0 && own + shared <= 320 && dv <= 256; }
+
+hipError_t launch_attend_shared(const AttendArgs& a, hipStream_t s) {
+    const int dk = a.k_own_width;
+    if (dk <= 192 && a.dv <= 128) return launch_sizes<192, 128, false>(a, 1, s);
+    if (dk <= 320 && a.dv <= 256) return launch_sizes<320, 256, false>(a, 1, s);
+    return launch_sizes<576, 512, false>(a, 1, s);
+}
+
+hipError_t launch_attend_expanded(const AttendArgs& a, int heads, hipStream_t s) {
+    const int dk = a.k_own_width + a.k_shared_width;
+    if (dk <= 128 && a.dv <= 64) return launch_sizes<128, 64, true>(a, heads, s);
+    if (dk <= 192 && a.dv <= 128) return launch_sizes<192, 128, true>(a, heads, s);
+    return launch_sizes<320, 256, true>(a, heads, s);
+}
+
+template <typename O>
+hipError_t launch_merge_shares(const AttendArgs& a, O* out, int ld_out, hipStream_t s) {
+    hipLaunchKernelGGL(merge_shares_kernel<O>, dim3(a.rows, (a.dv + 255) / 256), dim3(256), 0, s, a.part, a.ld_part, a.part_stats, a.rows,
+                       a.splits, a.dv, out, ld_out);
+    return hipGetLastError();
+}
+template hipError_t launch_merge_shares<bf16>(const AttendArgs&, bf16*, int, hipStream_t);
+template hipError_t launch_merge_shares<float>(const AttendArgs&, float*, int, hipStream_t);
+
+}  // namespace a81w41

@@ -117,10 +117,89 @@ template <typename T>
 hipError_t launch_rotate_queries(const float* q, int ld_q, const LatentRows& in, const LatentShape& sh, int M, T* nope, int ld_nope,
                                  T* rot_out, int ld_rot, hipStream_t s);
 // Attention in latent space: query rows [M heads][ld_cache] like cache rows (the key up-projection is in the query),
-// causal over cache rows 0 .. pos + m; out [M heads][ld_out] the weighted latents (T).
+// causal over cache rows 0 .. pos + m; out [M heads][ld_out] the weighted latents (T or float).
 // The vector kernel takes any sizes.
-template <typename T>
+template <typename T, typename O>
 hipError_t launch_latent_attention_vector(const T* q, const T* cache, const LatentShape& sh, const int* pos_dev, int max_seq, int M,
-                                          T* out, int ld_out, hipStream_t s);
+                                          O* out, int ld_out, hipStream_t s);
+
+// ---- attention on the matrix cores, bfloat16 (attend_mfma.hip) ------------------------------
+// Query row r of head z: q + z q_head + r ld_q; it belongs to token r / rows_per_token of the pass and sees the keys
+// 0 .. pos + token.  The results go to out, or, with splits > 1 (the keys dealt to that many workgroups), unnormalised
+// to part [splits][rows][ld_part] with part_stats [splits][rows][2] (maximum, sum), for launch_merge_shares.
+constexpr int kAttendMaxSplits = 64;
+struct AttendArgs {
+    const bf16* q = nullptr;
+    long long q_head = 0;
+    int ld_q = 0, rows = 0, rows_per_token = 1;
+    // key = [k_own + z k_own_head + key ld_k_own (k_own_width) | k_shared + key ld_k_shared (k_shared_width)]; widths
+    // are multiples of 8, rows 16-byte aligned
+    const bf16* k_own = nullptr;
+    long long k_own_head = 0;
+    int ld_k_own = 0, k_own_width = 0;
+    const bf16* k_shared = nullptr;
+    int ld_k_shared = 0, k_shared_width = 0;
+    // expanded: value column d of head z is v_t + (z dv + d) ld_v, readable up to a multiple of 64 keys
+    const bf16* v_t = nullptr;
+    int ld_v = 0, dv = 0;
+    const float* head_gate = nullptr;  // expanded: result times the sigmoid of head_gate[r ld_gate + z]
+    int ld_gate = 0;
+    bf16* out = nullptr;
+    long long out_head = 0;
+    int ld_out = 0;
+    int splits = 1;
+    float *part = nullptr, *part_stats = nullptr;
+    int ld_part = 0;  // a multiple of 4
+    float scale = 0.f;
+    const int* pos_dev = nullptr;
+    int max_seq = 0;
+};
+bool attend_shared_fits(int dk, int dv);
+bool attend_expanded_fits(int own, int shared, int dv);
+// Keys and values are the same rows (k_own), the values their first dv columns.
+hipError_t launch_attend_shared(const AttendArgs& a, hipStream_t s);
+hipError_t launch_attend_expanded(const AttendArgs& a, int heads, hipStream_t s);
+template <typename O>
+hipError_t launch_merge_shares(const AttendArgs& a, O* out, int ld_out, hipStream_t s);
+
+// ---- one-token products with the row work fused in (dense_gemv.hip) --------------------------
+// Their input rows sit in LDS as fp32: a row (or, for the experts' second product, all of a token's) may have at most
+// kGemvMaxRow elements, padding and norm groups included.
+constexpr int kGemvMaxRow = 15000;
+// r = x + norm_y(y) (y may be null), the stream before + *coef r (before null: r), the row its norm_h.  Workgroup 0
+// writes r to state and the stream to x_out (either may be null); neither may be a buffer the step reads.
+struct RowStep {
+    const float *x = nullptr, *y = nullptr;
+    GroupNorm norm_y;
+    const float *before = nullptr, *coef = nullptr;
+    float *state = nullptr, *x_out = nullptr;
+    GroupNorm norm_h;
+    int width = 0;
+};
+template <typename T>
+hipError_t launch_gemv_step(const RowStep& p, const T* w, int ld, int N, float* C, hipStream_t s);
+template <typename T>
+hipError_t launch_gemv_plain(const float* x, int K, const T* w, int ld, int N, float* C, hipStream_t s);
+// Queries; also the token's cache row (cache may be null) and before = sum_{j < depth.n} coef[j] states[j].
+template <typename T>
+hipError_t launch_gemv_query(const LatentRows& in, const LatentShape& sh, const T* w, int ld, float* q, T* cache, const DepthAverage& depth,
+                             int width, float* before, hipStream_t s);
+template <typename T>
+hipError_t launch_gemv_absorb(const float* q, const LatentRows& in, const LatentShape& sh, const T* uk_t, int ld, T* q_lat, hipStream_t s);
+template <typename T>
+hipError_t launch_gemv_values(const float* o_lat, int ld_o, const LatentShape& sh, const T* uv, int ld, const float* gates, float* attn,
+                              hipStream_t s);
+// The feed-forwards a token uses: `top` of `experts` by table (0: none), and one every token uses (dense_ff 0: none).
+struct ExpertRows {
+    const int *ids = nullptr, *table = nullptr;
+    int vocab = 1, top = 0, experts = 0, ff = 0, pair_rows = 0;  // pair_rows: gate/up rows of one expert
+    int dense_ff = 0;
+    int ld_act = 0;  // activations of slot k (the dense one after the experts) at k ld_act
+};
+template <typename T>
+hipError_t launch_gemv_gate_up(const RowStep& p, const ExpertRows& e, const T* experts, const T* dense, int ld, float* act, hipStream_t s);
+template <typename T>
+hipError_t launch_gemv_ff_down(const ExpertRows& e, const float* act, const T* experts, int ld, const T* dense, int ld_dense, int N,
+                               float* y, hipStream_t s);
 
 }  // namespace a81w41

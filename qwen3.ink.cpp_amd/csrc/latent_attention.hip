@@ -59,10 +59,10 @@ __global__ __launch_bounds__(kThreads) void rotate_queries_kernel(const float* _
 
 // One workgroup per (token, head).  Keys in blocks of kBlock: every wave scores a quarter of the block's keys, the block's
 // maximum rescales what is there, then every thread owns some of the output's elements.
-template <typename T>
+template <typename T, typename O>
 __global__ __launch_bounds__(kThreads) void latent_attention_vector_kernel(const T* __restrict__ q, const T* __restrict__ cache,
                                                                           LatentShape sh, const int* __restrict__ pos_dev,
-                                                                          int max_seq, T* __restrict__ out, int ld_out) {
+                                                                          int max_seq, O* __restrict__ out, int ld_out) {
     constexpr int kBlock = 64;
     extern __shared__ float smem[];
     float* qs = smem;                        // rank + rot
@@ -103,7 +103,7 @@ __global__ __launch_bounds__(kThreads) void latent_attention_vector_kernel(const
         }
         __syncthreads();
     }
-    for (int i = t; i < sh.rank; i += kThreads) out[(size_t)blockIdx.x * ld_out + i] = (T)(acc[i] / sum);
+    for (int i = t; i < sh.rank; i += kThreads) out[(size_t)blockIdx.x * ld_out + i] = (O)(acc[i] / sum);
 }
 
 }  // namespace
@@ -121,21 +121,25 @@ hipError_t launch_rotate_queries(const float* q, int ld_q, const LatentRows& in,
     return hipGetLastError();
 }
 
-template <typename T>
+template <typename T, typename O>
 hipError_t launch_latent_attention_vector(const T* q, const T* cache, const LatentShape& sh, const int* pos_dev, int max_seq, int M,
-                                          T* out, int ld_out, hipStream_t s) {
+                                          O* out, int ld_out, hipStream_t s) {
     const size_t lds = (2 * (size_t)sh.rank + sh.rot + 64) * sizeof(float);
-    hipLaunchKernelGGL(latent_attention_vector_kernel<T>, dim3(M * sh.heads), dim3(kThreads), lds, s, q, cache, sh, pos_dev, max_seq,
+    hipLaunchKernelGGL((latent_attention_vector_kernel<T, O>), dim3(M * sh.heads), dim3(kThreads), lds, s, q, cache, sh, pos_dev, max_seq,
                        out, ld_out);
     return hipGetLastError();
 }
+template hipError_t launch_latent_attention_vector<bf16, bf16>(const bf16*, const bf16*, const LatentShape&, const int*, int, int, bf16*, int,
+                                                               hipStream_t);
+template hipError_t launch_latent_attention_vector<bf16, float>(const bf16*, const bf16*, const LatentShape&, const int*, int, int, float*,
+                                                                int, hipStream_t);
+template hipError_t launch_latent_attention_vector<float, float>(const float*, const float*, const LatentShape&, const int*, int, int,
+                                                                 float*, int, hipStream_t);
 
 #define INSTANTIATE(T)                                                                                                           \
     template hipError_t launch_latent_rows<T>(const LatentRows&, const LatentShape&, int, T*, int, T*, hipStream_t);               \
     template hipError_t launch_rotate_queries<T>(const float*, int, const LatentRows&, const LatentShape&, int, T*, int, T*, int, \
-                                                 hipStream_t);                                                                   \
-    template hipError_t launch_latent_attention_vector<T>(const T*, const T*, const LatentShape&, const int*, int, int, T*, int, \
-                                                          hipStream_t);
+                                                 hipStream_t);
 INSTANTIATE(bf16)
 INSTANTIATE(float)
 

@@ -126,6 +126,20 @@ class TakosunModel final : public a81w41_model {
     }
     size_t weight_bytes() const override { return weight_bytes_; }
 
+    // unfused: one-token passes take the kernels of longer ones; attention: 0 by shape, 1 the vector kernel, 2 in latent
+    // space, 3 on formed keys and values; attention_split: shares of the keys in latent space, 0 by length
+    int set_option(const char* name, int value) override {
+        const std::string n = name;
+        if (n == "unfused" && value >= 0 && value <= 1)
+            opt_unfused_ = value;
+        else if (n == "attention" && value >= 0 && value <= 3)
+            opt_attention_ = value;
+        else if (n == "attention_split" && value >= 0 && value <= kAttendMaxSplits)
+            opt_split_ = value;
+        else
+            return failf(A81W41_ERR_INVALID_ARG, "no option '%s' with value %d", name, value);
+        return 0;
+    }
     // state<i>: [tokens of the last pass][width], the stream after i layers, before the mean over depth
     int read_buffer(const char* name, float* host_out, size_t count) override {
         int i = -1;
@@ -148,12 +162,17 @@ class TakosunModel final : public a81w41_model {
         float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr, *dwa = nullptr;
         float *q_norm = nullptr, *kv_norm = nullptr;
         Weight<T> down;  // [dq | dkv | g]
-        Weight<T> uq, uk_t, uv, o;
+        Weight<T> uq, uk, uk_t, uv, o;  // uk_t: per head, transposed; uk as stored, for formed keys
         FeedForward ff, shared;
         int* table = nullptr;
         T* cache = nullptr;
         float *cos_t = nullptr, *sin_t = nullptr;
     };
+    static constexpr bool kMatrixAttention = sizeof(T) == 2;
+    // whether a layer can form its keys and values per head for many new tokens
+    static bool can_expand(const LatentShape& sh) {
+        return kMatrixAttention && sh.rank % 8 == 0 && attend_expanded_fits(sh.dim, sh.rot, sh.vdim);
+    }
     int n_layers() const { return (int)cfg_.layers.size(); }
     long long state_step() const { return (long long)rows_ * cfg_.width; }
     GroupNorm norm(const float* w) const { return GroupNorm{w, cfg_.groups, cfg_.eps}; }
@@ -223,6 +242,12 @@ class TakosunModel final : public a81w41_model {
     int load_rotation(const LayerConfig& lc, int max_seq, Layer* L);
     int allocate(int max_seq);
     int attention(const Layer& L, const LayerConfig& lc, int M, hipStream_t s);
+    int attend_latent(const Layer& L, const LatentShape& sh, int M, hipStream_t s);
+    int attend_formed(const Layer& L, const LatentShape& sh, int M, const float* gates, hipStream_t s);
+    AttendArgs shared_attend(const Layer& L, const LatentShape& sh, int M) const;
+    int enqueue_one_token(int n_want, hipStream_t s);
+    int feed_forward_one_token(const Layer& L, const LayerConfig& lc, const RowStep& step, hipStream_t s);
+    LatentRows latent_rows(const Layer& L) const;
     int feed_forward(const Layer& L, const LayerConfig& lc, int M, hipStream_t s, SublayerOut* out);
     int pair_product(const FeedForward& f, int ff, const T* h, const GemmArgs& base, T* act, hipStream_t s);
     GemmArgs product(const T* A, int lda, const Weight<T>& w, void* C, int ldc, int M) const {
@@ -242,6 +267,17 @@ class TakosunModel final : public a81w41_model {
     int rows_ = 0, ld_h_ = 0, ld_down_ = 0, ld_q_ = 0, ld_cq_ = 0, ld_attn_ = 0;
     float *x_ = nullptr, *states_ = nullptr, *down_ = nullptr, *q_ = nullptr, *y_ = nullptr, *y2_ = nullptr, *y_shared_ = nullptr;
     T *h_ = nullptr, *c_q_ = nullptr, *nope_ = nullptr, *q_lat_ = nullptr, *o_lat_ = nullptr, *attn_ = nullptr, *act_ = nullptr;
+    bf16 *k_formed_ = nullptr, *v_formed_ = nullptr;  // [max_seq][heads dim], [heads vdim][ld_v_]
+    int ld_v_ = 0;
+    float *part_ = nullptr, *part_stats_ = nullptr;  // shares of the attention in latent space
+    size_t part_rows_ = 0;
+    int ld_part_ = 0;
+    // of the one-token pass
+    float *row_x_[2] = {nullptr, nullptr}, *row_mid_ = nullptr, *before_ = nullptr, *y_ff_ = nullptr;
+    float *o_lat_row_ = nullptr, *attn_row_ = nullptr, *act_row_ = nullptr;
+    int ld_act_row_ = 0;
+    bool one_token_fits_ = true;
+    int opt_unfused_ = 0, opt_attention_ = 0, opt_split_ = 0;
     int *src_rows_ = nullptr, *slot_rows_ = nullptr, *n_tiles_ = nullptr;
     GroupTile* tiles_ = nullptr;
 };
@@ -302,6 +338,11 @@ int TakosunModel<T>::load_weights(int max_seq, TensorSource& src) {
         {   // the key up-projection of a head, transposed: it maps an unrotated query to latent space
             std::vector<float> uk, row(sh.dim);
             A81W41_TRY(src.matrix(mix + "uk", sh.heads * sh.dim, sh.rank, uk));
+            if (can_expand(sh)) {
+                Staging st(sh.heads * sh.dim, sh.rank);
+                for (int r = 0; r < st.rows; r++) st.put(r, uk.data() + (size_t)r * sh.rank);
+                A81W41_TRY(finish(st, &L.uk));
+            }
             Staging t(sh.heads * sh.rank, sh.dim);
             for (int h = 0; h < sh.heads; h++)
                 for (int r = 0; r < sh.rank; r++) {
@@ -337,7 +378,9 @@ int TakosunModel<T>::allocate(int max_seq) {
     rows_ = std::min(max_seq, kPassRows);
     A81W41_TRY(init_session(max_seq, cfg_.vocab, rows_));
     ld_h_ = pad_k<T>(cfg_.width);
-    size_t nope = 0, q_lat = 0, o_lat = 0, act = 0, expert_rows = 0, tiles = 0;
+    size_t nope = 0, q_lat = 0, o_lat = 0, act = 0, expert_rows = 0, tiles = 0, formed_k = 0, formed_v = 0;
+    int slots = 1, heads = 0;
+    one_token_fits_ = ld_h_ + cfg_.groups <= kGemvMaxRow;
     for (const LayerConfig& lc : cfg_.layers) {
         const LatentShape& sh = lc.mix;
         ld_down_ = std::max(ld_down_, sh.q_rank + sh.rank + sh.rot + sh.heads);
@@ -347,10 +390,21 @@ int TakosunModel<T>::allocate(int max_seq) {
         nope = std::max(nope, (size_t)sh.heads * pad_k<T>(sh.dim));
         q_lat = std::max(q_lat, (size_t)sh.heads * sh.ld_cache);
         o_lat = std::max(o_lat, (size_t)sh.heads * pad_k<T>(sh.rank));
+        heads = std::max(heads, sh.heads);
+        ld_part_ = std::max(ld_part_, (sh.rank + 3) / 4 * 4);
+        one_token_fits_ = one_token_fits_ && pad_k<T>(sh.q_rank) <= kGemvMaxRow && pad_k<T>(sh.heads * sh.vdim) <= kGemvMaxRow;
+        if (can_expand(sh)) {
+            formed_k = std::max(formed_k, (size_t)sh.heads * sh.dim);
+            formed_v = std::max(formed_v, (size_t)sh.heads * sh.vdim);
+            nope = std::max(nope, (size_t)sh.heads * (sh.dim + sh.rot));
+        }
         const FeedForwardConfig& f = lc.mlp;
         if (!f.present) continue;
         act = std::max(act, (size_t)std::max(f.top, 1) * pad_k<T>(f.ff));
         act = std::max(act, (size_t)pad_k<T>(f.shared_ff));
+        ld_act_row_ = std::max(ld_act_row_, std::max(f.ff, f.shared_ff));
+        slots = std::max(slots, f.top + 1);
+        one_token_fits_ = one_token_fits_ && std::max(f.top, 1) * pad_k<T>(f.ff) + pad_k<T>(f.shared_ff) <= kGemvMaxRow;
         if (f.experts_by_table) {
             expert_rows = std::max(expert_rows, (size_t)f.top);
             tiles = std::max(tiles, (size_t)rows_ * f.top / kGroupTileRows + f.experts);
@@ -369,6 +423,18 @@ int TakosunModel<T>::allocate(int max_seq) {
     A81W41_TRY(allocate_array(R * ld_attn_, &attn_));
     A81W41_TRY(allocate_array(R * act, &act_));
     A81W41_TRY(allocate_array(R * W, &y_));
+    if (formed_k) {
+        ld_v_ = (max_seq + 63) / 64 * 64;
+        A81W41_TRY(allocate_array((size_t)max_seq * formed_k, &k_formed_));
+        A81W41_TRY(allocate_array(formed_v * ld_v_, &v_formed_));
+    }
+    part_rows_ = std::max((size_t)heads * kAttendMaxSplits, (size_t)8192);
+    A81W41_TRY(allocate_array(part_rows_ * ld_part_, &part_));
+    A81W41_TRY(allocate_array(part_rows_ * 2, &part_stats_));
+    for (float** row : {&row_x_[0], &row_x_[1], &row_mid_, &before_, &y_ff_}) A81W41_TRY(allocate_array(W, row));
+    A81W41_TRY(allocate_array(o_lat, &o_lat_row_));
+    A81W41_TRY(allocate_array((size_t)ld_attn_, &attn_row_));
+    A81W41_TRY(allocate_array((size_t)slots * ld_act_row_, &act_row_));
     if (expert_rows) {
         A81W41_TRY(allocate_array(R * expert_rows * W, &y2_));
         A81W41_TRY(allocate_array(R * W, &y_shared_));
@@ -380,29 +446,99 @@ int TakosunModel<T>::allocate(int max_seq) {
     return 0;
 }
 
+template <typename T>
+LatentRows TakosunModel<T>::latent_rows(const Layer& L) const {
+    LatentRows in;
+    in.down = down_, in.ld_down = ld_down_, in.q_norm = L.q_norm, in.kv_norm = L.kv_norm, in.eps = cfg_.eps;
+    in.cos_t = L.cos_t, in.sin_t = L.sin_t, in.pos_dev = pos, in.max_seq = max_seq();
+    return in;
+}
+
+// Query rows q_lat_ (like cache rows) against the layer's cache.
+template <typename T>
+AttendArgs TakosunModel<T>::shared_attend(const Layer& L, const LatentShape& sh, int M) const {
+    AttendArgs a;
+    a.q = reinterpret_cast<const bf16*>(q_lat_), a.ld_q = sh.ld_cache, a.rows = M * sh.heads, a.rows_per_token = sh.heads;
+    a.k_own = reinterpret_cast<const bf16*>(L.cache), a.ld_k_own = sh.ld_cache, a.k_own_width = (sh.rank + sh.rot + 7) / 8 * 8;
+    a.dv = sh.rank, a.scale = sh.scale, a.pos_dev = pos, a.max_seq = max_seq();
+    a.part = part_, a.part_stats = part_stats_, a.ld_part = (sh.rank + 3) / 4 * 4;
+    // enough workgroups for the chip, at least 64 keys for each
+    const int groups = a.rows <= 32 ? (a.rows + 15) / 16 : (a.rows + 63) / 64;
+    a.splits = opt_split_ ? opt_split_ : std::min({kAttendMaxSplits, (plan_ctx + 63) / 64, std::max(1, 512 / groups)});
+    a.splits = std::max<int>(1, std::min<size_t>(a.splits, part_rows_ / a.rows));
+    return a;
+}
+
+// Attention in latent space: the key up-projection moves into the query, the value up-projection behind the sum.
+// Leaves the weighted latents in o_lat_.
+template <typename T>
+int TakosunModel<T>::attend_latent(const Layer& L, const LatentShape& sh, int M, hipStream_t s) {
+    const LatentRows in = latent_rows(L);
+    const int ld_nope = pad_k<T>(sh.dim), ld_rank = pad_k<T>(sh.rank);
+    A81W41_HIP_TRY(launch_rotate_queries<T>(q_, ld_q_, in, sh, M, nope_, ld_nope, q_lat_ + sh.rank, sh.ld_cache, s));
+    GemmArgs g = product(nope_, sh.heads * ld_nope, L.uk_t, q_lat_, sh.heads * sh.ld_cache, M);
+    g.N = sh.rank, g.batches = sh.heads, g.a_step = ld_nope, g.w_step = (long long)sh.rank * L.uk_t.ld, g.c_step = sh.ld_cache;
+    A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kElement, s));
+    bool done = false;
+    if constexpr (kMatrixAttention) {
+        if (opt_attention_ != 1 && attend_shared_fits(sh.rank + sh.rot, sh.rank)) {
+            AttendArgs a = shared_attend(L, sh, M);
+            a.out = o_lat_, a.ld_out = ld_rank;
+            A81W41_HIP_TRY(launch_attend_shared(a, s));
+            if (a.splits > 1) A81W41_HIP_TRY(launch_merge_shares<bf16>(a, o_lat_, ld_rank, s));
+            done = true;
+        }
+    }
+    if (!done) A81W41_HIP_TRY((launch_latent_attention_vector<T, T>(q_lat_, L.cache, sh, pos, max_seq(), M, o_lat_, ld_rank, s)));
+    return 0;
+}
+
+// Attention on keys and values formed per head: fewer operations per key once there are many new tokens.
+template <typename T>
+int TakosunModel<T>::attend_formed(const Layer& L, const LatentShape& sh, int M, const float* gates, hipStream_t s) {
+    if constexpr (kMatrixAttention) {
+        const int ctx = plan_ctx, dk = sh.dim + sh.rot;  // a pass of several tokens is planned for exactly its context
+        GemmArgs g = product(L.cache, sh.ld_cache, L.uk, k_formed_, sh.heads * sh.dim, ctx);
+        A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kElement, s));
+        // values transposed: the roles of weight and cache change
+        g.A = L.uv.data, g.lda = L.uv.ld, g.M = L.uv.rows, g.W = L.cache, g.ldw = sh.ld_cache, g.N = ctx, g.K = L.uv.ld;
+        g.C = v_formed_, g.ldc = ld_v_;
+        A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kElement, s));
+        A81W41_HIP_TRY(launch_rotate_queries<T>(q_, ld_q_, latent_rows(L), sh, M, nope_, dk, nope_ + sh.dim, dk, s));
+        AttendArgs a;
+        a.q = nope_, a.q_head = dk, a.ld_q = sh.heads * dk, a.rows = M;
+        a.k_own = k_formed_, a.k_own_head = sh.dim, a.ld_k_own = sh.heads * sh.dim, a.k_own_width = sh.dim;
+        a.k_shared = L.cache + sh.rank, a.ld_k_shared = sh.ld_cache, a.k_shared_width = sh.rot;
+        a.v_t = v_formed_, a.ld_v = ld_v_, a.dv = sh.vdim;
+        a.head_gate = gates, a.ld_gate = ld_down_;
+        a.out = attn_, a.out_head = sh.vdim, a.ld_out = ld_attn_;
+        a.scale = sh.scale, a.pos_dev = pos, a.max_seq = max_seq();
+        A81W41_HIP_TRY(launch_attend_expanded(a, sh.heads, s));
+    }
+    return 0;
+}
+
 // The mixer on h_: leaves its output rows in y_.
 template <typename T>
 int TakosunModel<T>::attention(const Layer& L, const LayerConfig& lc, int M, hipStream_t s) {
     const LatentShape& sh = lc.mix;
     const bool own = lc.kv_from < 0;
-    const int gates_at = sh.q_rank + (own ? sh.rank + sh.rot : 0);
-    LatentRows in;
-    in.down = down_, in.ld_down = ld_down_, in.q_norm = L.q_norm, in.kv_norm = L.kv_norm, in.eps = cfg_.eps;
-    in.cos_t = L.cos_t, in.sin_t = L.sin_t, in.pos_dev = pos, in.max_seq = max_seq();
+    const float* gates = down_ + sh.q_rank + (own ? sh.rank + sh.rot : 0);
     A81W41_HIP_TRY(launch_dense_gemm<T>(product(h_, ld_h_, L.down, down_, ld_down_, M), Epilogue::kFloat, s));
-    A81W41_HIP_TRY(launch_latent_rows<T>(in, sh, M, c_q_, ld_cq_, own ? L.cache : nullptr, s));
+    A81W41_HIP_TRY(launch_latent_rows<T>(latent_rows(L), sh, M, c_q_, ld_cq_, own ? L.cache : nullptr, s));
     A81W41_HIP_TRY(launch_dense_gemm<T>(product(c_q_, ld_cq_, L.uq, q_, ld_q_, M), Epilogue::kFloat, s));
-    const int ld_nope = pad_k<T>(sh.dim), ld_rank = pad_k<T>(sh.rank);
-    // query rows like cache rows: the part in latent space comes from the product below
-    A81W41_HIP_TRY(launch_rotate_queries<T>(q_, ld_q_, in, sh, M, nope_, ld_nope, q_lat_ + sh.rank, sh.ld_cache, s));
-    GemmArgs g = product(nope_, sh.heads * ld_nope, L.uk_t, q_lat_, sh.heads * sh.ld_cache, M);
-    g.N = sh.rank, g.batches = sh.heads, g.a_step = ld_nope, g.w_step = (long long)sh.rank * L.uk_t.ld, g.c_step = sh.ld_cache;
-    A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kElement, s));
-    A81W41_HIP_TRY(launch_latent_attention_vector<T>(q_lat_, L.cache, sh, pos, max_seq(), M, o_lat_, ld_rank, s));
-    g = product(o_lat_, sh.heads * ld_rank, L.uv, attn_, ld_attn_, M);
-    g.N = sh.vdim, g.batches = sh.heads, g.a_step = ld_rank, g.w_step = (long long)sh.vdim * L.uv.ld, g.c_step = sh.vdim;
-    g.head_gate = down_ + gates_at, g.ld_gate = ld_down_;
-    A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kHeadGate, s));
+    // per key and head, latent space costs M (2 rank + rot) against M (dim + rot + vdim) and rank (dim + vdim) once
+    const bool many = (long long)M * (2 * sh.rank - sh.dim - sh.vdim) > (long long)sh.rank * (sh.dim + sh.vdim);
+    if (can_expand(sh) && (opt_attention_ == 3 || (opt_attention_ == 0 && many))) {
+        A81W41_TRY(attend_formed(L, sh, M, gates, s));
+    } else {
+        A81W41_TRY(attend_latent(L, sh, M, s));
+        const int ld_rank = pad_k<T>(sh.rank);
+        GemmArgs g = product(o_lat_, sh.heads * ld_rank, L.uv, attn_, ld_attn_, M);
+        g.N = sh.vdim, g.batches = sh.heads, g.a_step = ld_rank, g.w_step = (long long)sh.vdim * L.uv.ld, g.c_step = sh.vdim;
+        g.head_gate = gates, g.ld_gate = ld_down_;
+        A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kHeadGate, s));
+    }
     A81W41_HIP_TRY(launch_dense_gemm<T>(product(attn_, ld_attn_, L.o, y_, cfg_.width, M), Epilogue::kFloat, s));
     return 0;
 }
@@ -438,8 +574,81 @@ int TakosunModel<T>::feed_forward(const Layer& L, const LayerConfig& lc, int M, 
     return 0;
 }
 
+// The same feed-forward for one token behind the residual step `step`: leaves its output row in y_ff_.
+template <typename T>
+int TakosunModel<T>::feed_forward_one_token(const Layer& L, const LayerConfig& lc, const RowStep& step, hipStream_t s) {
+    const FeedForwardConfig& f = lc.mlp;
+    const FeedForward& every = f.experts_by_table ? L.shared : L.ff;  // what every token uses
+    ExpertRows e;
+    e.dense_ff = f.experts_by_table ? f.shared_ff : f.ff;
+    e.ld_act = ld_act_row_;
+    if (f.experts_by_table) {
+        e.ids = ids, e.table = L.table, e.vocab = cfg_.vocab, e.top = f.top, e.experts = f.experts, e.ff = f.ff;
+        e.pair_rows = pair_columns(f.ff);
+    }
+    A81W41_HIP_TRY(launch_gemv_gate_up<T>(step, e, L.ff.gate_up.data, every.gate_up.data, L.ff.gate_up.ld, act_row_, s));
+    A81W41_HIP_TRY(launch_gemv_ff_down<T>(e, act_row_, L.ff.down.data, L.ff.down.ld, every.down.data, every.down.ld, cfg_.width, y_ff_, s));
+    return 0;
+}
+
+// The pass for one token: the row work between two products runs inside the product that consumes it, eight launches a
+// layer (nine with the merge of the attention's shares).  The sum over the earlier states of the mean over depth is
+// formed beside the query product, so that the next layer's first product adds only the newest state.
+template <typename T>
+int TakosunModel<T>::enqueue_one_token(int n_want, hipStream_t s) {
+    const int W = cfg_.width, n = n_layers();
+    A81W41_HIP_TRY(launch_embed_rows(ids, embed_.data, sizeof(T) == 2 ? TableType::kBf16 : TableType::kFp32, embed_.ld, states_, 1, W,
+                                     cfg_.vocab, s));
+    RowStep step;  // what the next product's prologue does
+    step.x = states_, step.width = W, step.norm_h = norm(layers_[0].norm1);
+    for (int i = 0; i < n; i++) {
+        const Layer& L = layers_[i];
+        const LayerConfig& lc = cfg_.layers[i];
+        const LatentShape& sh = lc.mix;
+        const bool own = lc.kv_from < 0;
+        A81W41_HIP_TRY(launch_gemv_step<T>(step, L.down.data, L.down.ld, L.down.rows, down_, s));
+        const float* x = i ? step.x_out : states_;
+        DepthAverage depth;
+        depth.states = states_, depth.state_step = state_step(), depth.coef = L.dwa, depth.n = i + 1;
+        const LatentRows in = latent_rows(L);
+        A81W41_HIP_TRY(launch_gemv_query<T>(in, sh, L.uq.data, L.uq.ld, q_, own ? L.cache : nullptr, depth, W, before_, s));
+        A81W41_HIP_TRY(launch_gemv_absorb<T>(q_, in, sh, L.uk_t.data, L.uk_t.ld, q_lat_, s));
+        const int ld_rank = pad_k<T>(sh.rank);
+        bool done = false;
+        if constexpr (kMatrixAttention) {
+            if (opt_attention_ != 1 && attend_shared_fits(sh.rank + sh.rot, sh.rank)) {
+                AttendArgs a = shared_attend(L, sh, 1);
+                a.splits = std::max(a.splits, 2);  // the shares stay fp32 until they are merged
+                A81W41_HIP_TRY(launch_attend_shared(a, s));
+                A81W41_HIP_TRY(launch_merge_shares<float>(a, o_lat_row_, ld_rank, s));
+                done = true;
+            }
+        }
+        if (!done)
+            A81W41_HIP_TRY((launch_latent_attention_vector<T, float>(q_lat_, L.cache, sh, pos, max_seq(), 1, o_lat_row_, ld_rank, s)));
+        A81W41_HIP_TRY(launch_gemv_values<T>(o_lat_row_, ld_rank, sh, L.uv.data, L.uv.ld, down_ + sh.q_rank + (own ? sh.rank + sh.rot : 0),
+                                             attn_row_, s));
+        A81W41_HIP_TRY(launch_gemv_plain<T>(attn_row_, sh.heads * sh.vdim, L.o.data, L.o.ld, W, y_, s));
+        step = RowStep{};
+        step.width = W, step.x = x, step.y = y_, step.norm_y = norm(L.norm1b);
+        if (lc.mlp.present) {
+            step.x_out = row_mid_, step.norm_h = norm(L.norm2);
+            A81W41_TRY(feed_forward_one_token(L, lc, step, s));
+            step.x = row_mid_, step.y = y_ff_, step.norm_y = norm(L.norm2b);
+        }
+        step.before = before_, step.coef = L.dwa + i + 1, step.state = states_ + (i + 1) * state_step();
+        step.x_out = row_x_[i & 1];
+        step.norm_h = norm(i + 1 < n ? layers_[i + 1].norm1 : final_norm_);
+    }
+    if (n_want) A81W41_HIP_TRY(launch_gemv_step<T>(step, head_.data, head_.ld, head_.rows, logits, s));
+    A81W41_HIP_TRY(launch_advance(pos, 1, s));
+    return 0;
+}
+
 template <typename T>
 int TakosunModel<T>::enqueue_pass(int M, const int* want, int n_want, hipStream_t s) {
+    (void)want;  // the head product reads want_dev
+    if (M == 1 && one_token_fits_ && !opt_unfused_) return enqueue_one_token(n_want, s);
     const int W = cfg_.width, n = n_layers();
     A81W41_HIP_TRY(launch_embed_rows(ids, embed_.data, sizeof(T) == 2 ? TableType::kBf16 : TableType::kFp32, embed_.ld, states_, M, W,
                                      cfg_.vocab, s));

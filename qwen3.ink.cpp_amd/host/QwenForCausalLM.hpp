@@ -7,7 +7,7 @@
 // call forward() with the new token ids, read logits(0, 0, v) of the last token.  The
 // model keeps its own position, like the reference's past_sqlen member.
 //
-// Header only; link with -la81w41.  Failures throw std::runtime_error.
+// Header only; link with -la81w41 -la81w41_core.  Failures throw std::runtime_error.
 #pragma once
 
 #include <string>

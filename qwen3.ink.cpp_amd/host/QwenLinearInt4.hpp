@@ -10,7 +10,7 @@
 // activations are copied in and the result out on every call, like any caller
 // that keeps its tensors in host memory must.
 //
-// Header only; link with -la81w41.  Failures throw std::runtime_error with the
+// Header only; link with -la81w41 -la81w41_core.  Failures throw std::runtime_error with the
 // library's message (the reference aborts on asserts / throws on file errors).
 #pragma once
 
