@@ -11,6 +11,7 @@ import os
 _HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(_HERE, "csrc")
 LIB_PATH = os.path.join(CSRC, "liba81w41.so")
+DENSE_PATH = os.path.join(CSRC, "liba81w41_dense.so")
 CORE_PATH = os.path.join(CSRC, "liba81w41_core.so")
 
 OK = 0
@@ -101,6 +102,13 @@ CORE_SIGNATURES = {
     "a81w41_model_resident_bytes": (_sz, [_vp, C.POINTER(_sz), C.POINTER(_sz)]),
 }
 
+# every symbol include/a81w41_dense.h declares
+DENSE_SIGNATURES = {
+    "a81w41_dense_gemm": (_i, [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _vp]),
+    "a81w41_latent_attention": (_i, [_vp, _vp, _i, _i, _i, _i, _vp, _i, _i, C.c_float, _vp, _i, _i, _i, _vp, _vp, _vp]),
+    "a81w41_formed_attention": (_i, [_vp, _vp, _vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _vp, _i, _i, C.c_float, _vp, _vp]),
+}
+
 
 class Qwen3Config(C.Structure):
     """a81w41_qwen3_config"""
@@ -135,6 +143,11 @@ def load(path: str, signatures: dict):
 def lib():
     """The A81W41 layer and the Qwen3 model, every exported symbol bound."""
     return load(LIB_PATH, SIGNATURES)
+
+
+def dense():
+    """The models with dense weights and their parity hooks."""
+    return load(DENSE_PATH, DENSE_SIGNATURES)
 
 
 def core():

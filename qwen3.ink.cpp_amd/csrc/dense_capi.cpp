@@ -1,0 +1,78 @@
+// The parity hooks of include/a81w41_dense.h: argument checks in front of the launchers.
+#include "../../include/a81w41_dense.h"
+
+#include "decoder_session.h"
+#include "dense.h"
+
+using namespace a81w41;
+
+namespace {
+bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
+template <typename T>
+int gemm(const void* A, int lda, const void* W, int ldw, float* C, int ldc, int M, int N, int K, hipStream_t s) {
+    constexpr int step = 128 / (int)sizeof(T);
+    if (lda % step || ldw % step || lda < pad_k<T>(K) || ldw < pad_k<T>(K) || ldc < N)
+        return failf(A81W41_ERR_INVALID_ARG, "row strides must be whole multiples of 128 bytes and cover K");
+    GemmArgs g;
+    g.A = A, g.W = W, g.C = C, g.M = M, g.N = N, g.K = pad_k<T>(K), g.lda = lda, g.ldw = ldw, g.ldc = ldc;
+    A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kFloat, s));
+    return 0;
+}
+}  // namespace
+
+extern "C" {
+
+int a81w41_dense_gemm(const void* A, int lda, const void* W, int ldw, float* C, int ldc, int M, int N, int K, int is_bf16, void* stream) {
+    if (!A || !W || !C || M < 1 || N < 1 || K < 1 || !aligned16(A) || !aligned16(W)) return failf(A81W41_ERR_INVALID_ARG, "bad product");
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    return is_bf16 ? gemm<bf16>(A, lda, W, ldw, C, ldc, M, N, K, s) : gemm<float>(A, lda, W, ldw, C, ldc, M, N, K, s);
+}
+
+int a81w41_latent_attention(const void* q, const void* cache, int ld, int rank, int rot, int heads, const int* pos_dev, int max_seq, int M,
+                            float scale, void* out, int is_bf16, int variant, int splits, float* part, float* stats, void* stream) {
+    if (!q || !cache || !pos_dev || !out || rank < 1 || rot < 0 || heads < 1 || max_seq < 1 || M < 1 || rank + rot > 4096 ||
+        ld < rank + rot || ld % (is_bf16 ? 64 : 32) || variant < 0 || variant > 1 || !aligned16(q) || !aligned16(cache))
+        return failf(A81W41_ERR_INVALID_ARG, "bad attention shape");
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    LatentShape sh;
+    sh.heads = heads, sh.rank = rank, sh.rot = rot, sh.ld_cache = ld, sh.scale = scale;
+    if (variant == 0) {
+        if (is_bf16)
+            A81W41_HIP_TRY((launch_latent_attention_vector<bf16, bf16>(static_cast<const bf16*>(q), static_cast<const bf16*>(cache), sh, pos_dev,
+                                                                       max_seq, M, static_cast<bf16*>(out), rank, s)));
+        else
+            A81W41_HIP_TRY((launch_latent_attention_vector<float, float>(static_cast<const float*>(q), static_cast<const float*>(cache), sh,
+                                                                         pos_dev, max_seq, M, static_cast<float*>(out), rank, s)));
+        return 0;
+    }
+    if (!is_bf16 || !attend_shared_fits(rank + rot, rank) || splits < 1 || splits > kAttendMaxSplits || (splits > 1 && (!part || !stats)))
+        return failf(A81W41_ERR_INVALID_ARG, "the matrix-core attention does not take this shape");
+    AttendArgs a;
+    a.q = static_cast<const bf16*>(q), a.ld_q = ld, a.rows = M * heads, a.rows_per_token = heads;
+    a.k_own = static_cast<const bf16*>(cache), a.ld_k_own = ld, a.k_own_width = (rank + rot + 7) / 8 * 8, a.dv = rank;
+    a.out = static_cast<bf16*>(out), a.ld_out = rank, a.splits = splits, a.part = part, a.part_stats = stats, a.ld_part = (rank + 3) / 4 * 4;
+    a.scale = scale, a.pos_dev = pos_dev, a.max_seq = max_seq;
+    A81W41_HIP_TRY(launch_attend_shared(a, s));
+    if (splits > 1) A81W41_HIP_TRY(launch_merge_shares<bf16>(a, a.out, rank, s));
+    return 0;
+}
+
+int a81w41_formed_attention(const void* q, const void* k, const void* k_rot, int ld_rot, const void* v_t, int ld_v, const float* gates,
+                            int heads, int dim, int rot, int vdim, const int* pos_dev, int max_seq, int M, float scale, void* out,
+                            void* stream) {
+    if (!q || !k || !k_rot || !v_t || !gates || !pos_dev || !out || heads < 1 || dim < 1 || rot < 1 || vdim < 1 || max_seq < 1 || M < 1 ||
+        ld_rot < rot || ld_rot % 8 || ld_v % 64 || ld_v < max_seq || !attend_expanded_fits(dim, rot, vdim) || !aligned16(q) || !aligned16(k) ||
+        !aligned16(k_rot) || !aligned16(v_t))
+        return failf(A81W41_ERR_INVALID_ARG, "bad attention shape");
+    AttendArgs a;
+    a.q = static_cast<const bf16*>(q), a.q_head = dim + rot, a.ld_q = heads * (dim + rot), a.rows = M;
+    a.k_own = static_cast<const bf16*>(k), a.k_own_head = dim, a.ld_k_own = heads * dim, a.k_own_width = dim;
+    a.k_shared = static_cast<const bf16*>(k_rot), a.ld_k_shared = ld_rot, a.k_shared_width = rot;
+    a.v_t = static_cast<const bf16*>(v_t), a.ld_v = ld_v, a.dv = vdim, a.head_gate = gates, a.ld_gate = heads;
+    a.out = static_cast<bf16*>(out), a.out_head = vdim, a.ld_out = heads * vdim;
+    a.scale = scale, a.pos_dev = pos_dev, a.max_seq = max_seq;
+    A81W41_HIP_TRY(launch_attend_expanded(a, heads, static_cast<hipStream_t>(stream)));
+    return 0;
+}
+
+}  // extern "C"

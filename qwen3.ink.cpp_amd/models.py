@@ -16,10 +16,10 @@ import numpy as np
 
 from . import capi
 
-# architecture name in config.json -> (library, make target that builds it)
+# architecture name in config.json -> (loader of its library, the library's path, make target that builds it)
 ARCHITECTURES = {
-    "Qwen3": ("liba81w41.so", "liba81w41.so"),
-    "Takosun": ("liba81w41_dense.so", "dense"),
+    "Qwen3": (capi.lib, capi.LIB_PATH, "liba81w41.so"),
+    "Takosun": (capi.dense, capi.DENSE_PATH, "dense"),
 }
 
 
@@ -37,8 +37,7 @@ def read_config(model_dir: str) -> dict:
 
 def ensure_built(architecture: str) -> None:
     """Compile the architecture's library if it is not there (progress goes to stderr)."""
-    library, target = ARCHITECTURES[architecture]
-    path = os.path.join(capi.CSRC, library)
+    _, path, target = ARCHITECTURES[architecture]
     if os.path.exists(path):
         return
     with open(os.path.join(capi.CSRC, ".build.lock"), "w") as lock:
@@ -59,7 +58,7 @@ class Model:
     @classmethod
     def load(cls, model_dir: str, max_seq: int, dtype: str = "bfloat16") -> "Model":
         name = architecture_of(read_config(model_dir))
-        cls._library(name)
+        ARCHITECTURES[name][0]()
         h = C.c_void_p()
         capi.check(capi.core().a81w41_model_load(os.fsencode(model_dir), dtype.encode(), max_seq, C.byref(h)))
         return cls(h, name)
@@ -68,14 +67,10 @@ class Model:
     def random(cls, config: dict, max_seq: int, dtype: str = "bfloat16", seed: int = 0) -> "Model":
         """Seeded random weights of the configuration's shapes (for benchmarks)."""
         name = architecture_of(config)
-        cls._library(name)
+        ARCHITECTURES[name][0]()
         h = C.c_void_p()
         capi.check(capi.core().a81w41_model_create_random(json.dumps(config).encode(), dtype.encode(), max_seq, seed, C.byref(h)))
         return cls(h, name)
-
-    @staticmethod
-    def _library(name: str) -> None:
-        capi.load(os.path.join(capi.CSRC, ARCHITECTURES[name][0]), {})
 
     def reset(self) -> None:
         capi.check(capi.core().a81w41_model_reset(self.handle))

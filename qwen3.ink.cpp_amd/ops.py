@@ -194,6 +194,51 @@ def attention_one_token(qkv, q_w, k_w, cos, sin, k_cache, v_cache, pos: int, n_q
     return out
 
 
+# ---------------------------------------------------------------- mechanisms of the dense-weight models
+
+def _element(t):
+    torch = _torch()
+    assert t.dtype in (torch.bfloat16, torch.float32)
+    return int(t.dtype == torch.bfloat16)
+
+
+def dense_gemm(a, w, K: int):
+    """Parity hook a81w41_dense_gemm: a [M][lda], w [N][ldw] (CUDA, bfloat16 or float32, K padded) -> fp32 [M][N]."""
+    torch = _torch()
+    out = torch.empty((a.shape[0], w.shape[0]), dtype=torch.float32, device=a.device)
+    capi.check(capi.dense().a81w41_dense_gemm(_dev_ptr(a), a.shape[1], _dev_ptr(w), w.shape[1], _dev_ptr(out), w.shape[0], a.shape[0],
+                                              w.shape[0], K, _element(a), _stream()))
+    return out
+
+
+def latent_attention(q, cache, pos: int, rank: int, rot: int, heads: int, scale: float, variant: int = 0, splits: int = 1):
+    """Parity hook a81w41_latent_attention: q [M*heads][ld], cache [max_seq][ld] -> [M*heads][rank] of q's type."""
+    torch = _torch()
+    rows = q.shape[0]
+    out = torch.empty((rows, rank), dtype=q.dtype, device=q.device)
+    pos_dev = torch.tensor([pos], dtype=torch.int32, device=q.device)
+    part = torch.empty((splits * rows, (rank + 3) // 4 * 4), dtype=torch.float32, device=q.device)
+    stats = torch.empty((splits * rows, 2), dtype=torch.float32, device=q.device)
+    capi.check(capi.dense().a81w41_latent_attention(
+        _dev_ptr(q), _dev_ptr(cache), q.shape[1], rank, rot, heads, _dev_ptr(pos_dev), cache.shape[0], rows // heads, scale,
+        _dev_ptr(out), _element(q), variant, splits, _dev_ptr(part), _dev_ptr(stats), _stream()))
+    return out
+
+
+def formed_attention(q, k, k_rot, v_t, gates, pos: int, vdim: int, scale: float):
+    """Parity hook a81w41_formed_attention: q [M][heads][dim+rot], k [max_seq][heads*dim], k_rot [max_seq][ld],
+    v_t [heads*vdim][ld_v] (bfloat16), gates [M][heads] fp32 -> bfloat16 [M][heads*vdim]."""
+    torch = _torch()
+    M, heads, width = q.shape
+    dim = k.shape[1] // heads
+    out = torch.empty((M, heads * vdim), dtype=torch.bfloat16, device=q.device)
+    pos_dev = torch.tensor([pos], dtype=torch.int32, device=q.device)
+    capi.check(capi.dense().a81w41_formed_attention(
+        _dev_ptr(q), _dev_ptr(k), _dev_ptr(k_rot), k_rot.shape[1], _dev_ptr(v_t), v_t.shape[1], _dev_ptr(gates), heads, dim,
+        width - dim, vdim, _dev_ptr(pos_dev), k.shape[0], M, scale, _dev_ptr(out), _stream()))
+    return out
+
+
 # ---------------------------------------------------------------- layer objects
 
 class Context:

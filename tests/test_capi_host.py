@@ -11,15 +11,18 @@ import pytest
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
-def test_exports_every_declared_symbol(pkg):
-    L = pkg.capi.lib()
-    header = open(os.path.join(ROOT, "include", "a81w41.h")).read()
+@pytest.mark.parametrize("name", ["a81w41", "a81w41_model", "a81w41_dense"])
+def test_exports_every_declared_symbol(pkg, name):
+    L, signatures, also = {"a81w41": (pkg.capi.lib(), pkg.capi.SIGNATURES, set()),
+                           "a81w41_model": (pkg.capi.core(), pkg.capi.CORE_SIGNATURES, {"a81w41_status_string", "a81w41_last_error"}),
+                           "a81w41_dense": (pkg.capi.dense(), pkg.capi.DENSE_SIGNATURES, set())}[name]
+    header = open(os.path.join(ROOT, "include", name + ".h")).read()
     header = re.sub(r"/\*.*?\*/", "", header, flags=re.S)   # declarations only, not prose
-    declared = set(re.findall(r"\b(a81w41_[A-Za-z0-9_]+)\s*\(", header))
+    declared = set(re.findall(r"\b(a81w41_[A-Za-z0-9_]+)\s*\(", header)) | also
     assert declared, "no declarations parsed"
-    for name in sorted(declared):
-        assert hasattr(L, name), f"library lacks {name}"
-    assert declared == set(pkg.capi.SIGNATURES), declared ^ set(pkg.capi.SIGNATURES)
+    for symbol in sorted(declared):
+        assert hasattr(L, symbol), f"library lacks {symbol}"
+    assert declared == set(signatures), declared ^ set(signatures)
 
 
 def test_blob_sizes(pkg):
