@@ -22,6 +22,7 @@ Also reported in the same JSON line:
   m_sweep       forward at M in {1, 8, 32, 128, 512, 2048} on gate and down
   e2e           random-init Qwen3-8B: 322-token prefill + 128 greedy decode steps, resident bytes
   a80w40        the A80W40 variant's GEMV sweep and M=322 GEMM
+  (--takosun [SIZE] runs the Takosun model beside Qwen3 at equal size instead and prints that object)
 Every figure is the median of five timed windows (the minimum is reported beside it).
   cpu_baseline  the AVX2+OpenMP port of the reference's CPU path on this host
 """
@@ -56,6 +57,14 @@ LM_HEAD = ("lm_head", 4096, 151936)
 N_LAYERS = 36
 
 
+# Layers of the Takosun leg: every second layer reads the cache of the one before; MoE layers where `experts` is given.
+TAKOSUN_SIZES = {
+    "2k": dict(width=2048, heads=16, q_rank=768, ff=6144, layers=12),
+    "4k": dict(width=4096, heads=32, q_rank=1536, ff=12288, layers=8),
+    "2k-moe": dict(width=2048, heads=16, q_rank=768, ff=6144, layers=12, experts=64, top=6, expert_ff=1024, shared_ff=1024),
+}
+
+
 def gemv_bytes(K, N):
     return 0.625 * K * N + 1.125 * K + 4.0 * N
 
@@ -79,6 +88,11 @@ def parse():
     ap.add_argument("--branches", type=int, default=8,
                     help="parallel branches the step's independent launches are captured into (1 = one chain)")
     ap.add_argument("--e2e-only", action="store_true", help="run only the end-to-end leg (prints its JSON object)")
+    ap.add_argument("--takosun", nargs="?", const="all", choices=["all"] + sorted(TAKOSUN_SIZES), metavar="SIZE",
+                    help="run only the Takosun model at sizes like a real model's layers, beside Qwen3 at equal size "
+                         "(prints its JSON object)")
+    ap.add_argument("--takosun-prompt", type=int, default=2048)
+    ap.add_argument("--takosun-no-qwen", action="store_true", help="leave the Qwen3 runs of --takosun out (for profiles)")
     ap.add_argument("--no-m-sweep", action="store_true", help="skip the M sweep on the gate and down shapes")
     ap.add_argument("--no-e2e", action="store_true",
                     help="skip the random-init Qwen3-8B forward pass (322-token prefill + 128 greedy decode steps; "
@@ -145,6 +159,10 @@ def main():
     assert torch.cuda.is_available(), "bench.py needs a GPU"
     torch.cuda.set_device(0)
     ops, synth = pkg.ops, pkg.synth
+
+    if args.takosun:
+        print(json.dumps(takosun_leg(pkg, args.takosun, args.takosun_prompt, with_qwen=not args.takosun_no_qwen)), flush=True)
+        return
 
     if args.e2e_only:
         print(json.dumps(end_to_end(pkg)), flush=True)
@@ -624,13 +642,79 @@ def a80w40_leg(pkg, M):
             "note": "gemv: bytes-weighted over 36 x seven shapes + lm_head; gemm time includes the operand rewrite"}
 
 
-def build_e2e_model(pkg, n_prompt=322):
-    """Random-init Qwen3-8B (36 layers, hidden 4096, 32 q / 8 kv heads x 128, intermediate 12288,
+def takosun_config(size):
+    d = dict(TAKOSUN_SIZES[size])
+    layers = []
+    for i in range(d["layers"]):
+        mixer = {"heads": d["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": d["q_rank"], "kv_rank": 512,
+                 "scale": 192.0 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}
+        if i % 2:
+            mixer["kv_from"] = i - 1
+        mlp = {"kind": "dense", "ff": d["ff"]}
+        if "experts" in d and i % 2:
+            mlp = {"kind": "moe", "router": {"experts": d["experts"], "top": d["top"]}, "expert": {"ff": d["expert_ff"]},
+                   "shared": {"ff": d["shared_ff"]}}
+        layers.append({"type": "latent_attention", "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Takosun", "vocab": 32768, "width": d["width"], "norm": {"eps": 1e-6, "groups": 8}, "layers": layers}
+
+
+def takosun_work(cfg, n_prompt):
+    """(weight bytes a decoded token reads, multiply-add operations x 2 of the prompt outside attention, in attention)"""
+    W, weights, attn = cfg["width"], cfg["vocab"] * cfg["width"], 0
+    for l in cfg["layers"]:
+        m, f = l["mixer"], l["mlp"]
+        kv = 0 if "kv_from" in m else m["kv_rank"] + m["rot_dim"]
+        weights += W * (m["q_rank"] + kv + m["heads"]) + m["q_rank"] * m["heads"] * (m["dim"] + m["rot_dim"])
+        weights += m["heads"] * (m["dim"] + m["vdim"]) * m["kv_rank"] + W * m["heads"] * m["vdim"]
+        weights += 3 * W * (f["ff"] if f["kind"] == "dense" else f["router"]["top"] * f["expert"]["ff"] + f["shared"]["ff"])
+        attn += n_prompt * (n_prompt + 1) // 2 * m["heads"] * (m["dim"] + m["rot_dim"] + m["vdim"]) * 2
+    return 2 * weights, 2 * (weights - cfg["vocab"] * W) * n_prompt, attn
+
+
+def takosun_leg(pkg, which, n_prompt=2048, n_decode=128, with_qwen=True):
+    """Prefill and decode rates of Takosun (bfloat16 weights, seeded random) and, at equal width, feed-forward, depth and
+    vocabulary, of Qwen3 on A81W41 linears.  The two differ in weight format: bytes and operations stand beside the times."""
+    out = {}
+    for size in sorted(TAKOSUN_SIZES) if which == "all" else [which]:
+        cfg = takosun_config(size)
+        max_seq = n_prompt + n_decode + 2
+        t0 = time.time()
+        model = pkg.Model.random(cfg, max_seq, "bfloat16", seed=1)
+        print(f"[bench] Takosun {size} resident after {time.time() - t0:.1f}s", file=sys.stderr, flush=True)
+        prompt = np.random.default_rng(7).integers(0, cfg["vocab"], n_prompt).astype(np.int32)
+        toks, ms_pre, ms_dec = time_generation(model, prompt, n_decode)
+        nbytes, flops, attn = takosun_work(cfg, n_prompt)
+        row = {"prefill_tokens": n_prompt, "prefill_ms": round(ms_pre, 3), "prefill_tokens_per_s": round(n_prompt / ms_pre * 1e3, 1),
+               "prefill_TFLOPS": round((flops + attn) / ms_pre / 1e9, 1), "prefill_attention_share_of_flops": round(attn / (flops + attn), 3),
+               "decode_ms_per_token": round(ms_dec / n_decode, 4), "decode_tokens_per_s": round(n_decode / ms_dec * 1e3, 1),
+               "decode_weight_MB_per_token": round(nbytes / 1e6, 1), "decode_GBps": round(nbytes / (ms_dec / n_decode) / 1e6, 1),
+               "decode_hbm_frac": round(nbytes / (ms_dec / n_decode) / 1e6 / HBM_PEAK_GBS, 4), "config": TAKOSUN_SIZES[size]}
+        model.close()
+        if with_qwen and "experts" not in TAKOSUN_SIZES[size]:
+            d = TAKOSUN_SIZES[size]
+            q = dict(n_layers=d["layers"], hidden=d["width"], n_q_heads=d["heads"], n_kv_heads=d["heads"] // 4, intermediate=d["ff"],
+                     vocab=cfg["vocab"], max_seq=max_seq)
+            qwen, _, n_w = build_e2e_model(pkg, n_prompt, q)
+            _, ms_pre, ms_dec = time_generation(qwen, prompt, n_decode)
+            qbytes = 0.625 * n_w
+            row["qwen3_equal_size"] = {
+                "prefill_ms": round(ms_pre, 3), "prefill_tokens_per_s": round(n_prompt / ms_pre * 1e3, 1),
+                "prefill_TOPS": round(2 * (n_w - cfg["vocab"] * d["width"]) * n_prompt / ms_pre / 1e9, 1),
+                "decode_ms_per_token": round(ms_dec / n_decode, 4), "decode_tokens_per_s": round(n_decode / ms_dec * 1e3, 1),
+                "decode_weight_MB_per_token": round(qbytes / 1e6, 1), "decode_GBps": round(qbytes / (ms_dec / n_decode) / 1e6, 1),
+                "decode_hbm_frac": round(qbytes / (ms_dec / n_decode) / 1e6 / HBM_PEAK_GBS, 4)}
+            del qwen
+        out[size] = row
+    return out
+
+
+def build_e2e_model(pkg, n_prompt=322, cfg=None):
+    """Random-init Qwen3-8B (or the sizes of cfg; 36 layers, hidden 4096, 32 q / 8 kv heads x 128, intermediate 12288,
     vocab 151936, RoPE theta 1e6, fp16 KV cache), every linear A81W41 from the seeded generator
     (one weight set per shape, a distinct HBM copy per layer); uniform random prompt ids.
     -> (model, prompt, number of linear weights)"""
     ops, synth = pkg.ops, pkg.synth
-    cfg = dict(n_layers=N_LAYERS, hidden=4096, n_q_heads=32, n_kv_heads=8, intermediate=12288, vocab=151936, max_seq=512)
+    cfg = cfg or dict(n_layers=N_LAYERS, hidden=4096, n_q_heads=32, n_kv_heads=8, intermediate=12288, vocab=151936, max_seq=512)
     t0 = time.time()
     model = ops.Qwen3Model(**cfg)
     H, I, V = cfg["hidden"], cfg["intermediate"], cfg["vocab"]
@@ -664,7 +748,7 @@ def build_e2e_model(pkg, n_prompt=322):
         emb[r0:r1] = (8.0 * rng.standard_normal((r1 - r0, H), dtype=np.float32)).astype(np.float16)
     model.set_embedding(emb)
     del emb
-    print(f"[bench] Qwen3-8B random-init model resident after {time.time() - t0:.1f}s", file=sys.stderr, flush=True)
+    print(f"[bench] Qwen3 random-init model resident after {time.time() - t0:.1f}s", file=sys.stderr, flush=True)
     prompt = rng.integers(0, V, size=n_prompt).astype(np.int32)
     n_w = sum(n * k for n, k in dims) * cfg["n_layers"] + V * H
     return model, prompt, n_w
