@@ -21,21 +21,23 @@ constexpr float kLog2e = 1.4426950408889634f;
 constexpr float kLowest = -1e30f;
 
 // DK, DV: capacities for key and value columns.  KT keys per tile, NBUF tiles in LDS.
-template <int DK, int DV, int WAVES, int QS, int KT, int NBUF, bool EXPANDED>
+// COLS: all waves of the workgroup take the same query rows and each a quarter of the value columns (few rows).
+template <int DK, int DV, int WAVES, int QS, int KT, int NBUF, bool EXPANDED, bool COLS>
 __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
     constexpr int CK = DK / 8;                    // 16-byte chunks of a key row
     constexpr int kKeyBytes = KT * DK * 2, kValueBytes = EXPANDED ? DV * KT * 2 : 0;
     constexpr int CV = KT / 8;                    // chunks of a value row (transposed)
     constexpr int kBuf = kKeyBytes + kValueBytes;
-    constexpr int KS = DK / 32, VF = DV / 16;
+    constexpr int KS = DK / 32, VF = DV / 16 / (COLS ? WAVES : 1), kRows = 16 * QS * (COLS ? 1 : WAVES);
     static_assert(DK % 64 == 0 && DV % 16 == 0 && KT % 32 == 0 && (!EXPANDED || CV == 8), "tile sizes");
     __shared__ __attribute__((aligned(128))) uint8_t lds[NBUF * kBuf];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, g = lane >> 4;
+    const int row_wave = COLS ? 0 : wave, f0 = COLS ? wave * VF : 0;  // first 16 value columns of this wave
     const int z = blockIdx.y;
     // the longest rows first
-    const int row0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * (16 * QS * WAVES);
+    const int row0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * kRows;
     const int pos = min(max(a.pos_dev[0], 0), a.max_seq - 1);
-    const int last_row = min(row0 + 16 * QS * WAVES, a.rows) - 1;
+    const int last_row = min(row0 + kRows, a.rows) - 1;
     const int wg_keys = min(pos + last_row / a.rows_per_token, a.max_seq - 1) + 1;  // keys any row of the workgroup sees
     int key_begin = 0, key_end = wg_keys;
     if (a.splits > 1) {
@@ -70,7 +72,7 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
     int limit[QS];  // last visible key of this lane's query
 #pragma unroll
     for (int s = 0; s < QS; s++) {
-        const int r = row0 + (wave * QS + s) * 16 + l15, rc = min(r, a.rows - 1);
+        const int r = row0 + (row_wave * QS + s) * 16 + l15, rc = min(r, a.rows - 1);
         limit[s] = r < a.rows ? min(pos + rc / a.rows_per_token, a.max_seq - 1) : -1;
         const bf16* src = a.q + z * a.q_head + (size_t)rc * a.ld_q;
 #pragma unroll
@@ -91,14 +93,14 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
         for (int f = 0; f < VF; f++) acc[s][f] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
     // Values that are columns of the key rows: element (key row r, column 16 f + l15), r = 16 h + 4 g + j, sits at chunk
-    // (2 f + l15 / 8) ^ (r & 7); the exclusive or touches the low three bits only, so sixteen offsets serve all.
+    // (2 f + l15 / 8) ^ (r & 7); the exclusive or touches the low three bits only, so sixteen offsets serve all f and h.
     int value_at[4][4];
     if constexpr (!EXPANDED) {
 #pragma unroll
         for (int f = 0; f < 4; f++)
 #pragma unroll
             for (int j = 0; j < 4; j++)
-                value_at[f][j] = (4 * g + j) * (DK * 2) + (((2 * f + (l15 >> 3)) ^ ((4 * g + j) & 7)) << 4) + (l15 & 7) * 2;
+                value_at[f][j] = (4 * g + j) * (DK * 2) + (((2 * (f0 + f) + (l15 >> 3)) ^ ((4 * g + j) & 7)) << 4) + (l15 & 7) * 2;
     }
     const float scale = a.scale * kLog2e;
     const int n_tiles = (key_end - key_begin + KT - 1) / KT;
@@ -165,7 +167,7 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
             for (int f = 0; f < VF; f++) {
                 bf16x8 vf;
                 if constexpr (EXPANDED) {
-                    const int r = f * 16 + l15;
+                    const int r = (f0 + f) * 16 + l15;
                     const uint8_t* row = vb + r * (KT * 2);
                     const int c0 = u * 4 + (g >> 1);
                     uint2 lo = *reinterpret_cast<const uint2*>(row + ((c0 ^ (r & 7)) << 4) + (g & 1) * 8);
@@ -188,18 +190,18 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
         float all = sum[s];
         all += __shfl_xor(all, 16, 64);
         all += __shfl_xor(all, 32, 64);
-        const int r = row0 + (wave * QS + s) * 16 + l15;
+        const int r = row0 + (row_wave * QS + s) * 16 + l15;
         if (r >= a.rows) continue;
         if (a.splits > 1) {
             const size_t at = (size_t)blockIdx.z * a.rows + r;
-            if (g == 0) {
+            if (g == 0 && f0 == 0) {
                 a.part_stats[2 * at] = mx[s];
                 a.part_stats[2 * at + 1] = all;
             }
             float* dst = a.part + at * a.ld_part;
 #pragma unroll
             for (int f = 0; f < VF; f++)
-                if (f * 16 + 4 * g < a.ld_part) *reinterpret_cast<f32x4*>(dst + f * 16 + 4 * g) = acc[s][f];
+                if ((f0 + f) * 16 + 4 * g < a.ld_part) *reinterpret_cast<f32x4*>(dst + (f0 + f) * 16 + 4 * g) = acc[s][f];
         } else {
             float inv = 1.0f / all;
             if (a.head_gate) inv *= sigmoid(a.head_gate[(size_t)r * a.ld_gate + z]);
@@ -208,7 +210,7 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
             for (int f = 0; f < VF; f++)
 #pragma unroll
                 for (int i = 0; i < 4; i++) {
-                    const int d = f * 16 + 4 * g + i;
+                    const int d = (f0 + f) * 16 + 4 * g + i;
                     if (d < a.dv) dst[d] = (bf16)(acc[s][f][i] * inv);
                 }
         }
@@ -244,11 +246,11 @@ template <int DK, int DV, bool EXPANDED>
 hipError_t launch_sizes(const AttendArgs& a, int heads, hipStream_t s) {
     if constexpr (EXPANDED) {
         constexpr int rows = 16 * 2 * 4;
-        hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 2, 64, 2, true>), dim3((a.rows + rows - 1) / rows, heads, 1), dim3(256), 0, s, a);
+        hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 2, 64, 2, true, false>), dim3((a.rows + rows - 1) / rows, heads, 1), dim3(256), 0, s, a);
     } else if (a.rows <= 32) {
-        hipLaunchKernelGGL((attend_kernel<DK, DV, 1, 1, 32, 1, false>), dim3((a.rows + 15) / 16, 1, a.splits), dim3(64), 0, s, a);
+        hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 1, 64, 1, false, true>), dim3((a.rows + 15) / 16, 1, a.splits), dim3(256), 0, s, a);
     } else {
-        hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 1, 32, 1, false>), dim3((a.rows + 63) / 64, 1, a.splits), dim3(256), 0, s, a);
+        hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 1, 32, 1, false, false>), dim3((a.rows + 63) / 64, 1, a.splits), dim3(256), 0, s, a);
     }
     return hipGetLastError();
 }

@@ -186,9 +186,14 @@ hipError_t launch_gemv_query(const LatentRows& in, const LatentShape& sh, const 
                              int width, float* before, hipStream_t s);
 template <typename T>
 hipError_t launch_gemv_absorb(const float* q, const LatentRows& in, const LatentShape& sh, const T* uk_t, int ld, T* q_lat, hipStream_t s);
+// The weighted latents of the heads: o_lat [heads][ld_o], or the shares of launch_attend_shared over `heads` rows.
+struct LatentShares {
+    const float *part = nullptr, *stats = nullptr;
+    int splits = 0, ld = 0;
+};
 template <typename T>
-hipError_t launch_gemv_values(const float* o_lat, int ld_o, const LatentShape& sh, const T* uv, int ld, const float* gates, float* attn,
-                              hipStream_t s);
+hipError_t launch_gemv_values(const float* o_lat, int ld_o, const LatentShares& shares, const LatentShape& sh, const T* uv, int ld,
+                              const float* gates, float* attn, hipStream_t s);
 // The feed-forwards a token uses: `top` of `experts` by table (0: none), and one every token uses (dense_ff 0: none).
 struct ExpertRows {
     const int *ids = nullptr, *table = nullptr;

@@ -25,6 +25,14 @@ __device__ __forceinline__ void copy16_to_lds(const void* global_src, void* lds_
     __builtin_amdgcn_global_load_lds(global_src, (dense_lds_ptr)lds_base, 16, 0, 0);
 }
 
+// A barrier that orders LDS only: requested global loads stay in flight.
+__device__ __forceinline__ void dense_lds_barrier() {
+    __builtin_amdgcn_sched_barrier(0);
+    __builtin_amdgcn_s_waitcnt(0xC07F);  // lgkmcnt = 0; vector-memory and export counters left alone
+    __builtin_amdgcn_s_barrier();
+    __builtin_amdgcn_sched_barrier(0);
+}
+
 // 1 / sqrt(mean of squares + eps) of `groups` equal consecutive parts of a row, into inv[0..groups) (LDS).
 // x(i) is element i.  red: THREADS / 64 floats of LDS.  Ends with a barrier.
 template <int THREADS, typename F>
@@ -53,5 +61,59 @@ __device__ __forceinline__ void group_inverse_rms(F x, int width, int groups, fl
         __syncthreads();
     }
 }
+
+// A row whose norm groups are whole float4s, dealt to a workgroup so that a group's threads are neighbours and a thread
+// holds at most kParts float4s, all of one group: the row stays in registers between its norms.
+template <int THREADS>
+class RowParts {
+   public:
+    static constexpr int kParts = 4;
+    __device__ __forceinline__ RowParts(int width, int groups) : groups_(groups), size_(width / groups) {
+        int per = 1;
+        while (per < groups && per < THREADS) per <<= 1;
+        log_tpg_ = 31 - __builtin_clz((unsigned)(THREADS / per));
+        group_ = threadIdx.x >> log_tpg_;
+        at_ = threadIdx.x & ((1 << log_tpg_) - 1);
+    }
+    __device__ __forceinline__ bool fits() const {
+        return groups_ <= THREADS && (size_ & 3) == 0 && (size_ >> 2) <= (kParts << log_tpg_);
+    }
+    // first element of this thread's k-th float4, -1 if it has none
+    __device__ __forceinline__ int place(int k) const {
+        const int c = at_ + (k << log_tpg_);
+        return group_ < groups_ && 4 * c < size_ ? group_ * size_ + 4 * c : -1;
+    }
+    // of this thread's group; v: the thread's parts (absent ones zero), red: THREADS / 64 floats of LDS
+    __device__ __forceinline__ float inverse_rms(const float4* v, float eps, float* red) const {
+        float sum = 0.f;
+#pragma unroll
+        for (int k = 0; k < kParts; k++) {
+            sum = fmaf(v[k].x, v[k].x, sum), sum = fmaf(v[k].y, v[k].y, sum);
+            sum = fmaf(v[k].z, v[k].z, sum), sum = fmaf(v[k].w, v[k].w, sum);
+        }
+        sum = dense_wave_sum(sum, log_tpg_ < 6 ? 1 << log_tpg_ : 64);
+        if (log_tpg_ > 6) {
+            dense_lds_barrier();  // nobody still reads red
+            if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = sum;
+            dense_lds_barrier();
+            sum = 0.f;
+            const int waves = 1 << (log_tpg_ - 6);
+            for (int w = 0; w < waves; w++) sum += red[group_ * waves + w];
+        }
+        return 1.0f / sqrtf(sum / (float)size_ + eps);
+    }
+
+   private:
+    int groups_, size_, log_tpg_, group_, at_;
+};
+__device__ __forceinline__ float4 load4(const float* a) { return *reinterpret_cast<const float4*>(a); }
+__device__ __forceinline__ void store4(float* a, float4 v) { *reinterpret_cast<float4*>(a) = v; }
+__device__ __forceinline__ float4 fma4(float a, float4 b, float4 c) {
+    return make_float4(fmaf(a, b.x, c.x), fmaf(a, b.y, c.y), fmaf(a, b.z, c.z), fmaf(a, b.w, c.w));
+}
+__device__ __forceinline__ float4 scale4(float4 v, float s, float4 w) {
+    return make_float4(v.x * s * w.x, v.y * s * w.y, v.z * s * w.z, v.w * s * w.w);
+}
+__device__ __forceinline__ float4 add4(float4 a, float4 b) { return make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w); }
 
 }  // namespace a81w41

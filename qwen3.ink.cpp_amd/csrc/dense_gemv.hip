@@ -1,6 +1,7 @@
 // One-token products for dense weights, with the row work around them fused in: every workgroup forms the input row in
 // LDS (fp32) in its prologue -- residual step and norm, the norm of a latent, the attention output -- and its waves
-// then stream weight rows in pairs, 16 bytes per lane and load, eight loads of a pair in flight.  A row's sum is formed
+// then stream weight rows in pairs, 16 bytes per lane and load, the next eight loads in flight while eight are used; the
+// first ones are requested before the prologue.  A row's sum is formed
 // in an order that depends on the row's length only.
 #include "dense_common.h"
 
@@ -28,49 +29,98 @@ __device__ __forceinline__ float dot16(const uint4& w, const float* x, float*) {
     return fmaf(__uint_as_float(w.w), a.w, s);
 }
 
+constexpr int kAhead = 4;  // 16-byte chunks of a row that a lane requests at once
+__host__ __device__ constexpr int lanes_of(int chunks) {
+    int lanes = 1;
+    while (lanes < 64 && lanes * kAhead < chunks) lanes <<= 1;
+    return lanes;
+}
 // How rows are dealt: `lanes` lanes (a power of two) share a pair of rows; `group` counts the lane groups of the launch.
 struct Deal {
     int lanes, group, groups, at;
 };
 template <typename T>
-__device__ __forceinline__ Deal deal_rows(int chunks) {
+__device__ __forceinline__ Deal deal_rows(int chunks, int workgroups) {
     Deal d;
-    d.lanes = 1;
-    while (d.lanes < 64 && 2 * d.lanes <= chunks) d.lanes <<= 1;
+    d.lanes = lanes_of(chunks);
     const int per_wg = kThreads / d.lanes;
     d.group = blockIdx.x * per_wg + threadIdx.x / d.lanes;
-    d.groups = gridDim.x * per_wg;
+    d.groups = workgroups * per_wg;
     d.at = threadIdx.x & (d.lanes - 1);
     return d;
 }
 
-// The dot products of two weight rows with xs (LDS, zero-padded to whole chunks); every lane of the group gets both.
+// Up to kAhead chunks per lane of two weight rows.
+struct Pair {
+    uint4 a[kAhead], b[kAhead];
+};
+struct RowPair {
+    const void *w0, *w1;
+};
+__device__ __forceinline__ void load_pair(Pair& p, const RowPair& r, int c, int lanes, int chunks) {
+    const uint4 *p0 = static_cast<const uint4*>(r.w0), *p1 = static_cast<const uint4*>(r.w1);
+#pragma unroll
+    for (int u = 0; u < kAhead; u++) {
+        const int cc = min(c + u * lanes, chunks - 1);
+        p.a[u] = p0[cc];
+        p.b[u] = p1[cc];
+    }
+}
 template <typename T>
-__device__ __forceinline__ void two_row_dots(const T* w0, const T* w1, const float* xs, int chunks, const Deal& d, float& s0, float& s1) {
-    constexpr int U = 4, E = 16 / (int)sizeof(T);
-    const uint4* p0 = reinterpret_cast<const uint4*>(w0);
-    const uint4* p1 = reinterpret_cast<const uint4*>(w1);
-    s0 = s1 = 0.f;
-    for (int c = d.at; c < chunks; c += U * d.lanes) {
-        uint4 a[U], b[U];
+__device__ __forceinline__ void use_pair(const Pair& p, const float* xs, int c, int lanes, int chunks, float& s0, float& s1) {
+    constexpr int E = 16 / (int)sizeof(T);
 #pragma unroll
-        for (int u = 0; u < U; u++) {
-            const int cc = min(c + u * d.lanes, chunks - 1);
-            a[u] = p0[cc];
-            b[u] = p1[cc];
-        }
-#pragma unroll
-        for (int u = 0; u < U; u++) {
-            const int cc = c + u * d.lanes;
-            if (cc < chunks) {
-                s0 += dot16(a[u], xs + cc * E, static_cast<T*>(nullptr));
-                s1 += dot16(b[u], xs + cc * E, static_cast<T*>(nullptr));
-            }
+    for (int u = 0; u < kAhead; u++) {
+        const int cc = c + u * lanes;
+        if (cc < chunks) {
+            s0 += dot16(p.a[u], xs + cc * E, static_cast<T*>(nullptr));
+            s1 += dot16(p.b[u], xs + cc * E, static_cast<T*>(nullptr));
         }
     }
-    s0 = dense_wave_sum(s0, d.lanes);
-    s1 = dense_wave_sum(s1, d.lanes);
 }
+
+// The lane group's share of `pairs` row pairs: rows(n) names pair n, emit(n, s0, s1) gets the dot products with xs (LDS,
+// zero-padded to whole chunks).  The loads run one step ahead; `ahead` holds the first one's, requested by
+// request_first before the caller's prologue.
+template <typename Rows>
+__device__ __forceinline__ void request_first(Pair& ahead, Rows rows, int pairs, int chunks, const Deal& d) {
+    if (d.group < pairs) load_pair(ahead, rows(d.group), d.at, d.lanes, chunks);
+}
+template <typename T, typename Rows, typename Emit>
+__device__ __forceinline__ void stream_pairs(Pair& ahead, Rows rows, Emit emit, int pairs, const float* xs, int chunks, const Deal& d) {
+    const int per_step = kAhead * d.lanes, steps = (chunks + per_step - 1) / per_step;
+    for (int n = d.group; n < pairs; n += d.groups) {
+        float s0 = 0.f, s1 = 0.f;
+        for (int step = 0; step < steps; step++) {
+            const int c = d.at + step * per_step;
+            const Pair now = ahead;
+            if (step + 1 < steps)
+                load_pair(ahead, rows(n), c + per_step, d.lanes, chunks);
+            else if (n + d.groups < pairs)
+                load_pair(ahead, rows(n + d.groups), d.at, d.lanes, chunks);
+            use_pair<T>(now, xs, c, d.lanes, chunks, s0, s1);
+        }
+        s0 = dense_wave_sum(s0, d.lanes);
+        s1 = dense_wave_sum(s1, d.lanes);
+        if (d.at == 0) emit(n, s0, s1);
+    }
+}
+// Rows 2 n and 2 n + 1 of a plain matrix.
+template <typename T>
+struct PlainRows {
+    const T* w;
+    int ld, N;
+    __device__ RowPair operator()(int n) const { return {w + (size_t)(2 * n) * ld, w + (size_t)min(2 * n + 1, N - 1) * ld}; }
+};
+struct PlainEmit {
+    float* C;
+    int N;
+    float factor;
+    __device__ void operator()(int n, float s0, float s1) const {
+        C[2 * n] = s0 * factor;
+        if (2 * n + 1 < N) C[2 * n + 1] = s1 * factor;
+    }
+};
 
 // xs[0 .. padded) = f(i), zero from n on
 template <typename F>
@@ -78,50 +128,107 @@ __device__ __forceinline__ void fill_row(float* xs, int n, int padded, F f) {
     for (int i = threadIdx.x; i < padded; i += kThreads) xs[i] = i < n ? f(i) : 0.f;
 }
 
-// The residual step and the norm of RowStep into xs; workgroup 0 of the launch also writes the stream.
-template <typename T>
-__device__ __forceinline__ void row_step(const RowStep& p, float* xs, int padded, float* inv, float* red) {
-    const int t = threadIdx.x, W = p.width;
-    const bool writer = blockIdx.x == 0 && blockIdx.y == 0;
-    if (p.y) {
-        group_inverse_rms<kThreads>([&](int i) { return p.y[i]; }, W, p.norm_y.groups, p.norm_y.eps, inv, red);
+// xs[0 .. padded) = src[0 .. n), zero from n on; sixteen bytes per load where the row is made of whole float4s
+__device__ __forceinline__ void copy_row(float* xs, const float* src, int n, int padded) {
+    if (((n & 3) | (int)(reinterpret_cast<uintptr_t>(src) & 15)) == 0) {
+#pragma unroll 4
+        for (int i = 4 * threadIdx.x; i < n; i += 4 * kThreads) store4(xs + i, load4(src + i));
+        for (int i = n + threadIdx.x; i < padded; i += kThreads) xs[i] = 0.f;
+    } else {
+        fill_row(xs, n, padded, [&](int i) { return src[i]; });
     }
-    const float coef = p.before ? *p.coef : 0.f;
-    const int size_y = p.y ? W / p.norm_y.groups : 1;
-    for (int i = t; i < padded; i += kThreads) {
-        float r = 0.f;
-        if (i < W) {
-            r = p.x[i];
-            if (p.y) r += p.y[i] * inv[i / size_y] * p.norm_y.w[i];
-            if (writer && p.state) p.state[i] = r;
-            if (p.before) r = fmaf(coef, r, p.before[i]);
-            if (writer && p.x_out) p.x_out[i] = r;
-        }
-        xs[i] = r;
-    }
-    __syncthreads();
-    group_inverse_rms<kThreads>([&](int i) { return xs[i]; }, W, p.norm_h.groups, p.norm_h.eps, inv, red);
-    const int size_h = W / p.norm_h.groups;
-    for (int i = t; i < W; i += kThreads) xs[i] = xs[i] * inv[i / size_h] * p.norm_h.w[i];
-    __syncthreads();
 }
+
+// The residual step and the norm of RowStep into xs; workgroup 0 of the launch also writes the stream.  Rows whose parts
+// are whole float4s and fit four of them per thread are requested at once by load() and stay in registers (a part's
+// threads are neighbours); other rows are read when they are needed.
+class StepRow {
+   public:
+    __device__ __forceinline__ explicit StepRow(const RowStep& p) : p_(p), parts_(p.width, p.norm_h.groups), fast_(parts_.fits()) {}
+    __device__ __forceinline__ void load() {
+        if (!fast_) return;
+#pragma unroll
+        for (int k = 0; k < kParts; k++) {
+            const int i = parts_.place(k);
+            const bool in = i >= 0;
+            const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+            x_[k] = in ? load4(p_.x + i) : zero;
+            y_[k] = in && p_.y ? load4(p_.y + i) : zero;
+            wy_[k] = in && p_.y ? load4(p_.norm_y.w + i) : zero;
+            before_[k] = in && p_.before ? load4(p_.before + i) : zero;
+            wh_[k] = in ? load4(p_.norm_h.w + i) : zero;
+        }
+    }
+    __device__ __forceinline__ void finish(float* xs, int padded, float* inv, float* red) {
+        if (!fast_) return slow(xs, padded, inv, red);
+        const bool writer = blockIdx.x == 0 && blockIdx.y == 0;
+        const float coef = p_.before ? *p_.coef : 1.f;
+        const float inv_y = p_.y ? parts_.inverse_rms(y_, p_.norm_y.eps, red) : 0.f;
+#pragma unroll
+        for (int k = 0; k < kParts; k++) {
+            const int i = parts_.place(k);
+            float4 r = add4(x_[k], scale4(y_[k], inv_y, wy_[k]));
+            if (i >= 0 && writer && p_.state) store4(p_.state + i, r);
+            if (p_.before) r = fma4(coef, r, before_[k]);
+            if (i >= 0 && writer && p_.x_out) store4(p_.x_out + i, r);
+            x_[k] = r;
+        }
+        const float inv_h = parts_.inverse_rms(x_, p_.norm_h.eps, red);
+#pragma unroll
+        for (int k = 0; k < kParts; k++) {
+            const int i = parts_.place(k);
+            if (i >= 0) store4(xs + i, scale4(x_[k], inv_h, wh_[k]));
+        }
+        for (int i = p_.width + threadIdx.x; i < padded; i += kThreads) xs[i] = 0.f;
+        dense_lds_barrier();
+    }
+
+   private:
+    static constexpr int kParts = RowParts<kThreads>::kParts;
+    __device__ void slow(float* xs, int padded, float* inv, float* red) const {
+        const RowStep& p = p_;
+        const int t = threadIdx.x, W = p.width;
+        const bool writer = blockIdx.x == 0 && blockIdx.y == 0;
+        if (p.y) group_inverse_rms<kThreads>([&](int i) { return p.y[i]; }, W, p.norm_y.groups, p.norm_y.eps, inv, red);
+        const float coef = p.before ? *p.coef : 0.f;
+        const int size_y = p.y ? W / p.norm_y.groups : 1;
+        for (int i = t; i < padded; i += kThreads) {
+            float r = 0.f;
+            if (i < W) {
+                r = p.x[i];
+                if (p.y) r += p.y[i] * inv[i / size_y] * p.norm_y.w[i];
+                if (writer && p.state) p.state[i] = r;
+                if (p.before) r = fmaf(coef, r, p.before[i]);
+                if (writer && p.x_out) p.x_out[i] = r;
+            }
+            xs[i] = r;
+        }
+        __syncthreads();
+        group_inverse_rms<kThreads>([&](int i) { return xs[i]; }, W, p.norm_h.groups, p.norm_h.eps, inv, red);
+        const int size_h = W / p.norm_h.groups;
+        for (int i = t; i < W; i += kThreads) xs[i] = xs[i] * inv[i / size_h] * p.norm_h.w[i];
+        __syncthreads();
+    }
+    const RowStep& p_;
+    RowParts<kThreads> parts_;
+    bool fast_;
+    float4 x_[kParts], y_[kParts], wy_[kParts], before_[kParts], wh_[kParts];
+};
 
 // C[n] = W[n] . row
 template <typename T>
 __global__ __launch_bounds__(kThreads) void gemv_step_kernel(RowStep p, const T* __restrict__ w, int ld, int N, float* __restrict__ C) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     float *xs = smem, *red = xs + ld, *inv = red + kThreads / 64;
-    row_step<T>(p, xs, ld, inv, red);
-    const int chunks = ld * (int)sizeof(T) / 16;
-    const Deal d = deal_rows<T>(chunks);
-    for (int n = 2 * d.group; n < N; n += 2 * d.groups) {
-        float s0, s1;
-        two_row_dots<T>(w + (size_t)n * ld, w + (size_t)min(n + 1, N - 1) * ld, xs, chunks, d, s0, s1);
-        if (d.at == 0) {
-            C[n] = s0;
-            if (n + 1 < N) C[n + 1] = s1;
-        }
-    }
+    StepRow row(p);
+    row.load();
+    const int chunks = ld * (int)sizeof(T) / 16, pairs = (N + 1) / 2;
+    const Deal d = deal_rows<T>(chunks, gridDim.x);
+    const PlainRows<T> rows{w, ld, N};
+    Pair ahead;
+    request_first(ahead, rows, pairs, chunks, d);
+    row.finish(xs, ld, inv, red);
+    stream_pairs<T>(ahead, rows, PlainEmit{C, N, 1.f}, pairs, xs, chunks, d);
 }
 
 // C[n] = W[n] . x
@@ -129,18 +236,14 @@ template <typename T>
 __global__ __launch_bounds__(kThreads) void gemv_plain_kernel(const float* __restrict__ x, int K, const T* __restrict__ w, int ld, int N,
                                                              float* __restrict__ C) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
-    fill_row(smem, K, ld, [&](int i) { return x[i]; });
-    __syncthreads();
-    const int chunks = ld * (int)sizeof(T) / 16;
-    const Deal d = deal_rows<T>(chunks);
-    for (int n = 2 * d.group; n < N; n += 2 * d.groups) {
-        float s0, s1;
-        two_row_dots<T>(w + (size_t)n * ld, w + (size_t)min(n + 1, N - 1) * ld, smem, chunks, d, s0, s1);
-        if (d.at == 0) {
-            C[n] = s0;
-            if (n + 1 < N) C[n + 1] = s1;
-        }
-    }
+    const int chunks = ld * (int)sizeof(T) / 16, pairs = (N + 1) / 2;
+    const Deal d = deal_rows<T>(chunks, gridDim.x);
+    const PlainRows<T> rows{w, ld, N};
+    Pair ahead;
+    request_first(ahead, rows, pairs, chunks, d);
+    copy_row(smem, x, K, ld);
+    dense_lds_barrier();
+    stream_pairs<T>(ahead, rows, PlainEmit{C, N, 1.f}, pairs, smem, chunks, d);
 }
 
 // Queries from their normed latent.  The last workgroups of the launch do other work of the same stage: one appends the
@@ -177,20 +280,23 @@ __global__ __launch_bounds__(kThreads) void gemv_query_kernel(LatentRows in, Lat
         }
         return;
     }
-    group_inverse_rms<kThreads>([&](int i) { return in.down[i]; }, sh.q_rank, 1, in.eps, inv, red);
-    fill_row(xs, sh.q_rank, ld, [&](int i) { return in.down[i] * inv[0] * in.q_norm[i]; });
-    __syncthreads();
-    const int chunks = ld * (int)sizeof(T) / 16;
-    Deal d = deal_rows<T>(chunks);
-    d.groups = main_groups * (kThreads / d.lanes);
-    for (int n = 2 * d.group; n < N; n += 2 * d.groups) {
-        float s0, s1;
-        two_row_dots<T>(w + (size_t)n * ld, w + (size_t)min(n + 1, N - 1) * ld, xs, chunks, d, s0, s1);
-        if (d.at == 0) {
-            q[n] = s0;
-            if (n + 1 < N) q[n + 1] = s1;
-        }
-    }
+    const int chunks = ld * (int)sizeof(T) / 16, pairs = (N + 1) / 2;
+    const Deal d = deal_rows<T>(chunks, main_groups);
+    const PlainRows<T> rows{w, ld, N};
+    Pair ahead;
+    request_first(ahead, rows, pairs, chunks, d);
+    fill_row(xs, sh.q_rank, ld, [&](int i) { return in.down[i]; });
+    float sum = 0.f;  // of this thread's own elements
+    for (int i = t; i < sh.q_rank; i += kThreads) sum = fmaf(xs[i], xs[i], sum);
+    sum = dense_wave_sum(sum);
+    if ((t & 63) == 0) red[t >> 6] = sum;
+    dense_lds_barrier();
+    sum = 0.f;
+    for (int k = 0; k < kThreads / 64; k++) sum += red[k];
+    const float scale = 1.0f / sqrtf(sum / (float)sh.q_rank + in.eps);
+    for (int i = t; i < sh.q_rank; i += kThreads) xs[i] *= scale * in.q_norm[i];
+    dense_lds_barrier();
+    stream_pairs<T>(ahead, rows, PlainEmit{q, N, 1.f}, pairs, xs, chunks, d);
 }
 
 // Query rows in latent space, one head per blockIdx.y: columns 0..rank from the unrotated part through the transposed key
@@ -211,43 +317,83 @@ __global__ __launch_bounds__(kThreads) void gemv_absorb_kernel(const float* __re
             dst[sh.rank + half + j] = (T)(v * cs + u * sn);
         }
     }
-    fill_row(smem, sh.dim, ld, [&](int i) { return src[i]; });
-    __syncthreads();
-    const T* w = uk_t + (size_t)h * sh.rank * ld;
-    const int chunks = ld * (int)sizeof(T) / 16, N = sh.rank;
-    const Deal d = deal_rows<T>(chunks);
-    for (int n = 2 * d.group; n < N; n += 2 * d.groups) {
-        float s0, s1;
-        two_row_dots<T>(w + (size_t)n * ld, w + (size_t)min(n + 1, N - 1) * ld, smem, chunks, d, s0, s1);
-        if (d.at == 0) {
-            dst[n] = (T)s0;
-            if (n + 1 < N) dst[n + 1] = (T)s1;
-        }
-    }
+    const int N = sh.rank, chunks = ld * (int)sizeof(T) / 16, pairs = (N + 1) / 2;
+    const Deal d = deal_rows<T>(chunks, gridDim.x);
+    const PlainRows<T> rows{uk_t + (size_t)h * N * ld, ld, N};
+    Pair ahead;
+    request_first(ahead, rows, pairs, chunks, d);
+    copy_row(smem, src, sh.dim, ld);
+    dense_lds_barrier();
+    stream_pairs<T>(
+        ahead, rows,
+        [&](int n, float s0, float s1) {
+            dst[2 * n] = (T)s0;
+            if (2 * n + 1 < N) dst[2 * n + 1] = (T)s1;
+        },
+        pairs, smem, chunks, d);
 }
 
-// Values of a head (blockIdx.y) from its weighted latent, times the head's gate.
+// Values of a head (blockIdx.y) from its weighted latent, times the head's gate.  The latent is a row of o_lat, or is
+// merged here from the shares of the attention: sum_k w_k share_k / sum_k w_k sum_k, w_k = 2^(maximum_k - largest).
 template <typename T>
-__global__ __launch_bounds__(kThreads) void gemv_values_kernel(const float* __restrict__ o_lat, int ld_o, LatentShape sh,
-                                                              const T* __restrict__ uv, int ld, const float* __restrict__ gates,
-                                                              float* __restrict__ attn) {
+__global__ __launch_bounds__(kThreads) void gemv_values_kernel(const float* __restrict__ o_lat, int ld_o, LatentShares shares,
+                                                              LatentShape sh, const T* __restrict__ uv, int ld,
+                                                              const float* __restrict__ gates, float* __restrict__ attn) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
-    const int h = blockIdx.y;
-    const float* src = o_lat + (size_t)h * ld_o;
-    fill_row(smem, sh.rank, ld, [&](int i) { return src[i]; });
-    __syncthreads();
-    const T* w = uv + (size_t)h * sh.vdim * ld;
+    __shared__ float weight[kAttendMaxSplits];
+    const int h = blockIdx.y, t = threadIdx.x;
+    const int N = sh.vdim, chunks = ld * (int)sizeof(T) / 16, pairs = (N + 1) / 2;
+    const Deal d = deal_rows<T>(chunks, gridDim.x);
+    const PlainRows<T> rows{uv + (size_t)h * N * ld, ld, N};
     const float gate = sigmoid(gates[h]);
-    const int chunks = ld * (int)sizeof(T) / 16, N = sh.vdim;
-    const Deal d = deal_rows<T>(chunks);
-    for (int n = 2 * d.group; n < N; n += 2 * d.groups) {
-        float s0, s1;
-        two_row_dots<T>(w + (size_t)n * ld, w + (size_t)min(n + 1, N - 1) * ld, smem, chunks, d, s0, s1);
-        if (d.at == 0) {
-            attn[(size_t)h * N + n] = s0 * gate;
-            if (n + 1 < N) attn[(size_t)h * N + n + 1] = s1 * gate;
+    Pair ahead;
+    if (shares.part) {
+        // a thread takes four columns of every `teams`-th share; the teams' sums meet in LDS.  Requested in the order of use.
+        constexpr int U = 16;
+        const int n = shares.splits, quads = shares.ld >> 2, teams = max(1, kThreads / quads);
+        const int l63 = min(t & 63, n - 1);
+        const float maximum = shares.stats[2 * ((size_t)l63 * sh.heads + h)], total = shares.stats[2 * ((size_t)l63 * sh.heads + h) + 1];
+        const float* part = shares.part + (size_t)h * shares.ld;
+        const size_t step = (size_t)sh.heads * shares.ld;
+        float4 v[U];
+        auto request = [&](int q, int k) {
+#pragma unroll
+            for (int u = 0; u < U; u++) v[u] = load4(part + min(k + u * teams, n - 1) * step + 4 * (q % quads));
+        };
+        if (t < quads * teams) request(t, t / quads);
+        request_first(ahead, rows, pairs, chunks, d);
+        {   // every wave forms the shares' weights
+            const bool real = (t & 63) < n;
+            const float largest = dense_wave_max(real ? maximum : -3.402823466e38f), w = real ? exp2f(maximum - largest) : 0.f;
+            const float all = dense_wave_sum(w * total);
+            if (t < 64) weight[t] = w / all;
         }
+        dense_lds_barrier();
+        float* sums = smem + ld;
+        for (int q = t; q < quads * teams; q += kThreads) {
+            const int team = q / quads;
+            if (q != t) request(q, team);
+            float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
+            for (int k = team; k < n; k += U * teams) {
+                if (k != team) request(q, k);
+#pragma unroll
+                for (int u = 0; u < U; u++)
+                    if (k + u * teams < n) s = fma4(weight[k + u * teams], v[u], s);
+            }
+            store4(sums + team * shares.ld + 4 * (q % quads), s);
+        }
+        dense_lds_barrier();
+        fill_row(smem, sh.rank, ld, [&](int i) {
+            float s = 0.f;
+            for (int k = 0; k < teams; k++) s += sums[k * shares.ld + i];
+            return s;
+        });
+    } else {
+        request_first(ahead, rows, pairs, chunks, d);
+        copy_row(smem, o_lat + (size_t)h * ld_o, sh.rank, ld);
     }
+    dense_lds_barrier();
+    stream_pairs<T>(ahead, rows, PlainEmit{attn + (size_t)h * N, N, gate}, pairs, smem, chunks, d);
 }
 
 __device__ __forceinline__ int expert_of(const ExpertRows& e, int slot) {
@@ -261,19 +407,22 @@ __global__ __launch_bounds__(kThreads) void gemv_gate_up_kernel(RowStep p, Exper
                                                                const T* __restrict__ dense, int ld, float* __restrict__ act) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     float *xs = smem, *red = xs + ld, *inv = red + kThreads / 64;
+    StepRow row(p);
+    row.load();
     const int slot = blockIdx.y;
     const T* w = slot < e.top ? experts + (size_t)expert_of(e, slot) * e.pair_rows * ld : dense;
     const int ff = slot < e.top ? e.ff : e.dense_ff;
-    row_step<T>(p, xs, ld, inv, red);
     const int chunks = ld * (int)sizeof(T) / 16;
-    const Deal d = deal_rows<T>(chunks);
+    const Deal d = deal_rows<T>(chunks, gridDim.x);
+    auto rows = [&](int j) {  // the gate and the up row of column j
+        const T* r = w + (size_t)((j >> 4) * 32 + (j & 15)) * ld;
+        return RowPair{r, r + (size_t)16 * ld};
+    };
+    Pair ahead;
+    request_first(ahead, rows, ff, chunks, d);
+    row.finish(xs, ld, inv, red);
     float* dst = act + (size_t)slot * e.ld_act;
-    for (int j = d.group; j < ff; j += d.groups) {
-        const T* row = w + (size_t)((j >> 4) * 32 + (j & 15)) * ld;
-        float gate, up;
-        two_row_dots<T>(row, row + (size_t)16 * ld, xs, chunks, d, gate, up);
-        if (d.at == 0) dst[j] = silu(gate) * up;
-    }
+    stream_pairs<T>(ahead, rows, [&](int j, float gate, float up) { dst[j] = silu(gate) * up; }, ff, xs, chunks, d);
 }
 
 // y[n] = mean over the token's experts of W_e[n] . act_e, plus the dense or shared feed-forward's.
@@ -283,45 +432,67 @@ __global__ __launch_bounds__(kThreads) void gemv_ff_down_kernel(ExpertRows e, co
                                                                float* __restrict__ y) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     __shared__ int chosen[64];
-    for (int k = 0; k < e.top; k++) fill_row(smem + k * ld, e.ff, ld, [&](int i) { return act[(size_t)k * e.ld_act + i]; });
+    const int chunks = ld * (int)sizeof(T) / 16, chunks_dense = ld_dense * (int)sizeof(T) / 16, pairs = (N + 1) / 2;
     float* xs_dense = smem + e.top * ld;
-    if (e.dense_ff) fill_row(xs_dense, e.dense_ff, ld_dense, [&](int i) { return act[(size_t)e.top * e.ld_act + i]; });
+    auto fill = [&]() {
+        for (int k = 0; k < e.top; k++) copy_row(smem + k * ld, act + (size_t)k * e.ld_act, e.ff, ld);
+        if (e.dense_ff) copy_row(xs_dense, act + (size_t)e.top * e.ld_act, e.dense_ff, ld_dense);
+    };
+    if (!e.top) {
+        const Deal d = deal_rows<T>(chunks_dense, gridDim.x);
+        const PlainRows<T> rows{dense, ld_dense, N};
+        Pair ahead;
+        request_first(ahead, rows, pairs, chunks_dense, d);
+        fill();
+        dense_lds_barrier();
+        stream_pairs<T>(ahead, rows, PlainEmit{y, N, 1.f}, pairs, xs_dense, chunks_dense, d);
+        return;
+    }
+    // a pair of rows of every expert in turn, then of the shared feed-forward; the loads run one step ahead
+    const Deal d = deal_rows<T>(chunks, gridDim.x);
     if ((int)threadIdx.x < e.top) chosen[threadIdx.x] = expert_of(e, threadIdx.x);
+    fill();
     __syncthreads();
-    const int chunks = ld * (int)sizeof(T) / 16, chunks_dense = ld_dense * (int)sizeof(T) / 16;
-    const Deal d = deal_rows<T>(e.dense_ff ? chunks_dense : chunks);
-    const float share = 1.0f / (float)max(e.top, 1);
-    for (int n = 2 * d.group; n < N; n += 2 * d.groups) {
-        const int n1 = min(n + 1, N - 1);
-        float a0 = 0.f, a1 = 0.f, s0, s1;
-        for (int k = 0; k < e.top; k++) {
-            const T* w = experts + (size_t)chosen[k] * N * ld;
-            two_row_dots<T>(w + (size_t)n * ld, w + (size_t)n1 * ld, smem + k * ld, chunks, d, s0, s1);
-            a0 += s0;
-            a1 += s1;
+    const int parts = e.top + (e.dense_ff ? 1 : 0), per_step = kAhead * d.lanes;
+    const float share = 1.0f / (float)e.top;
+    auto rows_of = [&](int n, int k) {
+        return k < e.top ? PlainRows<T>{experts + (size_t)chosen[k] * N * ld, ld, N}(n) : PlainRows<T>{dense, ld_dense, N}(n);
+    };
+    Pair ahead;
+    if (d.group < pairs) load_pair(ahead, rows_of(d.group, 0), d.at, d.lanes, chunks);
+    for (int n = d.group; n < pairs; n += d.groups) {
+        float a0 = 0.f, a1 = 0.f;
+        for (int k = 0; k < parts; k++) {
+            const bool expert = k < e.top;
+            const int all = expert ? chunks : chunks_dense, steps = (all + per_step - 1) / per_step;
+            const float* xs = expert ? smem + k * ld : xs_dense;
+            float s0 = 0.f, s1 = 0.f;
+            for (int step = 0; step < steps; step++) {
+                const int c = d.at + step * per_step;
+                const Pair now = ahead;
+                if (step + 1 < steps)
+                    load_pair(ahead, rows_of(n, k), c + per_step, d.lanes, all);
+                else if (k + 1 < parts)
+                    load_pair(ahead, rows_of(n, k + 1), d.at, d.lanes, k + 1 < e.top ? chunks : chunks_dense);
+                else if (n + d.groups < pairs)
+                    load_pair(ahead, rows_of(n + d.groups, 0), d.at, d.lanes, chunks);
+                use_pair<T>(now, xs, c, d.lanes, all, s0, s1);
+            }
+            a0 = fmaf(expert ? share : 1.f, s0, a0);
+            a1 = fmaf(expert ? share : 1.f, s1, a1);
         }
-        a0 *= share;
-        a1 *= share;
-        if (e.dense_ff) {
-            two_row_dots<T>(dense + (size_t)n * ld_dense, dense + (size_t)n1 * ld_dense, xs_dense, chunks_dense, d, s0, s1);
-            a0 += s0;
-            a1 += s1;
-        }
-        if (d.at == 0) {
-            y[n] = a0;
-            if (n + 1 < N) y[n + 1] = a1;
-        }
+        a0 = dense_wave_sum(a0, d.lanes);
+        a1 = dense_wave_sum(a1, d.lanes);
+        if (d.at == 0) PlainEmit{y, N, 1.f}(n, a0, a1);
     }
 }
 
-// Workgroups for N rows of `ld` elements: a pair of rows per lane group and turn, at most `limit`.
+// Workgroups for N rows of `ld` elements: at most `limit`, and as many as give every lane group the same number of pairs.
 template <typename T>
 int workgroups(int N, int ld, int limit) {
-    const int chunks = ld * (int)sizeof(T) / 16;
-    int lanes = 1;
-    while (lanes < 64 && 2 * lanes <= chunks) lanes <<= 1;
-    const int per_wg = 2 * (kThreads / lanes), n = (N + per_wg - 1) / per_wg;
-    return n < 1 ? 1 : n > limit ? limit : n;
+    const int per_wg = kThreads / lanes_of(ld * (int)sizeof(T) / 16), pairs = (N + 1) / 2;
+    const int rounds = (pairs + per_wg * limit - 1) / (per_wg * limit);
+    return (pairs + per_wg * rounds - 1) / (per_wg * rounds);
 }
 constexpr int kMaxGrid = 1024;
 
@@ -358,10 +529,12 @@ hipError_t launch_gemv_absorb(const float* q, const LatentRows& in, const Latent
     return hipGetLastError();
 }
 template <typename T>
-hipError_t launch_gemv_values(const float* o_lat, int ld_o, const LatentShape& sh, const T* uv, int ld, const float* gates, float* attn,
-                              hipStream_t s) {
-    hipLaunchKernelGGL(gemv_values_kernel<T>, dim3(workgroups<T>(sh.vdim, ld, 64), sh.heads), dim3(kThreads), ld * sizeof(float), s, o_lat,
-                       ld_o, sh, uv, ld, gates, attn);
+hipError_t launch_gemv_values(const float* o_lat, int ld_o, const LatentShares& shares, const LatentShape& sh, const T* uv, int ld,
+                              const float* gates, float* attn, hipStream_t s) {
+    // every workgroup of a head repeats the merge of its shares
+    const int teams = shares.part ? (kThreads * 4 > shares.ld ? kThreads * 4 / shares.ld : 1) : 0;
+    hipLaunchKernelGGL(gemv_values_kernel<T>, dim3(workgroups<T>(sh.vdim, ld, shares.part ? 4 : 64), sh.heads), dim3(kThreads),
+                       (ld + teams * shares.ld) * sizeof(float), s, o_lat, ld_o, shares, sh, uv, ld, gates, attn);
     return hipGetLastError();
 }
 template <typename T>
@@ -387,8 +560,8 @@ hipError_t launch_gemv_ff_down(const ExpertRows& e, const float* act, const T* e
     template hipError_t launch_gemv_query<T>(const LatentRows&, const LatentShape&, const T*, int, float*, T*, const DepthAverage&, \
                                              int, float*, hipStream_t);                                                           \
     template hipError_t launch_gemv_absorb<T>(const float*, const LatentRows&, const LatentShape&, const T*, int, T*, hipStream_t); \
-    template hipError_t launch_gemv_values<T>(const float*, int, const LatentShape&, const T*, int, const float*, float*,          \
-                                              hipStream_t);                                                                       \
+    template hipError_t launch_gemv_values<T>(const float*, int, const LatentShares&, const LatentShape&, const T*, int,           \
+                                              const float*, float*, hipStream_t);                                                                       \
     template hipError_t launch_gemv_gate_up<T>(const RowStep&, const ExpertRows&, const T*, const T*, int, float*, hipStream_t);   \
     template hipError_t launch_gemv_ff_down<T>(const ExpertRows&, const float*, const T*, int, const T*, int, int, float*,         \
                                                hipStream_t);

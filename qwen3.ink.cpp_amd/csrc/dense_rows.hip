@@ -21,8 +21,9 @@ __global__ __launch_bounds__(kThreads) void group_norm_kernel(const float* __res
     for (int i = threadIdx.x; i < width; i += kThreads) dst[i] = (T)(row[i] * inv[i / size] * norm.w[i]);
 }
 
+// Any sizes.
 template <typename T>
-__global__ __launch_bounds__(kThreads) void residual_norm_kernel(const float* x, SublayerOut y, GroupNorm norm_y, DepthAverage depth,
+__global__ __launch_bounds__(kThreads) void residual_norm_any_kernel(const float* x, SublayerOut y, GroupNorm norm_y, DepthAverage depth,
                                                                 float* x_out, GroupNorm norm_h, T* __restrict__ h, int ld_h,
                                                                 int width) {
     extern __shared__ float smem[];
@@ -68,22 +69,99 @@ __global__ __launch_bounds__(kThreads) void residual_norm_kernel(const float* x,
     for (int i = t; i < width; i += kThreads) dst[i] = (T)(v[i] * inv[i / size_h] * norm_h.w[i]);
 }
 
-// Exclusive prefix sum of a[0..n) in place, total returned to every thread; 1024 threads.
+// The same for rows that RowParts can hold: every operand is read once, sixteen bytes at a time, and the row stays in
+// registers between the two norms.
+template <typename T>
+__global__ __launch_bounds__(kThreads) void residual_norm_kernel(const float* x, SublayerOut y, GroupNorm norm_y, DepthAverage depth,
+                                                                float* x_out, GroupNorm norm_h, T* __restrict__ h, int ld_h,
+                                                                int width) {
+    constexpr int P = RowParts<kThreads>::kParts;
+    __shared__ float red[kThreads / 64];
+    const RowParts<kThreads> parts(width, norm_h.groups);
+    const size_t m = blockIdx.x, base = m * width;
+    const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+    float4 r[P], v[P];
+#pragma unroll
+    for (int k = 0; k < P; k++) {
+        const int i = parts.place(k);
+        r[k] = i >= 0 ? load4(x + base + i) : zero;
+        v[k] = zero;
+        if (i < 0 || !y.y) continue;
+        if (y.slot_rows) {
+            for (int s = 0; s < y.top; s++) v[k] = add4(v[k], load4(y.y + (size_t)y.slot_rows[m * y.top + s] * width + i));
+            v[k] = fma4(1.0f / (float)y.top, v[k], y.shared ? load4(y.shared + base + i) : zero);
+        } else {
+            v[k] = load4(y.y + base + i);
+        }
+    }
+    if (y.y) {
+        const float inv = parts.inverse_rms(v, norm_y.eps, red);
+#pragma unroll
+        for (int k = 0; k < P; k++) {
+            const int i = parts.place(k);
+            if (i >= 0) r[k] = add4(r[k], scale4(v[k], inv, load4(norm_y.w + i)));
+        }
+    }
+    if (depth.states) {
+#pragma unroll
+        for (int k = 0; k < P; k++) {
+            const int i = parts.place(k);
+            v[k] = zero;
+            if (i < 0) continue;
+            store4(depth.states + depth.n * depth.state_step + base + i, r[k]);
+            const float* st = depth.states + base + i;
+            int j = 0;
+            for (; j + 4 <= depth.n; j += 4) {
+                float4 a[4];
+#pragma unroll
+                for (int u = 0; u < 4; u++) a[u] = load4(st + (j + u) * depth.state_step);
+#pragma unroll
+                for (int u = 0; u < 4; u++) v[k] = fma4(depth.coef[j + u], a[u], v[k]);
+            }
+            for (; j < depth.n; j++) v[k] = fma4(depth.coef[j], load4(st + j * depth.state_step), v[k]);
+            r[k] = fma4(depth.coef[depth.n], r[k], v[k]);
+        }
+    }
+#pragma unroll
+    for (int k = 0; k < P; k++) {
+        const int i = parts.place(k);
+        if (i >= 0) store4(x_out + base + i, r[k]);
+    }
+    const float inv = parts.inverse_rms(r, norm_h.eps, red);
+#pragma unroll
+    for (int k = 0; k < P; k++) {
+        const int i = parts.place(k);
+        if (i < 0) continue;
+        const float4 o = scale4(r[k], inv, load4(norm_h.w + i));
+        T* dst = h + m * ld_h + i;  // i and the row stride are multiples of 4
+        alignas(16) T packed[4] = {(T)o.x, (T)o.y, (T)o.z, (T)o.w};
+        if constexpr (sizeof(T) == 2)
+            *reinterpret_cast<uint2*>(dst) = *reinterpret_cast<const uint2*>(packed);
+        else
+            *reinterpret_cast<uint4*>(dst) = *reinterpret_cast<const uint4*>(packed);
+    }
+}
+
+// Exclusive prefix sum of a[0..n) in place, total returned to every thread; 1024 threads, tmp: 16 ints of LDS.
 __device__ int block_exclusive_scan(int* a, int n, int* tmp) {
-    const int t = threadIdx.x;
+    const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
     int carry = 0;
     for (int base = 0; base < n; base += 1024) {
         const int own = base + t < n ? a[base + t] : 0;
-        tmp[t] = own;
-        __syncthreads();
-        for (int off = 1; off < 1024; off <<= 1) {
-            const int add = t >= off ? tmp[t - off] : 0;
-            __syncthreads();
-            tmp[t] += add;
-            __syncthreads();
+        int upto = own;
+        for (int off = 1; off < 64; off <<= 1) {
+            const int add = __shfl_up(upto, off, 64);
+            if (lane >= off) upto += add;
         }
-        if (base + t < n) a[base + t] = carry + tmp[t] - own;
-        carry += tmp[1023];
+        if (lane == 63) tmp[wave] = upto;
+        __syncthreads();
+        int before = 0, all = 0;
+        for (int w = 0; w < 16; w++) {
+            if (w < wave) before += tmp[w];
+            all += tmp[w];
+        }
+        if (base + t < n) a[base + t] = carry + before + upto - own;
+        carry += all;
         __syncthreads();
     }
     return carry;
@@ -93,7 +171,7 @@ __global__ __launch_bounds__(1024) void table_route_kernel(const int* __restrict
                                                          int top, int experts, int M, int* __restrict__ src_rows,
                                                          int* __restrict__ slot_rows, GroupTile* __restrict__ tiles,
                                                          int* __restrict__ n_tiles) {
-    extern __shared__ int cnt[];  // [experts] counts, [experts] first rows, [experts] first tiles, [1024]
+    extern __shared__ int cnt[];  // [experts] counts, [experts] first rows, [experts] first tiles, [16]
     int *first = cnt + experts, *tile0 = first + experts, *tmp = tile0 + experts;
     const int t = threadIdx.x, total = M * top;
     for (int e = t; e < experts; e += 1024) cnt[e] = 0;
@@ -102,7 +180,18 @@ __global__ __launch_bounds__(1024) void table_route_kernel(const int* __restrict
         const int id = min(max(ids[i / top], 0), vocab - 1);
         return min(max(table[(size_t)id * top + i % top], 0), experts - 1);
     };
-    for (int i = t; i < total; i += 1024) atomicAdd(&cnt[expert_of(i)], 1);
+    constexpr int U = 4;
+    for (int i0 = t; i0 < total; i0 += U * 1024) {  // slot_rows keeps the expert until the row is known
+        int e[U];
+#pragma unroll
+        for (int u = 0; u < U; u++) e[u] = i0 + u * 1024 < total ? expert_of(i0 + u * 1024) : 0;
+#pragma unroll
+        for (int u = 0; u < U; u++)
+            if (i0 + u * 1024 < total) {
+                slot_rows[i0 + u * 1024] = e[u];
+                atomicAdd(&cnt[e[u]], 1);
+            }
+    }
     __syncthreads();
     for (int e = t; e < experts; e += 1024) {
         first[e] = cnt[e];
@@ -119,10 +208,17 @@ __global__ __launch_bounds__(1024) void table_route_kernel(const int* __restrict
     }
     __syncthreads();
     // where a token's row lands among its expert's rows does not matter: a row's result does not depend on its place
-    for (int i = t; i < total; i += 1024) {
-        const int r = atomicAdd(&first[expert_of(i)], 1);
-        src_rows[r] = i / top;
-        slot_rows[i] = r;
+    for (int i0 = t; i0 < total; i0 += U * 1024) {
+        int e[U];
+#pragma unroll
+        for (int u = 0; u < U; u++) e[u] = i0 + u * 1024 < total ? slot_rows[i0 + u * 1024] : 0;
+#pragma unroll
+        for (int u = 0; u < U; u++)
+            if (i0 + u * 1024 < total) {
+                const int r = atomicAdd(&first[e[u]], 1);
+                src_rows[r] = (i0 + u * 1024) / top;
+                slot_rows[i0 + u * 1024] = r;
+            }
     }
 }
 
@@ -139,14 +235,22 @@ template <typename T>
 hipError_t launch_residual_norm(const float* x, const SublayerOut& y, const GroupNorm& norm_y, const DepthAverage& depth, float* x_out,
                                 const GroupNorm& norm_h, T* h, int ld_h, int M, int width, hipStream_t s) {
     const int groups = norm_y.groups > norm_h.groups ? norm_y.groups : norm_h.groups;
-    const size_t lds = (width + groups + kThreads / 64) * sizeof(float);
-    hipLaunchKernelGGL(residual_norm_kernel<T>, dim3(M), dim3(kThreads), lds, s, x, y, norm_y, depth, x_out, norm_h, h, ld_h, width);
+    int per = 1;  // what RowParts holds
+    while (per < norm_h.groups && per < kThreads) per <<= 1;
+    const int size = width / norm_h.groups;
+    if ((!y.y || norm_y.groups == norm_h.groups) && norm_h.groups <= kThreads && size % 4 == 0 &&
+        size / 4 <= RowParts<kThreads>::kParts * (kThreads / per)) {
+        hipLaunchKernelGGL(residual_norm_kernel<T>, dim3(M), dim3(kThreads), 0, s, x, y, norm_y, depth, x_out, norm_h, h, ld_h, width);
+    } else {
+        const size_t lds = (width + groups + kThreads / 64) * sizeof(float);
+        hipLaunchKernelGGL(residual_norm_any_kernel<T>, dim3(M), dim3(kThreads), lds, s, x, y, norm_y, depth, x_out, norm_h, h, ld_h, width);
+    }
     return hipGetLastError();
 }
 
 hipError_t launch_table_route(const int* ids, const int* table, int vocab, int top, int experts, int M, int* src_rows,
                               int* slot_rows, GroupTile* tiles, int* n_tiles, hipStream_t s) {
-    const size_t lds = (3 * (size_t)experts + 1024) * sizeof(int);
+    const size_t lds = (3 * (size_t)experts + 16) * sizeof(int);
     hipLaunchKernelGGL(table_route_kernel, dim3(1), dim3(1024), lds, s, ids, table, vocab, top, experts, M, src_rows, slot_rows,
                        tiles, n_tiles);
     return hipGetLastError();

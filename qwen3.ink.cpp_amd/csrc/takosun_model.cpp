@@ -402,7 +402,7 @@ int TakosunModel<T>::allocate(int max_seq) {
         if (!f.present) continue;
         act = std::max(act, (size_t)std::max(f.top, 1) * pad_k<T>(f.ff));
         act = std::max(act, (size_t)pad_k<T>(f.shared_ff));
-        ld_act_row_ = std::max(ld_act_row_, std::max(f.ff, f.shared_ff));
+        ld_act_row_ = std::max(ld_act_row_, (std::max(f.ff, f.shared_ff) + 3) / 4 * 4);
         slots = std::max(slots, f.top + 1);
         one_token_fits_ = one_token_fits_ && std::max(f.top, 1) * pad_k<T>(f.ff) + pad_k<T>(f.shared_ff) <= kGemvMaxRow;
         if (f.experts_by_table) {
@@ -592,7 +592,7 @@ int TakosunModel<T>::feed_forward_one_token(const Layer& L, const LayerConfig& l
 }
 
 // The pass for one token: the row work between two products runs inside the product that consumes it, eight launches a
-// layer (nine with the merge of the attention's shares).  The sum over the earlier states of the mean over depth is
+// layer.  The sum over the earlier states of the mean over depth is
 // formed beside the query product, so that the next layer's first product adds only the newest state.
 template <typename T>
 int TakosunModel<T>::enqueue_one_token(int n_want, hipStream_t s) {
@@ -614,19 +614,18 @@ int TakosunModel<T>::enqueue_one_token(int n_want, hipStream_t s) {
         A81W41_HIP_TRY(launch_gemv_query<T>(in, sh, L.uq.data, L.uq.ld, q_, own ? L.cache : nullptr, depth, W, before_, s));
         A81W41_HIP_TRY(launch_gemv_absorb<T>(q_, in, sh, L.uk_t.data, L.uk_t.ld, q_lat_, s));
         const int ld_rank = pad_k<T>(sh.rank);
-        bool done = false;
+        LatentShares shares;
         if constexpr (kMatrixAttention) {
             if (opt_attention_ != 1 && attend_shared_fits(sh.rank + sh.rot, sh.rank)) {
                 AttendArgs a = shared_attend(L, sh, 1);
-                a.splits = std::max(a.splits, 2);  // the shares stay fp32 until they are merged
+                a.splits = std::max(a.splits, 2);  // shares stay fp32; the product with W_uv merges them
                 A81W41_HIP_TRY(launch_attend_shared(a, s));
-                A81W41_HIP_TRY(launch_merge_shares<float>(a, o_lat_row_, ld_rank, s));
-                done = true;
+                shares = LatentShares{a.part, a.part_stats, a.splits, a.ld_part};
             }
         }
-        if (!done)
+        if (!shares.part)
             A81W41_HIP_TRY((launch_latent_attention_vector<T, float>(q_lat_, L.cache, sh, pos, max_seq(), 1, o_lat_row_, ld_rank, s)));
-        A81W41_HIP_TRY(launch_gemv_values<T>(o_lat_row_, ld_rank, sh, L.uv.data, L.uv.ld, down_ + sh.q_rank + (own ? sh.rank + sh.rot : 0),
+        A81W41_HIP_TRY(launch_gemv_values<T>(o_lat_row_, ld_rank, shares, sh, L.uv.data, L.uv.ld, down_ + sh.q_rank + (own ? sh.rank + sh.rot : 0),
                                              attn_row_, s));
         A81W41_HIP_TRY(launch_gemv_plain<T>(attn_row_, sh.heads * sh.vdim, L.o.data, L.o.ld, W, y_, s));
         step = RowStep{};

@@ -56,6 +56,11 @@ WIDE = config(300, 256, 1, [
 ])
 # latents past the matrix-core attention's sizes
 HUGE_LATENT = config(64, 64, 2, [layer(mixer(2, 8, 8, 16, 16, 640, 0.3), dense(64))])
+# rows that the row kernels hold in registers, with idle threads; and rows too long for that
+LONG_ROWS = config(43, 1100, 5, [layer(mixer(1, 8, 8, 8, 16, 24, 0.4), moe(2, 1, 16, shared=24)),
+                                 layer(mixer(1, 8, 8, 8, 16, 24, 0.4, kv_from=0), dense(40))])
+LONGER_ROWS = config(43, 4200, 1, [layer(mixer(1, 8, 8, 8, 16, 24, 0.4), dense(40)),
+                                   layer(mixer(2, 8, 8, 8, 16, 24, 0.4, kv_from=0), moe(2, 2, 16))])
 
 
 def write_model(root, cfg, weights):

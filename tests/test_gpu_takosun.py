@@ -8,11 +8,12 @@ import numpy as np
 import pytest
 
 from oracle import takosun_forward as tf
-from tests.takosun_fixture import HUGE_LATENT, ODD, SMALL, WIDE, config, dense, layer, mixer, moe, write_model
+from tests.takosun_fixture import HUGE_LATENT, LONG_ROWS, LONGER_ROWS, ODD, SMALL, WIDE, config, dense, layer, mixer, moe, write_model
 
 pytestmark = pytest.mark.gpu
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-CONFIGS = {"small": SMALL, "odd": ODD, "wide": WIDE, "huge_latent": HUGE_LATENT}
+CONFIGS = {"small": SMALL, "odd": ODD, "wide": WIDE, "huge_latent": HUGE_LATENT, "long_rows": LONG_ROWS,
+           "longer_rows": LONGER_ROWS}
 TOL = {"float32": 3e-5, "bfloat16": 0.06}
 
 
@@ -167,7 +168,8 @@ def test_formed_attention(pkg, M, heads, dim, rot, vdim, pos):
 # ---- the model -------------------------------------------------------------------------------
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name,n", [("small", 1), ("small", 2), ("small", 75), ("odd", 40), ("wide", 150), ("huge_latent", 20)])
+@pytest.mark.parametrize("name,n", [("small", 1), ("small", 2), ("small", 75), ("odd", 40), ("wide", 150), ("huge_latent", 20), ("long_rows", 9),
+                                    ("longer_rows", 9)])
 def test_whole_prompt(built, name, n, dtype):
     model, oracle, _ = built(name, dtype)
     ids, want, states = truth(name, oracle, n)
@@ -181,7 +183,7 @@ def test_whole_prompt(built, name, n, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name,n", [("small", 75), ("odd", 40), ("wide", 70), ("huge_latent", 20)])
+@pytest.mark.parametrize("name,n", [("small", 75), ("odd", 40), ("wide", 70), ("huge_latent", 20), ("long_rows", 9), ("longer_rows", 9)])
 @pytest.mark.parametrize("sizes", [[1], [2], [3], [31, 1, 2, 33, 1], [64, 2, 1], [5, 17, 1]])
 def test_portions(built, name, n, dtype, sizes):
     model, oracle, _ = built(name, dtype)
