@@ -17,11 +17,15 @@
 namespace a81w41 {
 namespace {
 
+typedef __attribute__((ext_vector_type(4))) short s16x4;
+typedef __attribute__((ext_vector_type(8))) short s16x8;
+typedef __attribute__((address_space(3))) s16x4* lds_s16x4;
 constexpr float kLog2e = 1.4426950408889634f;
 constexpr float kLowest = -1e30f;
 
 // DK, DV: capacities for key and value columns.  KT keys per tile, NBUF tiles in LDS.
-// COLS: all waves of the workgroup take the same query rows and each a quarter of the value columns (few rows).
+// COLS (few rows): all four waves take the same query rows; each scores its 16 keys of a tile, the scores meet in LDS,
+// and each sums its quarter of the value columns.
 template <int DK, int DV, int WAVES, int QS, int KT, int NBUF, bool EXPANDED, bool COLS>
 __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
     constexpr int CK = DK / 8;                    // 16-byte chunks of a key row
@@ -30,7 +34,10 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
     constexpr int kBuf = kKeyBytes + kValueBytes;
     constexpr int KS = DK / 32, VF = DV / 16 / (COLS ? WAVES : 1), kRows = 16 * QS * (COLS ? 1 : WAVES);
     static_assert(DK % 64 == 0 && DV % 16 == 0 && KT % 32 == 0 && (!EXPANDED || CV == 8), "tile sizes");
+    constexpr int kScoreRow = 16 * QS + 4;  // floats of a key's scores in LDS: lane groups fall into different banks
+    static_assert(!COLS || KT == 16 * WAVES, "a wave scores 16 keys of a tile");
     __shared__ __attribute__((aligned(128))) uint8_t lds[NBUF * kBuf];
+    __shared__ float scores[COLS ? KT * kScoreRow : 1];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l15 = lane & 15, g = lane >> 4;
     const int row_wave = COLS ? 0 : wave, f0 = COLS ? wave * VF : 0;  // first 16 value columns of this wave
     const int z = blockIdx.y;
@@ -92,15 +99,16 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
 #pragma unroll
         for (int f = 0; f < VF; f++) acc[s][f] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    // Values that are columns of the key rows: element (key row r, column 16 f + l15), r = 16 h + 4 g + j, sits at chunk
-    // (2 f + l15 / 8) ^ (r & 7); the exclusive or touches the low three bits only, so sixteen offsets serve all f and h.
-    int value_at[4][4];
+    // Values that are columns of the key rows come by transposing reads (ds_read_b64_tr_b16): in a group of 16 lanes lane
+    // i names four columns of key 4 g + i / 4 and receives its own column of the four keys.  The exclusive or of the chunk
+    // places touches the low three bits of 2 f + ..., so four offsets serve all f.
+    int value_at[4];
     if constexpr (!EXPANDED) {
 #pragma unroll
-        for (int f = 0; f < 4; f++)
-#pragma unroll
-            for (int j = 0; j < 4; j++)
-                value_at[f][j] = (4 * g + j) * (DK * 2) + (((2 * (f0 + f) + (l15 >> 3)) ^ ((4 * g + j) & 7)) << 4) + (l15 & 7) * 2;
+        for (int f = 0; f < 4; f++) {
+            const int r = 4 * g + (l15 >> 2);
+            value_at[f] = r * (DK * 2) + (((2 * (f0 + f) + ((l15 >> 1) & 1)) ^ (r & 7)) << 4) + (l15 & 1) * 8;
+        }
     }
     const float scale = a.scale * kLog2e;
     const int n_tiles = (key_end - key_begin + KT - 1) / KT;
@@ -117,17 +125,33 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
         const uint8_t* kb = lds + (tile % NBUF) * kBuf;
         const uint8_t* vb = kb + kKeyBytes;
         f32x4 sc[QS][KT / 16];
-#pragma unroll
-        for (int t = 0; t < KT / 16; t++) {
+        auto score = [&](int t) {
 #pragma unroll
             for (int s = 0; s < QS; s++) sc[s][t] = f32x4{0.f, 0.f, 0.f, 0.f};
-            const uint8_t* row = kb + (t * 16 + l15) * (DK * 2);
+            const uint8_t* row = kb + ((COLS ? wave : t) * 16 + l15) * (DK * 2);
 #pragma unroll
             for (int k = 0; k < KS; k++) {
                 const bf16x8 kf = *reinterpret_cast<const bf16x8*>(row + (((k * 4 + g) ^ (l15 & 7)) << 4));
 #pragma unroll
                 for (int s = 0; s < QS; s++) sc[s][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s][k], sc[s][t], 0, 0, 0);
             }
+        };
+        if constexpr (COLS) {
+            score(0);
+#pragma unroll
+            for (int s = 0; s < QS; s++)
+#pragma unroll
+                for (int i = 0; i < 4; i++) scores[(wave * 16 + 4 * g + i) * kScoreRow + s * 16 + l15] = sc[s][0][i];
+            dense_lds_barrier();
+#pragma unroll
+            for (int s = 0; s < QS; s++)
+#pragma unroll
+                for (int t = 0; t < KT / 16; t++)
+#pragma unroll
+                    for (int i = 0; i < 4; i++) sc[s][t][i] = scores[(t * 16 + 4 * g + i) * kScoreRow + s * 16 + l15];
+        } else {
+#pragma unroll
+            for (int t = 0; t < KT / 16; t++) score(t);
         }
         bf16x8 pf[QS][KT / 32];
 #pragma unroll
@@ -175,10 +199,11 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
                     const uint4 w = make_uint4(lo.x, lo.y, hi.x, hi.y);
                     vf = *reinterpret_cast<const bf16x8*>(&w);
                 } else {
-#pragma unroll
-                    for (int j = 0; j < 8; j++)
-                        vf[j] = *reinterpret_cast<const bf16*>(kb + value_at[f & 3][j & 3] + (f >> 2) * 128 +
-                                                               (u * 32 + (j >> 2) * 16) * (DK * 2));
+                    const uint8_t* at = kb + value_at[f & 3] + (f >> 2) * 128 + u * 32 * (DK * 2);
+                    const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(at));
+                    const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4)(at + 16 * (DK * 2)));
+                    const s16x8 both = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
+                    vf = *reinterpret_cast<const bf16x8*>(&both);
                 }
 #pragma unroll
                 for (int s = 0; s < QS; s++) acc[s][f] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[s][u], acc[s][f], 0, 0, 0);
@@ -218,9 +243,8 @@ __global__ __launch_bounds__(64 * WAVES, 1) void attend_kernel(AttendArgs a) {
 }
 
 // out[row] = sum_s w_s part_s / sum_s w_s sum_s with w_s = 2^(m_s - max m); one workgroup per row and 256 columns
-template <typename O>
 __global__ __launch_bounds__(256) void merge_shares_kernel(const float* __restrict__ part, int ld_part, const float* __restrict__ stats,
-                                                         int rows, int splits, int dv, O* __restrict__ out, int ld_out) {
+                                                         int rows, int splits, int dv, bf16* __restrict__ out, int ld_out) {
     __shared__ float w[kAttendMaxSplits];
     __shared__ float norm;
     const int r = blockIdx.x, t = threadIdx.x;
@@ -238,7 +262,7 @@ __global__ __launch_bounds__(256) void merge_shares_kernel(const float* __restri
     if (d >= dv) return;
     float s = 0.f;
     for (int k = 0; k < splits; k++) s = fmaf(w[k], part[((size_t)k * rows + r) * ld_part + d], s);
-    out[(size_t)r * ld_out + d] = (O)(s * norm);
+    out[(size_t)r * ld_out + d] = (bf16)(s * norm);
 }
 static_assert(kAttendMaxSplits <= 64, "the merge reads one share per lane");
 
@@ -247,8 +271,8 @@ hipError_t launch_sizes(const AttendArgs& a, int heads, hipStream_t s) {
     if constexpr (EXPANDED) {
         constexpr int rows = 16 * 2 * 4;
         hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 2, 64, 2, true, false>), dim3((a.rows + rows - 1) / rows, heads, 1), dim3(256), 0, s, a);
-    } else if (a.rows <= 32) {
-        hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 1, 64, 1, false, true>), dim3((a.rows + 15) / 16, 1, a.splits), dim3(256), 0, s, a);
+    } else if (a.rows <= kAttendFewRows) {
+        hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 1, 64, 2, false, true>), dim3((a.rows + 15) / 16, 1, a.splits), dim3(256), 0, s, a);
     } else {
         hipLaunchKernelGGL((attend_kernel<DK, DV, 4, 1, 32, 1, false, false>), dim3((a.rows + 63) / 64, 1, a.splits), dim3(256), 0, s, a);
     }
@@ -274,13 +298,10 @@ hipError_t launch_attend_expanded(const AttendArgs& a, int heads, hipStream_t s)
     return launch_sizes<320, 256, true>(a, heads, s);
 }
 
-template <typename O>
-hipError_t launch_merge_shares(const AttendArgs& a, O* out, int ld_out, hipStream_t s) {
-    hipLaunchKernelGGL(merge_shares_kernel<O>, dim3(a.rows, (a.dv + 255) / 256), dim3(256), 0, s, a.part, a.ld_part, a.part_stats, a.rows,
-                       a.splits, a.dv, out, ld_out);
+hipError_t launch_merge_shares(const AttendArgs& a, hipStream_t s) {
+    hipLaunchKernelGGL(merge_shares_kernel, dim3(a.rows, (a.dv + 255) / 256), dim3(256), 0, s, a.part, a.ld_part, a.part_stats, a.rows,
+                       a.splits, a.dv, a.out, a.ld_out);
     return hipGetLastError();
 }
-template hipError_t launch_merge_shares<bf16>(const AttendArgs&, bf16*, int, hipStream_t);
-template hipError_t launch_merge_shares<float>(const AttendArgs&, float*, int, hipStream_t);
 
 }  // namespace a81w41

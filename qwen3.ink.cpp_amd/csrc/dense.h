@@ -128,6 +128,7 @@ hipError_t launch_latent_attention_vector(const T* q, const T* cache, const Late
 // 0 .. pos + token.  The results go to out, or, with splits > 1 (the keys dealt to that many workgroups), unnormalised
 // to part [splits][rows][ld_part] with part_stats [splits][rows][2] (maximum, sum), for launch_merge_shares.
 constexpr int kAttendMaxSplits = 64;
+constexpr int kAttendFewRows = 64;  // up to here a workgroup takes 16 query rows, above 64
 struct AttendArgs {
     const bf16* q = nullptr;
     long long q_head = 0;
@@ -159,8 +160,7 @@ bool attend_expanded_fits(int own, int shared, int dv);
 // Keys and values are the same rows (k_own), the values their first dv columns.
 hipError_t launch_attend_shared(const AttendArgs& a, hipStream_t s);
 hipError_t launch_attend_expanded(const AttendArgs& a, int heads, hipStream_t s);
-template <typename O>
-hipError_t launch_merge_shares(const AttendArgs& a, O* out, int ld_out, hipStream_t s);
+hipError_t launch_merge_shares(const AttendArgs& a, hipStream_t s);
 
 // ---- one-token products with the row work fused in (dense_gemv.hip) --------------------------
 // Their input rows sit in LDS as fp32: a row (or, for the experts' second product, all of a token's) may have at most

@@ -53,7 +53,7 @@ int a81w41_latent_attention(const void* q, const void* cache, int ld, int rank, 
     a.out = static_cast<bf16*>(out), a.ld_out = rank, a.splits = splits, a.part = part, a.part_stats = stats, a.ld_part = (rank + 3) / 4 * 4;
     a.scale = scale, a.pos_dev = pos_dev, a.max_seq = max_seq;
     A81W41_HIP_TRY(launch_attend_shared(a, s));
-    if (splits > 1) A81W41_HIP_TRY(launch_merge_shares<bf16>(a, a.out, rank, s));
+    if (splits > 1) A81W41_HIP_TRY(launch_merge_shares(a, s));
     return 0;
 }
 

@@ -463,7 +463,7 @@ AttendArgs TakosunModel<T>::shared_attend(const Layer& L, const LatentShape& sh,
     a.dv = sh.rank, a.scale = sh.scale, a.pos_dev = pos, a.max_seq = max_seq();
     a.part = part_, a.part_stats = part_stats_, a.ld_part = (sh.rank + 3) / 4 * 4;
     // enough workgroups for the chip, at least 64 keys for each
-    const int groups = a.rows <= 32 ? (a.rows + 15) / 16 : (a.rows + 63) / 64;
+    const int groups = a.rows <= kAttendFewRows ? (a.rows + 15) / 16 : (a.rows + 63) / 64;
     a.splits = opt_split_ ? opt_split_ : std::min({kAttendMaxSplits, (plan_ctx + 63) / 64, std::max(1, 512 / groups)});
     a.splits = std::max<int>(1, std::min<size_t>(a.splits, part_rows_ / a.rows));
     return a;
@@ -485,7 +485,7 @@ int TakosunModel<T>::attend_latent(const Layer& L, const LatentShape& sh, int M,
             AttendArgs a = shared_attend(L, sh, M);
             a.out = o_lat_, a.ld_out = ld_rank;
             A81W41_HIP_TRY(launch_attend_shared(a, s));
-            if (a.splits > 1) A81W41_HIP_TRY(launch_merge_shares<bf16>(a, o_lat_, ld_rank, s));
+            if (a.splits > 1) A81W41_HIP_TRY(launch_merge_shares(a, s));
             done = true;
         }
     }

@@ -13,7 +13,7 @@ from tests.takosun_fixture import SMALL, write_model
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
 
-def refused(pkg, cfg, match, tmp_path=None):
+def refused(pkg, cfg, match):
     with pytest.raises(pkg.capi.A81W41Error, match=match):
         pkg.Model.random(cfg, 16)
 
@@ -78,8 +78,7 @@ def test_qwen3_is_registered_and_has_no_32_bit_path(pkg, tmp_path):
 def test_fixture_round_trip(tmp_path):
     w = tf.random_weights(SMALL, 1)
     write_model(str(tmp_path), SMALL, w)
-    import safetensors.numpy  # noqa: F401  (an independent reader of the same format)
-    from safetensors import safe_open
+    from safetensors import safe_open  # an independent reader of the same format
     with safe_open(str(tmp_path / "model.safetensors"), "pt") as f:
         assert set(f.keys()) == set(w)
         assert np.array_equal(f.get_tensor("l2.mix.dkv").float().numpy(), w["l2.mix.dkv"])
