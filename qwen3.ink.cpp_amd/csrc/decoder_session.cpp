@@ -29,6 +29,17 @@ int CachePlanes::add(size_t bytes, void** plane) {
     return 0;
 }
 
+int CachePlanes::add_state(size_t bytes, void** state) {
+    A81W41_TRY(add(bytes, state));
+    states_.emplace_back(*state, bytes);
+    return 0;
+}
+
+int CachePlanes::clear_states() {
+    for (const auto& st : states_) A81W41_HIP_TRY(hipMemset(st.first, 0, st.second));
+    return 0;
+}
+
 int DecoderSession::init_session(int max_seq, int vocab, int max_rows) {
     max_seq_ = max_seq;
     vocab_ = vocab;
@@ -69,6 +80,7 @@ int DecoderSession::reset() {
     A81W41_HIP_TRY(hipStreamSynchronize(stream));
     A81W41_HIP_TRY(hipMemset(pos, 0, sizeof(int)));
     A81W41_HIP_TRY(hipMemset(step, 0, sizeof(int)));
+    A81W41_TRY(cache.clear_states());
     host_pos = 0;
     return 0;
 }

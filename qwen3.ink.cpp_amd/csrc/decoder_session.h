@@ -41,7 +41,8 @@ hipError_t launch_argmax_token(const float* logits, int n, int* next_id, int* hi
                                hipStream_t s);
 hipError_t launch_advance(int* pos_dev, int by, hipStream_t s);
 
-// The cache of a sequence: planes of max_seq rows, zero when allocated, freed with the object.
+// What a sequence holds on the device, zero when allocated, freed with the object: cache planes of max_seq rows, which a new
+// sequence overwrites, and recurrent states, which go back to zero when the sequence is given back.
 class CachePlanes {
    public:
     CachePlanes() = default;
@@ -49,10 +50,13 @@ class CachePlanes {
     CachePlanes& operator=(const CachePlanes&) = delete;
     ~CachePlanes();
     int add(size_t bytes, void** plane);
+    int add_state(size_t bytes, void** state);
+    int clear_states();
     size_t bytes() const { return bytes_; }
 
    private:
     std::vector<void*> planes_;
+    std::vector<std::pair<void*, size_t>> states_;
     size_t bytes_ = 0;
 };
 

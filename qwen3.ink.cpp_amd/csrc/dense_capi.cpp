@@ -34,26 +34,31 @@ int a81w41_latent_attention(const void* q, const void* cache, int ld, int rank, 
         ld < rank + rot || ld % (is_bf16 ? 64 : 32) || variant < 0 || variant > 1 || !aligned16(q) || !aligned16(cache))
         return failf(A81W41_ERR_INVALID_ARG, "bad attention shape");
     hipStream_t s = static_cast<hipStream_t>(stream);
-    LatentShape sh;
-    sh.heads = heads, sh.rank = rank, sh.rot = rot, sh.ld_cache = ld, sh.scale = scale;
-    if (variant == 0) {
-        if (is_bf16)
-            A81W41_HIP_TRY((launch_latent_attention_vector<bf16, bf16>(static_cast<const bf16*>(q), static_cast<const bf16*>(cache), sh, pos_dev,
-                                                                       max_seq, M, static_cast<bf16*>(out), rank, s)));
-        else
-            A81W41_HIP_TRY((launch_latent_attention_vector<float, float>(static_cast<const float*>(q), static_cast<const float*>(cache), sh,
-                                                                         pos_dev, max_seq, M, static_cast<float*>(out), rank, s)));
+    const int width = (rank + rot + 7) / 8 * 8;
+    auto set = [&](auto& a, auto type) {
+        using T = decltype(type);
+        a.q = static_cast<const T*>(q), a.ld_q = ld, a.q_token = heads * ld, a.rows = M * heads, a.rows_per_token = heads;
+        a.k_own = static_cast<const T*>(cache), a.ld_k_own = ld, a.k_own_width = width, a.dv = rank;
+        a.ld_out = rank, a.out_token = heads * rank, a.scale = scale, a.pos_dev = pos_dev, a.max_seq = max_seq;
+    };
+    AttendArgs<float> af;
+    AttendArgs<bf16> a;
+    if (!is_bf16) {
+        if (variant) return failf(A81W41_ERR_INVALID_ARG, "the matrix-core attention does not take this shape");
+        set(af, 0.f);
+        A81W41_HIP_TRY((launch_attend_vector<float, float>(af, 1, static_cast<float*>(out), s)));
         return 0;
     }
-    if (!is_bf16 || !attend_shared_fits(rank + rot, rank) || splits < 1 || splits > kAttendMaxSplits || (splits > 1 && (!part || !stats)))
+    set(a, bf16{});
+    if (variant == 0) {
+        A81W41_HIP_TRY((launch_attend_vector<bf16, bf16>(a, 1, static_cast<bf16*>(out), s)));
+        return 0;
+    }
+    if (!attend_shared_fits(rank + rot, rank) || splits < 1 || splits > kAttendMaxSplits || (splits > 1 && (!part || !stats)))
         return failf(A81W41_ERR_INVALID_ARG, "the matrix-core attention does not take this shape");
-    AttendArgs a;
-    a.q = static_cast<const bf16*>(q), a.ld_q = ld, a.rows = M * heads, a.rows_per_token = heads;
-    a.k_own = static_cast<const bf16*>(cache), a.ld_k_own = ld, a.k_own_width = (rank + rot + 7) / 8 * 8, a.dv = rank;
-    a.out = static_cast<bf16*>(out), a.ld_out = rank, a.splits = splits, a.part = part, a.part_stats = stats, a.ld_part = (rank + 3) / 4 * 4;
-    a.scale = scale, a.pos_dev = pos_dev, a.max_seq = max_seq;
+    a.out = static_cast<bf16*>(out), a.splits = splits, a.part = part, a.part_stats = stats, a.ld_part = (rank + 3) / 4 * 4;
     A81W41_HIP_TRY(launch_attend_shared(a, s));
-    if (splits > 1) A81W41_HIP_TRY(launch_merge_shares(a, s));
+    if (splits > 1) A81W41_HIP_TRY(launch_merge_shares(a, 1, s));
     return 0;
 }
 
@@ -64,12 +69,12 @@ int a81w41_formed_attention(const void* q, const void* k, const void* k_rot, int
         ld_rot < rot || ld_rot % 8 || ld_v % 64 || ld_v < max_seq || !attend_expanded_fits(dim, rot, vdim) || !aligned16(q) || !aligned16(k) ||
         !aligned16(k_rot) || !aligned16(v_t))
         return failf(A81W41_ERR_INVALID_ARG, "bad attention shape");
-    AttendArgs a;
-    a.q = static_cast<const bf16*>(q), a.q_head = dim + rot, a.ld_q = heads * (dim + rot), a.rows = M;
+    AttendArgs<bf16> a;
+    a.q = static_cast<const bf16*>(q), a.q_head = dim + rot, a.q_token = heads * (dim + rot), a.rows = M;
     a.k_own = static_cast<const bf16*>(k), a.k_own_head = dim, a.ld_k_own = heads * dim, a.k_own_width = dim;
     a.k_shared = static_cast<const bf16*>(k_rot), a.ld_k_shared = ld_rot, a.k_shared_width = rot;
     a.v_t = static_cast<const bf16*>(v_t), a.ld_v = ld_v, a.dv = vdim, a.head_gate = gates, a.ld_gate = heads;
-    a.out = static_cast<bf16*>(out), a.out_head = vdim, a.ld_out = heads * vdim;
+    a.out = static_cast<bf16*>(out), a.out_head = vdim, a.out_token = heads * vdim;
     a.scale = scale, a.pos_dev = pos_dev, a.max_seq = max_seq;
     A81W41_HIP_TRY(launch_attend_expanded(a, heads, static_cast<hipStream_t>(stream)));
     return 0;

@@ -19,6 +19,46 @@ __device__ __forceinline__ float dense_wave_max(float v, int width = 64) {
 }
 __device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float gated_unit(const GatedUnit& p, float gate, float up) {
+    const float g = fminf(gate, p.limit), u = fminf(fmaxf(up, -p.limit), p.limit);
+    return g / (1.0f + expf(-p.slope * g)) * (u + p.shift);
+}
+
+// How many of z[0 .. n) come before z[e]: the larger ones, and the equal ones with lower numbers.
+__device__ __forceinline__ int expert_rank(const float* z, int n, int e) {
+    const float own = z[e];
+    int rank = 0;
+#pragma unroll 4
+    for (int j = 0; j < n; j++) rank += (z[j] > own || (z[j] == own && j < e)) ? 1 : 0;
+    return rank;
+}
+
+// One column of a HeadRows product for row m: `own` is its value, `other` that of its pair's other column.
+template <typename T>
+__device__ __forceinline__ void store_head_column(const HeadRows<T>& p, int pos, int m, int col, float own, float other) {
+    const int nq = p.heads * p.dim, nk = p.kv_heads * p.dim, nv = p.kv_heads * p.vdim;
+    if (col >= nq + nk + nv) {
+        p.rest[(size_t)m * p.ld_rest + col - nq - nk - nv] = own;
+        return;
+    }
+    const int at = min(pos + m, p.max_seq - 1);
+    if (col >= nq + nk) {
+        const int c = col - nq - nk, h = c / p.vdim;
+        p.cache[(size_t)at * p.ld_cache + h * (p.vdim + p.dim) + (c - h * p.vdim)] = (T)own;
+        return;
+    }
+    const bool key = col >= nq;
+    const int c = key ? col - nq : col, h = c / p.dim, d = c - h * p.dim;
+    if ((d >> 1) < p.rot_pairs) {
+        const size_t i = (size_t)at * p.rot_pairs + (d >> 1);
+        const float cs = p.cos_t[i], sn = p.sin_t[i];
+        own = (d & 1) ? own * cs + other * sn : own * cs - other * sn;
+    }
+    if (key)
+        p.cache[(size_t)at * p.ld_cache + h * (p.vdim + p.dim) + p.vdim + d] = (T)own;
+    else
+        p.q[(size_t)m * nq + c] = (T)own;
+}
 
 // One direct copy global -> LDS of 16 bytes per lane: lane l's bytes land at lds_base + 16 l (lds_base uniform).
 __device__ __forceinline__ void copy16_to_lds(const void* global_src, void* lds_base) {

@@ -21,8 +21,11 @@ __device__ __forceinline__ void mma(f32x16& acc, const uint4& a, const uint4& b,
     acc = __builtin_amdgcn_mfma_f32_32x32x2f32(__uint_as_float(a.w), __uint_as_float(b.w), acc, 0, 0, 0);
 }
 
-template <typename T, int BM, int BN, Epilogue EPI>
-__global__ __launch_bounds__(256, 2) void dense_gemm_kernel(GemmArgs g) {
+struct NoHeads {};
+
+// X: HeadRows<T> with the epilogue kHeads, NoHeads with the others
+template <typename T, int BM, int BN, Epilogue EPI, typename X>
+__global__ __launch_bounds__(256, 2) void dense_gemm_kernel(GemmArgs g, X heads) {
     constexpr int WM = BM / 2, WN = BN / 2, FM = WM / 32, FN = WN / 32;
     constexpr int LA = BM / 32, LB = BN / 32;  // direct copies per thread and stage
     constexpr int kStage = (BM + BN) * 128;
@@ -103,6 +106,8 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(GemmArgs g) {
                 for (int j = 0; j < FN; j++) mma(acc[i][j], a[i], b[j], static_cast<T*>(nullptr));
         }
     }
+    [[maybe_unused]] int pos = 0;
+    if constexpr (EPI == Epilogue::kHeads) pos = min(max(heads.pos_dev[0], 0), heads.max_seq - 1);
     // register v of lane l holds row 8 (v / 4) + 4 (l / 32) + v % 4, column l % 32 of a piece
 #pragma unroll
     for (int i = 0; i < FM; i++)
@@ -113,10 +118,13 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(GemmArgs g) {
             for (int v = 0; v < 16; v++) {
                 const int r = wm + i * 32 + 8 * (v >> 2) + 4 * half + (v & 3);
                 const size_t row = m0 + r;
-                if constexpr (EPI == Epilogue::kSiluPair) {
+                if constexpr (EPI == Epilogue::kGatedPair) {
                     const float up = __shfl_xor(acc[i][j][v], 16, 64);
                     if (r < rows && col < g.N && !(lane & 16))
-                        static_cast<T*>(g.C)[row * g.ldc + (col >> 5) * 16 + (col & 15)] = (T)(silu(acc[i][j][v]) * up);
+                        static_cast<T*>(g.C)[row * g.ldc + (col >> 5) * 16 + (col & 15)] = (T)gated_unit(g.unit, acc[i][j][v], up);
+                } else if constexpr (EPI == Epilogue::kHeads) {
+                    const float other = __shfl_xor(acc[i][j][v], 1, 64);
+                    if (r < rows && col < g.N) store_head_column(heads, pos, (int)row, col, acc[i][j][v], other);
                 } else if (r < rows && col < g.N) {
                     if constexpr (EPI == Epilogue::kFloat) {
                         (static_cast<float*>(g.C) + (g.tiles ? 0 : batch * g.c_step))[row * g.ldc + col] = acc[i][j][v];
@@ -130,30 +138,43 @@ __global__ __launch_bounds__(256, 2) void dense_gemm_kernel(GemmArgs g) {
         }
 }
 
-template <typename T, int BM, int BN>
-hipError_t launch_tile(const GemmArgs& g, Epilogue epi, hipStream_t s) {
+template <typename T, int BM, int BN, Epilogue EPI, typename X>
+hipError_t launch_kernel(const GemmArgs& g, const X& heads, hipStream_t s) {
     const int n_mt = g.tiles ? g.max_tiles : (g.M + BM - 1) / BM, n_nt = (g.N + BN - 1) / BN;
-    const dim3 grid(n_mt * n_nt, g.batches), block(256);
-    switch (epi) {
-        case Epilogue::kFloat: hipLaunchKernelGGL((dense_gemm_kernel<T, BM, BN, Epilogue::kFloat>), grid, block, 0, s, g); break;
-        case Epilogue::kElement: hipLaunchKernelGGL((dense_gemm_kernel<T, BM, BN, Epilogue::kElement>), grid, block, 0, s, g); break;
-        case Epilogue::kSiluPair: hipLaunchKernelGGL((dense_gemm_kernel<T, BM, BN, Epilogue::kSiluPair>), grid, block, 0, s, g); break;
-        case Epilogue::kHeadGate: hipLaunchKernelGGL((dense_gemm_kernel<T, BM, BN, Epilogue::kHeadGate>), grid, block, 0, s, g); break;
-    }
+    hipLaunchKernelGGL((dense_gemm_kernel<T, BM, BN, EPI, X>), dim3(n_mt * n_nt, g.batches), dim3(256), 0, s, g, heads);
     return hipGetLastError();
+}
+
+template <typename T, Epilogue EPI, typename X>
+hipError_t launch_by_size(const GemmArgs& g, const X& heads, hipStream_t s) {
+    // large tiles where they still give every CU work; a grouped product's row tiles are kGroupTileRows high
+    const long long big = (long long)((g.M + 127) / 128) * ((g.N + 127) / 128) * g.batches;
+    if (!g.tiles && g.M > 64 && big >= 192) return launch_kernel<T, 128, 128, EPI>(g, heads, s);
+    if (g.tiles && g.N >= 1024) return launch_kernel<T, kGroupTileRows, 128, EPI>(g, heads, s);
+    return launch_kernel<T, 64, 64, EPI>(g, heads, s);
 }
 
 }  // namespace
 
 template <typename T>
 hipError_t launch_dense_gemm(const GemmArgs& g, Epilogue epi, hipStream_t s) {
-    // large tiles where they still give every CU work; a grouped product's row tiles are kGroupTileRows high
-    const long long big = (long long)((g.M + 127) / 128) * ((g.N + 127) / 128) * g.batches;
-    if (!g.tiles && g.M > 64 && big >= 192) return launch_tile<T, 128, 128>(g, epi, s);
-    if (g.tiles && g.N >= 1024) return launch_tile<T, kGroupTileRows, 128>(g, epi, s);
-    return launch_tile<T, 64, 64>(g, epi, s);
+    switch (epi) {
+        case Epilogue::kFloat: return launch_by_size<T, Epilogue::kFloat>(g, NoHeads{}, s);
+        case Epilogue::kElement: return launch_by_size<T, Epilogue::kElement>(g, NoHeads{}, s);
+        case Epilogue::kGatedPair: return launch_by_size<T, Epilogue::kGatedPair>(g, NoHeads{}, s);
+        case Epilogue::kHeadGate: return launch_by_size<T, Epilogue::kHeadGate>(g, NoHeads{}, s);
+        case Epilogue::kHeads: break;  // has a launcher of its own
+    }
+    return hipErrorInvalidValue;
 }
-template hipError_t launch_dense_gemm<bf16>(const GemmArgs&, Epilogue, hipStream_t);
-template hipError_t launch_dense_gemm<float>(const GemmArgs&, Epilogue, hipStream_t);
+template <typename T>
+hipError_t launch_dense_gemm_heads(const GemmArgs& g, const HeadRows<T>& heads, hipStream_t s) {
+    return launch_by_size<T, Epilogue::kHeads>(g, heads, s);
+}
+#define INSTANTIATE(T)                                                              \
+    template hipError_t launch_dense_gemm<T>(const GemmArgs&, Epilogue, hipStream_t); \
+    template hipError_t launch_dense_gemm_heads<T>(const GemmArgs&, const HeadRows<T>&, hipStream_t);
+INSTANTIATE(bf16)
+INSTANTIATE(float)
 
 }  // namespace a81w41

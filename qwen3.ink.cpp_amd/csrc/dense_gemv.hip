@@ -154,7 +154,7 @@ class StepRow {
             const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
             x_[k] = in ? load4(p_.x + i) : zero;
             y_[k] = in && p_.y ? load4(p_.y + i) : zero;
-            wy_[k] = in && p_.y ? load4(p_.norm_y.w + i) : zero;
+            wy_[k] = in && p_.norm_y.w ? load4(p_.norm_y.w + i) : zero;
             before_[k] = in && p_.before ? load4(p_.before + i) : zero;
             wh_[k] = in ? load4(p_.norm_h.w + i) : zero;
         }
@@ -162,12 +162,13 @@ class StepRow {
     __device__ __forceinline__ void finish(float* xs, int padded, float* inv, float* red) {
         if (!fast_) return slow(xs, padded, inv, red);
         const bool writer = blockIdx.x == 0 && blockIdx.y == 0;
-        const float coef = p_.before ? *p_.coef : 1.f;
-        const float inv_y = p_.y ? parts_.inverse_rms(y_, p_.norm_y.eps, red) : 0.f;
+        const float coef = p_.before && p_.coef ? *p_.coef : 1.f;
+        const bool normed = p_.y && p_.norm_y.w;
+        const float inv_y = normed ? parts_.inverse_rms(y_, p_.norm_y.eps, red) : 0.f;
 #pragma unroll
         for (int k = 0; k < kParts; k++) {
             const int i = parts_.place(k);
-            float4 r = add4(x_[k], scale4(y_[k], inv_y, wy_[k]));
+            float4 r = normed ? add4(x_[k], scale4(y_[k], inv_y, wy_[k])) : fma4(p_.norm_y.scale, y_[k], x_[k]);
             if (i >= 0 && writer && p_.state) store4(p_.state + i, r);
             if (p_.before) r = fma4(coef, r, before_[k]);
             if (i >= 0 && writer && p_.x_out) store4(p_.x_out + i, r);
@@ -177,7 +178,10 @@ class StepRow {
 #pragma unroll
         for (int k = 0; k < kParts; k++) {
             const int i = parts_.place(k);
-            if (i >= 0) store4(xs + i, scale4(x_[k], inv_h, wh_[k]));
+            if (i < 0) continue;
+            const float4 h = scale4(x_[k], inv_h, wh_[k]);
+            store4(xs + i, h);
+            if (writer && p_.h_out) store4(p_.h_out + i, h);
         }
         for (int i = p_.width + threadIdx.x; i < padded; i += kThreads) xs[i] = 0.f;
         dense_lds_barrier();
@@ -189,14 +193,15 @@ class StepRow {
         const RowStep& p = p_;
         const int t = threadIdx.x, W = p.width;
         const bool writer = blockIdx.x == 0 && blockIdx.y == 0;
-        if (p.y) group_inverse_rms<kThreads>([&](int i) { return p.y[i]; }, W, p.norm_y.groups, p.norm_y.eps, inv, red);
-        const float coef = p.before ? *p.coef : 0.f;
-        const int size_y = p.y ? W / p.norm_y.groups : 1;
+        const bool normed = p.y && p.norm_y.w;
+        if (normed) group_inverse_rms<kThreads>([&](int i) { return p.y[i]; }, W, p.norm_y.groups, p.norm_y.eps, inv, red);
+        const float coef = p.before && p.coef ? *p.coef : 1.f;
+        const int size_y = normed ? W / p.norm_y.groups : 1;
         for (int i = t; i < padded; i += kThreads) {
             float r = 0.f;
             if (i < W) {
                 r = p.x[i];
-                if (p.y) r += p.y[i] * inv[i / size_y] * p.norm_y.w[i];
+                if (p.y) r = normed ? r + p.y[i] * inv[i / size_y] * p.norm_y.w[i] : fmaf(p.norm_y.scale, p.y[i], r);
                 if (writer && p.state) p.state[i] = r;
                 if (p.before) r = fmaf(coef, r, p.before[i]);
                 if (writer && p.x_out) p.x_out[i] = r;
@@ -206,7 +211,10 @@ class StepRow {
         __syncthreads();
         group_inverse_rms<kThreads>([&](int i) { return xs[i]; }, W, p.norm_h.groups, p.norm_h.eps, inv, red);
         const int size_h = W / p.norm_h.groups;
-        for (int i = t; i < W; i += kThreads) xs[i] = xs[i] * inv[i / size_h] * p.norm_h.w[i];
+        for (int i = t; i < W; i += kThreads) {
+            xs[i] = xs[i] * inv[i / size_h] * p.norm_h.w[i];
+            if (writer && p.h_out) p.h_out[i] = xs[i];
+        }
         __syncthreads();
     }
     const RowStep& p_;
@@ -215,9 +223,20 @@ class StepRow {
     float4 x_[kParts], y_[kParts], wy_[kParts], before_[kParts], wh_[kParts];
 };
 
-// C[n] = W[n] . row
 template <typename T>
-__global__ __launch_bounds__(kThreads) void gemv_step_kernel(RowStep p, const T* __restrict__ w, int ld, int N, float* __restrict__ C) {
+struct HeadsEmit {
+    HeadRows<T> heads;
+    int N;
+    __device__ void operator()(int n, float s0, float s1) const {
+        const int pos = min(max(heads.pos_dev[0], 0), heads.max_seq - 1);
+        store_head_column(heads, pos, 0, 2 * n, s0, s1);
+        if (2 * n + 1 < N) store_head_column(heads, pos, 0, 2 * n + 1, s1, s0);
+    }
+};
+
+// emit gets W[n] . row, in pairs of n
+template <typename T, typename Emit>
+__global__ __launch_bounds__(kThreads) void gemv_step_kernel(RowStep p, const T* __restrict__ w, int ld, int N, Emit emit) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     float *xs = smem, *red = xs + ld, *inv = red + kThreads / 64;
     StepRow row(p);
@@ -228,7 +247,7 @@ __global__ __launch_bounds__(kThreads) void gemv_step_kernel(RowStep p, const T*
     Pair ahead;
     request_first(ahead, rows, pairs, chunks, d);
     row.finish(xs, ld, inv, red);
-    stream_pairs<T>(ahead, rows, PlainEmit{C, N, 1.f}, pairs, xs, chunks, d);
+    stream_pairs<T>(ahead, rows, emit, pairs, xs, chunks, d);
 }
 
 // C[n] = W[n] . x
@@ -401,16 +420,42 @@ __device__ __forceinline__ int expert_of(const ExpertRows& e, int slot) {
     return min(max(e.table[(size_t)id * e.top + slot], 0), e.experts - 1);
 }
 
-// act = silu(gate) * up for the token's experts (blockIdx.y < top) and the dense or shared feed-forward (the last).
+// The router's choice for one token, formed by a whole workgroup from its logits (z, best: LDS): ids[0 .. top).
+__device__ __forceinline__ void choose_experts(const ExpertRows& e, float* z, int* ids, float* best) {
+    for (int i = threadIdx.x; i < e.experts; i += kThreads) z[i] = e.logits[i] + e.bias[i];
+    __syncthreads();
+    for (int i = threadIdx.x; i < e.experts; i += kThreads) {
+        const int rank = expert_rank(z, e.experts, i);
+        if (rank < e.top) {
+            ids[rank] = i;
+            best[rank] = z[i];
+        }
+    }
+    __syncthreads();
+    if (blockIdx.x == 0 && blockIdx.y == 0 && threadIdx.x < 64) {
+        const int k = threadIdx.x;
+        const float w = k < e.top ? expf(best[k] - best[0]) : 0.f, sum = dense_wave_sum(w);
+        if (k < e.top) {
+            e.chosen[k] = ids[k];
+            e.weights[k] = w / sum;
+        }
+    }
+}
+
+// act = unit(gate, up) for the token's experts (blockIdx.y < top) and the dense or shared feed-forward (the last).
 template <typename T>
-__global__ __launch_bounds__(kThreads) void gemv_gate_up_kernel(RowStep p, ExpertRows e, const T* __restrict__ experts,
-                                                               const T* __restrict__ dense, int ld, float* __restrict__ act) {
+__global__ __launch_bounds__(kThreads) void gemv_gate_up_kernel(RowStep p, const float* __restrict__ h, ExpertRows e,
+                                                               const T* __restrict__ experts, const T* __restrict__ dense, int ld,
+                                                               float* __restrict__ act) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
+    __shared__ int ids[kMaxTop];
+    __shared__ float best[kMaxTop];
     float *xs = smem, *red = xs + ld, *inv = red + kThreads / 64;
-    StepRow row(p);
-    row.load();
     const int slot = blockIdx.y;
-    const T* w = slot < e.top ? experts + (size_t)expert_of(e, slot) * e.pair_rows * ld : dense;
+    StepRow row(p);
+    if (!h) row.load();
+    if (e.logits) choose_experts(e, red, ids, best);  // the places of red and inv are free until the row is formed
+    const T* w = slot < e.top ? experts + (size_t)(e.logits ? ids[slot] : expert_of(e, slot)) * e.pair_rows * ld : dense;
     const int ff = slot < e.top ? e.ff : e.dense_ff;
     const int chunks = ld * (int)sizeof(T) / 16;
     const Deal d = deal_rows<T>(chunks, gridDim.x);
@@ -420,9 +465,15 @@ __global__ __launch_bounds__(kThreads) void gemv_gate_up_kernel(RowStep p, Exper
     };
     Pair ahead;
     request_first(ahead, rows, ff, chunks, d);
-    row.finish(xs, ld, inv, red);
+    if (h) {
+        copy_row(xs, h, p.width, ld);
+        dense_lds_barrier();
+    } else {
+        if (e.logits) __syncthreads();
+        row.finish(xs, ld, inv, red);
+    }
     float* dst = act + (size_t)slot * e.ld_act;
-    stream_pairs<T>(ahead, rows, [&](int j, float gate, float up) { dst[j] = silu(gate) * up; }, ff, xs, chunks, d);
+    stream_pairs<T>(ahead, rows, [&](int j, float gate, float up) { dst[j] = gated_unit(e.unit, gate, up); }, ff, xs, chunks, d);
 }
 
 // y[n] = mean over the token's experts of W_e[n] . act_e, plus the dense or shared feed-forward's.
@@ -487,6 +538,88 @@ __global__ __launch_bounds__(kThreads) void gemv_ff_down_kernel(ExpertRows e, co
     }
 }
 
+// The mixer's row into xs (LDS, zero-padded).  inv: a float for every head, or for every head and share.
+__device__ __forceinline__ void form_mixer_row(const MixerRow& m, float* xs, int padded, float* inv, float* red) {
+    const int t = threadIdx.x;
+    if (m.shares.part) {  // per head sum_k w_k share_k / sum_k w_k sum_k, w_k = 2^(maximum_k - largest)
+        const int n = m.shares.splits, H = m.heads;
+        for (int h = t; h < H; h += kThreads) {
+            float top = -3.402823466e38f;
+            for (int k = 0; k < n; k++) top = fmaxf(top, m.shares.stats[2 * ((size_t)k * H + h)]);
+            float all = 0.f;
+            for (int k = 0; k < n; k++) {
+                const float w = exp2f(m.shares.stats[2 * ((size_t)k * H + h)] - top);
+                inv[h * n + k] = w;
+                all = fmaf(w, m.shares.stats[2 * ((size_t)k * H + h) + 1], all);
+            }
+            for (int k = 0; k < n; k++) inv[h * n + k] /= all;
+        }
+        __syncthreads();
+        fill_row(xs, m.width, padded, [&](int i) {
+            const int h = i / m.vdim, d = i - h * m.vdim;
+            float s = 0.f;
+            for (int k = 0; k < n; k++) s = fmaf(inv[h * n + k], m.shares.part[((size_t)k * H + h) * m.shares.ld + d], s);
+            return s;
+        });
+    } else if (m.norm) {
+        group_inverse_rms<kThreads>([&](int i) { return m.row[i]; }, m.width, m.heads, m.eps, inv, red);
+        fill_row(xs, m.width, padded, [&](int i) { return m.row[i] * inv[i / m.vdim] * m.norm[i] * sigmoid(m.gates[i]); });
+    } else {
+        copy_row(xs, m.row, m.width, padded);
+    }
+}
+
+// y[n] = W_o[n] . mixer row + sum_k weights[k] W_e(k)[n] . act_k: a pair of rows of every expert in turn, then of W_o; the
+// loads run one step ahead.
+template <typename T>
+__global__ __launch_bounds__(kThreads) void gemv_mixer_down_kernel(MixerRow m, const T* __restrict__ wo, int ld_wo, ExpertRows e,
+                                                                  const float* __restrict__ act, const T* __restrict__ experts, int ld,
+                                                                  int N, float* __restrict__ y) {
+    extern __shared__ __attribute__((aligned(16))) float smem[];
+    __shared__ int chosen[kMaxTop];
+    __shared__ float weights[kMaxTop];
+    const int chunks = ld * (int)sizeof(T) / 16, chunks_wo = ld_wo * (int)sizeof(T) / 16, pairs = (N + 1) / 2;
+    float *xs_mixer = smem, *xs = xs_mixer + ld_wo, *red = xs + e.top * ld, *inv = red + kThreads / 64;
+    const Deal d = deal_rows<T>(chunks_wo, gridDim.x);
+    if ((int)threadIdx.x < e.top) {
+        chosen[threadIdx.x] = min(max(e.chosen[threadIdx.x], 0), e.experts - 1);
+        weights[threadIdx.x] = e.weights[threadIdx.x];
+    }
+    const int parts = e.top + 1, per_step = kAhead * d.lanes;
+    auto rows_of = [&](int n, int k) {
+        return k == 0 ? PlainRows<T>{wo, ld_wo, N}(n) : PlainRows<T>{experts + (size_t)chosen[k - 1] * N * ld, ld, N}(n);
+    };
+    Pair ahead;
+    if (d.group < pairs) load_pair(ahead, rows_of(d.group, 0), d.at, d.lanes, chunks_wo);
+    for (int k = 0; k < e.top; k++) copy_row(xs + k * ld, act + (size_t)k * e.ld_act, e.ff, ld);
+    form_mixer_row(m, xs_mixer, ld_wo, inv, red);
+    __syncthreads();
+    for (int n = d.group; n < pairs; n += d.groups) {
+        float a0 = 0.f, a1 = 0.f;
+        for (int k = 0; k < parts; k++) {
+            const int all = k ? chunks : chunks_wo, steps = (all + per_step - 1) / per_step;
+            const float* row = k ? xs + (k - 1) * ld : xs_mixer;
+            float s0 = 0.f, s1 = 0.f;
+            for (int step = 0; step < steps; step++) {
+                const int c = d.at + step * per_step;
+                const Pair now = ahead;
+                if (step + 1 < steps)
+                    load_pair(ahead, rows_of(n, k), c + per_step, d.lanes, all);
+                else if (k + 1 < parts)
+                    load_pair(ahead, rows_of(n, k + 1), d.at, d.lanes, chunks);
+                else if (n + d.groups < pairs)
+                    load_pair(ahead, rows_of(n + d.groups, 0), d.at, d.lanes, chunks_wo);
+                use_pair<T>(now, row, c, d.lanes, all, s0, s1);
+            }
+            a0 = fmaf(k ? weights[k - 1] : 1.f, s0, a0);
+            a1 = fmaf(k ? weights[k - 1] : 1.f, s1, a1);
+        }
+        a0 = dense_wave_sum(a0, d.lanes);
+        a1 = dense_wave_sum(a1, d.lanes);
+        if (d.at == 0) PlainEmit{y, N, 1.f}(n, a0, a1);
+    }
+}
+
 // Workgroups for N rows of `ld` elements: at most `limit`, and as many as give every lane group the same number of pairs.
 template <typename T>
 int workgroups(int N, int ld, int limit) {
@@ -505,7 +638,14 @@ size_t step_lds(int ld, const RowStep& p) {
 
 template <typename T>
 hipError_t launch_gemv_step(const RowStep& p, const T* w, int ld, int N, float* C, hipStream_t s) {
-    hipLaunchKernelGGL(gemv_step_kernel<T>, dim3(workgroups<T>(N, ld, kMaxGrid)), dim3(kThreads), step_lds(ld, p), s, p, w, ld, N, C);
+    hipLaunchKernelGGL((gemv_step_kernel<T, PlainEmit>), dim3(workgroups<T>(N, ld, kMaxGrid)), dim3(kThreads), step_lds(ld, p), s, p, w, ld,
+                       N, PlainEmit{C, N, 1.f});
+    return hipGetLastError();
+}
+template <typename T>
+hipError_t launch_gemv_step_heads(const RowStep& p, const T* w, int ld, int N, const HeadRows<T>& heads, hipStream_t s) {
+    hipLaunchKernelGGL((gemv_step_kernel<T, HeadsEmit<T>>), dim3(workgroups<T>(N, ld, kMaxGrid)), dim3(kThreads), step_lds(ld, p), s, p, w,
+                       ld, N, HeadsEmit<T>{heads, N});
     return hipGetLastError();
 }
 template <typename T>
@@ -538,11 +678,13 @@ hipError_t launch_gemv_values(const float* o_lat, int ld_o, const LatentShares& 
     return hipGetLastError();
 }
 template <typename T>
-hipError_t launch_gemv_gate_up(const RowStep& p, const ExpertRows& e, const T* experts, const T* dense, int ld, float* act, hipStream_t s) {
+hipError_t launch_gemv_gate_up(const RowStep& p, const float* h, const ExpertRows& e, const T* experts, const T* dense, int ld, float* act,
+                               hipStream_t s) {
     const int most = e.top && e.ff > e.dense_ff ? e.ff : e.dense_ff;
     const int slots = e.top + (e.dense_ff ? 1 : 0);
-    hipLaunchKernelGGL(gemv_gate_up_kernel<T>, dim3(workgroups<T>(2 * most, ld, kMaxGrid), slots), dim3(kThreads), step_lds(ld, p), s, p, e,
-                       experts, dense, ld, act);
+    const size_t router = e.logits ? (ld + e.experts) * sizeof(float) : 0, lds = step_lds(ld, p);
+    hipLaunchKernelGGL(gemv_gate_up_kernel<T>, dim3(workgroups<T>(2 * most, ld, kMaxGrid), slots), dim3(kThreads), lds > router ? lds : router,
+                       s, p, h, e, experts, dense, ld, act);
     return hipGetLastError();
 }
 template <typename T>
@@ -554,6 +696,16 @@ hipError_t launch_gemv_ff_down(const ExpertRows& e, const float* act, const T* e
     return hipGetLastError();
 }
 
+template <typename T>
+hipError_t launch_gemv_mixer_down(const MixerRow& m, const T* wo, int ld_wo, const ExpertRows& e, const float* act, const T* experts,
+                                  int ld, int N, float* y, hipStream_t s) {
+    const int inv = m.shares.part ? m.heads * m.shares.splits : m.heads;
+    const size_t lds = (ld_wo + (size_t)e.top * ld + kThreads / 64 + inv) * sizeof(float);
+    hipLaunchKernelGGL(gemv_mixer_down_kernel<T>, dim3(workgroups<T>(N, ld_wo, kMaxGrid)), dim3(kThreads), lds, s, m, wo, ld_wo, e, act,
+                       experts, ld, N, y);
+    return hipGetLastError();
+}
+
 #define INSTANTIATE(T)                                                                                                            \
     template hipError_t launch_gemv_step<T>(const RowStep&, const T*, int, int, float*, hipStream_t);                              \
     template hipError_t launch_gemv_plain<T>(const float*, int, const T*, int, int, float*, hipStream_t);                          \
@@ -562,7 +714,11 @@ hipError_t launch_gemv_ff_down(const ExpertRows& e, const float* act, const T* e
     template hipError_t launch_gemv_absorb<T>(const float*, const LatentRows&, const LatentShape&, const T*, int, T*, hipStream_t); \
     template hipError_t launch_gemv_values<T>(const float*, int, const LatentShares&, const LatentShape&, const T*, int,           \
                                               const float*, float*, hipStream_t);                                                                       \
-    template hipError_t launch_gemv_gate_up<T>(const RowStep&, const ExpertRows&, const T*, const T*, int, float*, hipStream_t);   \
+    template hipError_t launch_gemv_gate_up<T>(const RowStep&, const float*, const ExpertRows&, const T*, const T*, int, float*,    \
+                                               hipStream_t);                                                                       \
+    template hipError_t launch_gemv_step_heads<T>(const RowStep&, const T*, int, int, const HeadRows<T>&, hipStream_t);             \
+    template hipError_t launch_gemv_mixer_down<T>(const MixerRow&, const T*, int, const ExpertRows&, const float*, const T*, int,   \
+                                                  int, float*, hipStream_t);                                                       \
     template hipError_t launch_gemv_ff_down<T>(const ExpertRows&, const float*, const T*, int, const T*, int, int, float*,         \
                                                hipStream_t);
 INSTANTIATE(bf16)

@@ -1,6 +1,6 @@
 // Row kernels around the dense matrix products: norms in groups, the residual step between two norms with an
-// optional weighted mean over depth, and the routing of tokens to experts by a table.  One workgroup per row; the
-// row sits in LDS as fp32.
+// optional weighted mean over depth, the choice of experts by a router, and the sorting of tokens by expert.  One workgroup
+// per row; the row sits in LDS as fp32.
 #include "dense_common.h"
 
 namespace a81w41 {
@@ -25,7 +25,7 @@ __global__ __launch_bounds__(kThreads) void group_norm_kernel(const float* __res
 template <typename T>
 __global__ __launch_bounds__(kThreads) void residual_norm_any_kernel(const float* x, SublayerOut y, GroupNorm norm_y, DepthAverage depth,
                                                                 float* x_out, GroupNorm norm_h, T* __restrict__ h, int ld_h,
-                                                                int width) {
+                                                                int width, const float* __restrict__ add) {
     extern __shared__ float smem[];
     float* v = smem;
     float* inv = v + width;
@@ -38,8 +38,10 @@ __global__ __launch_bounds__(kThreads) void residual_norm_any_kernel(const float
             float s;
             if (y.slot_rows) {
                 s = 0.f;
-                for (int k = 0; k < y.top; k++) s += y.y[(size_t)y.slot_rows[m * y.top + k] * width + i];
-                s *= share;
+                for (int k = 0; k < y.top; k++) {
+                    const float w = y.weights ? y.weights[m * y.top + k] : share;
+                    s = fmaf(w, y.y[(size_t)y.slot_rows[m * y.top + k] * width + i], s);
+                }
                 if (y.shared) s += y.shared[base + i];
             } else {
                 s = y.y[base + i];
@@ -47,18 +49,19 @@ __global__ __launch_bounds__(kThreads) void residual_norm_any_kernel(const float
             v[i] = s;
         }
         __syncthreads();
-        group_inverse_rms<kThreads>([&](int i) { return v[i]; }, width, norm_y.groups, norm_y.eps, inv, red);
+        if (norm_y.w) group_inverse_rms<kThreads>([&](int i) { return v[i]; }, width, norm_y.groups, norm_y.eps, inv, red);
     }
     const int size_y = width / max(norm_y.groups, 1);
     for (int i = t; i < width; i += kThreads) {  // every element of v is read and written by the same thread from here on
         float r = x[base + i];
-        if (y.y) r += v[i] * inv[i / size_y] * norm_y.w[i];
-        if (depth.states) {
-            depth.states[depth.n * depth.state_step + base + i] = r;
+        if (y.y) r = norm_y.w ? r + v[i] * inv[i / size_y] * norm_y.w[i] : fmaf(norm_y.scale, v[i], r);
+        if (depth.states) depth.states[depth.n * depth.state_step + base + i] = r;
+        if (depth.coef) {
             float s = 0.f;
             for (int j = 0; j < depth.n; j++) s = fmaf(depth.coef[j], depth.states[j * depth.state_step + base + i], s);
             r = fmaf(depth.coef[depth.n], r, s);
         }
+        if (add) r += add[i];
         x_out[base + i] = r;
         v[i] = r;
     }
@@ -74,7 +77,7 @@ __global__ __launch_bounds__(kThreads) void residual_norm_any_kernel(const float
 template <typename T>
 __global__ __launch_bounds__(kThreads) void residual_norm_kernel(const float* x, SublayerOut y, GroupNorm norm_y, DepthAverage depth,
                                                                 float* x_out, GroupNorm norm_h, T* __restrict__ h, int ld_h,
-                                                                int width) {
+                                                                int width, const float* __restrict__ add) {
     constexpr int P = RowParts<kThreads>::kParts;
     __shared__ float red[kThreads / 64];
     const RowParts<kThreads> parts(width, norm_h.groups);
@@ -88,19 +91,24 @@ __global__ __launch_bounds__(kThreads) void residual_norm_kernel(const float* x,
         v[k] = zero;
         if (i < 0 || !y.y) continue;
         if (y.slot_rows) {
-            for (int s = 0; s < y.top; s++) v[k] = add4(v[k], load4(y.y + (size_t)y.slot_rows[m * y.top + s] * width + i));
-            v[k] = fma4(1.0f / (float)y.top, v[k], y.shared ? load4(y.shared + base + i) : zero);
+            const float share = 1.0f / (float)y.top;
+            if (y.shared) v[k] = load4(y.shared + base + i);
+            for (int s = 0; s < y.top; s++)
+                v[k] = fma4(y.weights ? y.weights[m * y.top + s] : share, load4(y.y + (size_t)y.slot_rows[m * y.top + s] * width + i), v[k]);
         } else {
             v[k] = load4(y.y + base + i);
         }
     }
-    if (y.y) {
+    if (y.y && norm_y.w) {
         const float inv = parts.inverse_rms(v, norm_y.eps, red);
 #pragma unroll
         for (int k = 0; k < P; k++) {
             const int i = parts.place(k);
             if (i >= 0) r[k] = add4(r[k], scale4(v[k], inv, load4(norm_y.w + i)));
         }
+    } else if (y.y) {
+#pragma unroll
+        for (int k = 0; k < P; k++) r[k] = fma4(norm_y.scale, v[k], r[k]);
     }
     if (depth.states) {
 #pragma unroll
@@ -109,6 +117,7 @@ __global__ __launch_bounds__(kThreads) void residual_norm_kernel(const float* x,
             v[k] = zero;
             if (i < 0) continue;
             store4(depth.states + depth.n * depth.state_step + base + i, r[k]);
+            if (!depth.coef) continue;
             const float* st = depth.states + base + i;
             int j = 0;
             for (; j + 4 <= depth.n; j += 4) {
@@ -125,7 +134,9 @@ __global__ __launch_bounds__(kThreads) void residual_norm_kernel(const float* x,
 #pragma unroll
     for (int k = 0; k < P; k++) {
         const int i = parts.place(k);
-        if (i >= 0) store4(x_out + base + i, r[k]);
+        if (i < 0) continue;
+        if (add) r[k] = add4(r[k], load4(add + i));
+        store4(x_out + base + i, r[k]);
     }
     const float inv = parts.inverse_rms(r, norm_h.eps, red);
 #pragma unroll
@@ -167,7 +178,36 @@ __device__ int block_exclusive_scan(int* a, int n, int* tmp) {
     return carry;
 }
 
-__global__ __launch_bounds__(1024) void table_route_kernel(const int* __restrict__ ids, const int* __restrict__ table, int vocab,
+// One wave per token.  An expert's rank is the number of experts before it; ranks below `top` are the choice.  A row of
+// logits sits in LDS.
+constexpr int kRouterWaves = 4;
+__global__ __launch_bounds__(64 * kRouterWaves) void router_kernel(const float* __restrict__ logits, int ld, const float* __restrict__ bias,
+                                                                  int experts, int top, int M, int* __restrict__ chosen,
+                                                                  float* __restrict__ weights) {
+    extern __shared__ float smem[];
+    __shared__ float best[kRouterWaves][kMaxTop];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m = blockIdx.x * kRouterWaves + wave;
+    float* z = smem + wave * experts;
+    const bool real = m < M;
+    if (real)
+        for (int e = lane; e < experts; e += 64) z[e] = logits[(size_t)m * ld + e] + bias[e];
+    __syncthreads();
+    if (real)
+        for (int e = lane; e < experts; e += 64) {
+            const int rank = expert_rank(z, experts, e);
+            if (rank < top) {
+                chosen[(size_t)m * top + rank] = e;
+                best[wave][rank] = z[e];
+            }
+        }
+    __syncthreads();
+    if (!real) return;
+    const float w = lane < top ? expf(best[wave][lane] - best[wave][0]) : 0.f, sum = dense_wave_sum(w);
+    if (lane < top) weights[(size_t)m * top + lane] = w / sum;
+}
+static_assert(kMaxTop <= 64, "one weight per lane");
+
+__global__ __launch_bounds__(1024) void expert_rows_kernel(const int* __restrict__ ids, const int* __restrict__ table, int vocab,
                                                          int top, int experts, int M, int* __restrict__ src_rows,
                                                          int* __restrict__ slot_rows, GroupTile* __restrict__ tiles,
                                                          int* __restrict__ n_tiles) {
@@ -177,6 +217,7 @@ __global__ __launch_bounds__(1024) void table_route_kernel(const int* __restrict
     for (int e = t; e < experts; e += 1024) cnt[e] = 0;
     __syncthreads();
     auto expert_of = [&](int i) {
+        if (!ids) return min(max(table[i], 0), experts - 1);
         const int id = min(max(ids[i / top], 0), vocab - 1);
         return min(max(table[(size_t)id * top + i % top], 0), experts - 1);
     };
@@ -233,25 +274,32 @@ hipError_t launch_group_norm(const float* x, int M, int width, const GroupNorm& 
 
 template <typename T>
 hipError_t launch_residual_norm(const float* x, const SublayerOut& y, const GroupNorm& norm_y, const DepthAverage& depth, float* x_out,
-                                const GroupNorm& norm_h, T* h, int ld_h, int M, int width, hipStream_t s) {
+                                const GroupNorm& norm_h, T* h, int ld_h, int M, int width, hipStream_t s, const float* add) {
     const int groups = norm_y.groups > norm_h.groups ? norm_y.groups : norm_h.groups;
     int per = 1;  // what RowParts holds
     while (per < norm_h.groups && per < kThreads) per <<= 1;
     const int size = width / norm_h.groups;
-    if ((!y.y || norm_y.groups == norm_h.groups) && norm_h.groups <= kThreads && size % 4 == 0 &&
+    if ((!y.y || !norm_y.w || norm_y.groups == norm_h.groups) && norm_h.groups <= kThreads && size % 4 == 0 &&
         size / 4 <= RowParts<kThreads>::kParts * (kThreads / per)) {
-        hipLaunchKernelGGL(residual_norm_kernel<T>, dim3(M), dim3(kThreads), 0, s, x, y, norm_y, depth, x_out, norm_h, h, ld_h, width);
+        hipLaunchKernelGGL(residual_norm_kernel<T>, dim3(M), dim3(kThreads), 0, s, x, y, norm_y, depth, x_out, norm_h, h, ld_h, width, add);
     } else {
         const size_t lds = (width + groups + kThreads / 64) * sizeof(float);
-        hipLaunchKernelGGL(residual_norm_any_kernel<T>, dim3(M), dim3(kThreads), lds, s, x, y, norm_y, depth, x_out, norm_h, h, ld_h, width);
+        hipLaunchKernelGGL(residual_norm_any_kernel<T>, dim3(M), dim3(kThreads), lds, s, x, y, norm_y, depth, x_out, norm_h, h, ld_h, width, add);
     }
     return hipGetLastError();
 }
 
-hipError_t launch_table_route(const int* ids, const int* table, int vocab, int top, int experts, int M, int* src_rows,
+hipError_t launch_router(const float* logits, int ld, const float* bias, int experts, int top, int M, int* chosen, float* weights,
+                         hipStream_t s) {
+    hipLaunchKernelGGL(router_kernel, dim3((M + kRouterWaves - 1) / kRouterWaves), dim3(64 * kRouterWaves),
+                       (size_t)kRouterWaves * experts * sizeof(float), s, logits, ld, bias, experts, top, M, chosen, weights);
+    return hipGetLastError();
+}
+
+hipError_t launch_expert_rows(const int* ids, const int* table, int vocab, int top, int experts, int M, int* src_rows,
                               int* slot_rows, GroupTile* tiles, int* n_tiles, hipStream_t s) {
     const size_t lds = (3 * (size_t)experts + 16) * sizeof(int);
-    hipLaunchKernelGGL(table_route_kernel, dim3(1), dim3(1024), lds, s, ids, table, vocab, top, experts, M, src_rows, slot_rows,
+    hipLaunchKernelGGL(expert_rows_kernel, dim3(1), dim3(1024), lds, s, ids, table, vocab, top, experts, M, src_rows, slot_rows,
                        tiles, n_tiles);
     return hipGetLastError();
 }
@@ -259,7 +307,7 @@ hipError_t launch_table_route(const int* ids, const int* table, int vocab, int t
 #define INSTANTIATE(T)                                                                                                          \
     template hipError_t launch_group_norm<T>(const float*, int, int, const GroupNorm&, T*, int, hipStream_t);                     \
     template hipError_t launch_residual_norm<T>(const float*, const SublayerOut&, const GroupNorm&, const DepthAverage&, float*, \
-                                                const GroupNorm&, T*, int, int, int, hipStream_t);
+                                                const GroupNorm&, T*, int, int, int, hipStream_t, const float*);
 INSTANTIATE(bf16)
 INSTANTIATE(float)
 

@@ -57,55 +57,6 @@ __global__ __launch_bounds__(kThreads) void rotate_queries_kernel(const float* _
     }
 }
 
-// One workgroup per (token, head).  Keys in blocks of kBlock: every wave scores a quarter of the block's keys, the block's
-// maximum rescales what is there, then every thread owns some of the output's elements.
-template <typename T, typename O>
-__global__ __launch_bounds__(kThreads) void latent_attention_vector_kernel(const T* __restrict__ q, const T* __restrict__ cache,
-                                                                          LatentShape sh, const int* __restrict__ pos_dev,
-                                                                          int max_seq, O* __restrict__ out, int ld_out) {
-    constexpr int kBlock = 64;
-    extern __shared__ float smem[];
-    float* qs = smem;                        // rank + rot
-    float* acc = qs + sh.rank + sh.rot;      // rank
-    float* p = acc + sh.rank;                // kBlock
-    const int t = threadIdx.x, lane = t & 63, wave = t >> 6, width = sh.rank + sh.rot;
-    const int m = blockIdx.x / sh.heads;
-    const int n_keys = min(max(pos_dev[0] + m, 0), max_seq - 1) + 1;
-    const T* qr = q + (size_t)blockIdx.x * sh.ld_cache;
-    for (int i = t; i < width; i += kThreads) qs[i] = (float)qr[i];
-    for (int i = t; i < sh.rank; i += kThreads) acc[i] = 0.f;
-    float mx = -3.402823466e38f, sum = 0.f;
-    __syncthreads();
-    for (int k0 = 0; k0 < n_keys; k0 += kBlock) {
-        const int nk = min(kBlock, n_keys - k0);
-        for (int k = wave; k < nk; k += kThreads / 64) {
-            const T* row = cache + (size_t)(k0 + k) * sh.ld_cache;
-            float s = 0.f;
-            for (int i = lane; i < width; i += 64) s = fmaf(qs[i], (float)row[i], s);
-            s = dense_wave_sum(s) * sh.scale;
-            if (lane == 0) p[k] = s;
-        }
-        __syncthreads();
-        float bm = -3.402823466e38f;
-        for (int k = 0; k < nk; k++) bm = fmaxf(bm, p[k]);
-        const float nm = fmaxf(mx, bm), keep = expf(mx - nm);
-        __syncthreads();
-        if (t < nk) p[t] = expf(p[t] - nm);
-        __syncthreads();
-        float bs = 0.f;
-        for (int k = 0; k < nk; k++) bs += p[k];
-        sum = sum * keep + bs;
-        mx = nm;
-        for (int i = t; i < sh.rank; i += kThreads) {
-            float a = acc[i] * keep;
-            for (int k = 0; k < nk; k++) a = fmaf(p[k], (float)cache[(size_t)(k0 + k) * sh.ld_cache + i], a);
-            acc[i] = a;
-        }
-        __syncthreads();
-    }
-    for (int i = t; i < sh.rank; i += kThreads) out[(size_t)blockIdx.x * ld_out + i] = (O)(acc[i] / sum);
-}
-
 }  // namespace
 
 template <typename T>
@@ -120,21 +71,6 @@ hipError_t launch_rotate_queries(const float* q, int ld_q, const LatentRows& in,
     hipLaunchKernelGGL(rotate_queries_kernel<T>, dim3(M), dim3(kThreads), 0, s, q, ld_q, in, sh, nope, ld_nope, rot_out, ld_rot);
     return hipGetLastError();
 }
-
-template <typename T, typename O>
-hipError_t launch_latent_attention_vector(const T* q, const T* cache, const LatentShape& sh, const int* pos_dev, int max_seq, int M,
-                                          O* out, int ld_out, hipStream_t s) {
-    const size_t lds = (2 * (size_t)sh.rank + sh.rot + 64) * sizeof(float);
-    hipLaunchKernelGGL((latent_attention_vector_kernel<T, O>), dim3(M * sh.heads), dim3(kThreads), lds, s, q, cache, sh, pos_dev, max_seq,
-                       out, ld_out);
-    return hipGetLastError();
-}
-template hipError_t launch_latent_attention_vector<bf16, bf16>(const bf16*, const bf16*, const LatentShape&, const int*, int, int, bf16*, int,
-                                                               hipStream_t);
-template hipError_t launch_latent_attention_vector<bf16, float>(const bf16*, const bf16*, const LatentShape&, const int*, int, int, float*,
-                                                                int, hipStream_t);
-template hipError_t launch_latent_attention_vector<float, float>(const float*, const float*, const LatentShape&, const int*, int, int,
-                                                                 float*, int, hipStream_t);
 
 #define INSTANTIATE(T)                                                                                                           \
     template hipError_t launch_latent_rows<T>(const LatentRows&, const LatentShape&, int, T*, int, T*, hipStream_t);               \

@@ -8,21 +8,14 @@
 //   X_{i+1} = a + N2b(feed_forward(N2(a)))            (or a, without a feed-forward)
 //   x       = sum_{j <= i+1} dwa_i[j] X_j
 // logits = head N(x).
-#include <algorithm>
-#include <cmath>
 #include <cstring>
-#include <map>
 #include <memory>
-#include <new>
 
-#include "dense.h"
+#include "dense_model.h"
 #include "json.h"
-#include "tensor_source.h"
 
 namespace a81w41 {
 namespace {
-
-constexpr int kPassRows = 4096;  // tokens of one pass; longer portions are cut
 
 struct FeedForwardConfig {
     bool present = false, experts_by_table = false;
@@ -40,10 +33,6 @@ struct Config {
     float eps = 0.f;
     std::vector<LayerConfig> layers;
 };
-
-void require(bool ok, const std::string& what) {
-    if (!ok) throw std::runtime_error(what);
-}
 
 Config read_config(const Json& j) {
     Config c;
@@ -99,33 +88,23 @@ Config read_config(const Json& j) {
     return c;
 }
 
-// Columns of a gate/up pair: 16 gates, their 16 ups, and so on.
-int pair_columns(int ff) { return (ff + 15) / 16 * 32; }
-int pair_row(int j, bool up) { return (j >> 4) * 32 + (up ? 16 : 0) + (j & 15); }
-
-template <typename T>
-struct Weight {  // [rows][ld], K padded with zeros
-    T* data = nullptr;
-    int rows = 0, k = 0, ld = 0;
-};
-
 }  // namespace
 
 template <typename T>
-class TakosunModel final : public a81w41_model {
+class TakosunModel final : public DenseModel<T> {
+    using Base = DenseModel<T>;
+    using Base::cache, Base::ids, Base::logits, Base::max_seq, Base::plan_ctx, Base::pos, Base::stream, Base::want_dev;
+    using Base::allocate_array, Base::finish, Base::init_session, Base::kMatrixAttention, Base::kTable, Base::load_feed_forward,
+        Base::load_matrix, Base::load_rotation, Base::load_vector, Base::product, Base::put_matrix, Base::upload_array;
+    using Staging = typename Base::Staging;
+
    public:
     explicit TakosunModel(Config c) : cfg_(std::move(c)) {}
-    ~TakosunModel() override {
-        if (stream) (void)hipStreamSynchronize(stream);
-        for (void* p : owned_) (void)hipFree(p);
-    }
     int create(int max_seq, TensorSource& src) {
         A81W41_TRY(load_weights(max_seq, src));
         A81W41_TRY(allocate(max_seq));
         return 0;
     }
-    size_t weight_bytes() const override { return weight_bytes_; }
-
     // unfused: one-token passes take the kernels of longer ones; attention: 0 by shape, 1 the vector kernel, 2 in latent
     // space, 3 on formed keys and values; attention_split: shares of the keys in latent space, 0 by length
     int set_option(const char* name, int value) override {
@@ -151,13 +130,10 @@ class TakosunModel final : public a81w41_model {
     }
 
    protected:
-    int ready() const override { return 0; }  // create() loads everything or fails
     int enqueue_pass(int M, const int* want, int n_want, hipStream_t s) override;
 
    private:
-    struct FeedForward {
-        Weight<T> gate_up, down;  // experts: one after the other
-    };
+    using FeedForward = GatedWeights<T>;
     struct Layer {
         float *norm1 = nullptr, *norm1b = nullptr, *norm2 = nullptr, *norm2b = nullptr, *dwa = nullptr;
         float *q_norm = nullptr, *kv_norm = nullptr;
@@ -168,7 +144,6 @@ class TakosunModel final : public a81w41_model {
         T* cache = nullptr;
         float *cos_t = nullptr, *sin_t = nullptr;
     };
-    static constexpr bool kMatrixAttention = sizeof(T) == 2;
     // whether a layer can form its keys and values per head for many new tokens
     static bool can_expand(const LatentShape& sh) {
         return kMatrixAttention && sh.rank % 8 == 0 && attend_expanded_fits(sh.dim, sh.rot, sh.vdim);
@@ -177,92 +152,22 @@ class TakosunModel final : public a81w41_model {
     long long state_step() const { return (long long)rows_ * cfg_.width; }
     GroupNorm norm(const float* w) const { return GroupNorm{w, cfg_.groups, cfg_.eps}; }
 
-    template <typename E>
-    int allocate_array(size_t n, E** out, bool weight = false) {
-        void* p = nullptr;
-        A81W41_HIP_TRY(hipMalloc(&p, std::max<size_t>(n, 1) * sizeof(E)));
-        owned_.push_back(p);
-        A81W41_HIP_TRY(hipMemset(p, 0, std::max<size_t>(n, 1) * sizeof(E)));
-        if (weight) weight_bytes_ += n * sizeof(E);
-        *out = static_cast<E*>(p);
-        return 0;
-    }
-    template <typename E>
-    int upload_array(const std::vector<E>& v, E** out) {
-        A81W41_TRY(allocate_array(v.size(), out, true));
-        A81W41_HIP_TRY(hipMemcpy(*out, v.data(), v.size() * sizeof(E), hipMemcpyHostToDevice));
-        return 0;
-    }
-    // A weight under construction on the host: rows are put one tensor at a time, then it goes to the device.
-    struct Staging {
-        std::vector<T> data;
-        int rows, k, ld;
-        Staging(int rows_, int k_) : data((size_t)rows_ * pad_k<T>(k_)), rows(rows_), k(k_), ld(pad_k<T>(k_)) {}
-        void put(int row, const float* src) {
-            for (int i = 0; i < k; i++) data[(size_t)row * ld + i] = (T)src[i];
-        }
-    };
-    int finish(const Staging& st, Weight<T>* w) {
-        w->rows = st.rows;
-        w->k = st.k;
-        w->ld = st.ld;
-        return upload_array(st.data, &w->data);
-    }
-    int load_vector(TensorSource& src, const std::string& name, int n, float** out) {
-        std::vector<float> v;
-        A81W41_TRY(src.matrix(name, 0, n, v));
-        return upload_array(v, out);
-    }
-    int put_matrix(TensorSource& src, const std::string& name, int rows, int k, Staging& st, int row0) {
-        std::vector<float> v;
-        A81W41_TRY(src.matrix(name, rows, k, v));
-        for (int r = 0; r < rows; r++) st.put(row0 + r, v.data() + (size_t)r * k);
-        return 0;
-    }
-    int load_matrix(TensorSource& src, const std::string& name, int rows, int k, Weight<T>* w) {
-        Staging st(rows, k);
-        A81W41_TRY(put_matrix(src, name, rows, k, st, 0));
-        return finish(st, w);
-    }
-    int load_feed_forward(TensorSource& src, const std::vector<std::string>& prefixes, int ff, FeedForward* out) {
-        const int n = (int)prefixes.size(), width = cfg_.width, cols = pair_columns(ff);
-        Staging gu(n * cols, width), down(n * width, ff);
-        std::vector<float> v;
-        for (int e = 0; e < n; e++) {
-            for (int up = 0; up < 2; up++) {
-                A81W41_TRY(src.matrix(prefixes[e] + (up ? "up" : "gate"), ff, width, v));
-                for (int j = 0; j < ff; j++) gu.put(e * cols + pair_row(j, up), v.data() + (size_t)j * width);
-            }
-            A81W41_TRY(put_matrix(src, prefixes[e] + "down", width, ff, down, e * width));
-        }
-        A81W41_TRY(finish(gu, &out->gate_up));
-        return finish(down, &out->down);
-    }
     int load_weights(int max_seq, TensorSource& src);
-    int load_rotation(const LayerConfig& lc, int max_seq, Layer* L);
     int allocate(int max_seq);
     int attention(const Layer& L, const LayerConfig& lc, int M, hipStream_t s);
     int attend_latent(const Layer& L, const LatentShape& sh, int M, hipStream_t s);
     int attend_formed(const Layer& L, const LatentShape& sh, int M, const float* gates, hipStream_t s);
-    AttendArgs shared_attend(const Layer& L, const LatentShape& sh, int M) const;
+    AttendArgs<T> shared_attend(const Layer& L, const LatentShape& sh, int M) const;
     int enqueue_one_token(int n_want, hipStream_t s);
     int feed_forward_one_token(const Layer& L, const LayerConfig& lc, const RowStep& step, hipStream_t s);
     LatentRows latent_rows(const Layer& L) const;
     int feed_forward(const Layer& L, const LayerConfig& lc, int M, hipStream_t s, SublayerOut* out);
     int pair_product(const FeedForward& f, int ff, const T* h, const GemmArgs& base, T* act, hipStream_t s);
-    GemmArgs product(const T* A, int lda, const Weight<T>& w, void* C, int ldc, int M) const {
-        GemmArgs g;
-        g.A = A, g.lda = lda, g.W = w.data, g.ldw = w.ld, g.K = w.ld, g.N = w.rows, g.C = C, g.ldc = ldc, g.M = M;
-        return g;
-    }
 
     Config cfg_;
     std::vector<Layer> layers_;
     Weight<T> embed_, head_;
     float* final_norm_ = nullptr;
-    std::vector<void*> owned_;
-    size_t weight_bytes_ = 0;
-    std::map<std::pair<int, double>, std::pair<float*, float*>> rotations_;
     // activations of one pass
     int rows_ = 0, ld_h_ = 0, ld_down_ = 0, ld_q_ = 0, ld_cq_ = 0, ld_attn_ = 0;
     float *x_ = nullptr, *states_ = nullptr, *down_ = nullptr, *q_ = nullptr, *y_ = nullptr, *y2_ = nullptr, *y_shared_ = nullptr;
@@ -281,27 +186,6 @@ class TakosunModel final : public a81w41_model {
     int *src_rows_ = nullptr, *slot_rows_ = nullptr, *n_tiles_ = nullptr;
     GroupTile* tiles_ = nullptr;
 };
-
-template <typename T>
-int TakosunModel<T>::load_rotation(const LayerConfig& lc, int max_seq, Layer* L) {
-    auto& slot = rotations_[{lc.mix.rot, lc.rot_base}];
-    if (!slot.first) {
-        const int half = lc.mix.rot / 2;
-        std::vector<float> cs((size_t)max_seq * half), sn(cs.size());
-        for (int i = 0; i < half; i++) {
-            const double f = std::pow(lc.rot_base, -2.0 * i / lc.mix.rot);
-            for (int p = 0; p < max_seq; p++) {
-                cs[(size_t)p * half + i] = (float)std::cos(p * f);
-                sn[(size_t)p * half + i] = (float)std::sin(p * f);
-            }
-        }
-        A81W41_TRY(upload_array(cs, &slot.first));
-        A81W41_TRY(upload_array(sn, &slot.second));
-    }
-    L->cos_t = slot.first;
-    L->sin_t = slot.second;
-    return 0;
-}
 
 template <typename T>
 int TakosunModel<T>::load_weights(int max_seq, TensorSource& src) {
@@ -333,7 +217,7 @@ int TakosunModel<T>::load_weights(int max_seq, TensorSource& src) {
         }
         A81W41_TRY(put_matrix(src, mix + "g", sh.heads, width, down, sh.q_rank + kv));
         A81W41_TRY(finish(down, &L.down));
-        A81W41_TRY(load_rotation(lc, max_seq, &L));
+        A81W41_TRY(load_rotation(sh.rot, lc.rot_base, max_seq, &L.cos_t, &L.sin_t));
         A81W41_TRY(load_matrix(src, mix + "uq", sh.heads * (sh.dim + sh.rot), sh.q_rank, &L.uq));
         {   // the key up-projection of a head, transposed: it maps an unrotated query to latent space
             std::vector<float> uk, row(sh.dim);
@@ -358,13 +242,13 @@ int TakosunModel<T>::load_weights(int max_seq, TensorSource& src) {
         A81W41_TRY(load_vector(src, p + "norm2", width, &L.norm2));
         A81W41_TRY(load_vector(src, p + "norm2b", width, &L.norm2b));
         if (!f.experts_by_table) {
-            A81W41_TRY(load_feed_forward(src, {mlp}, f.ff, &L.ff));
+            A81W41_TRY(load_feed_forward(src, {mlp}, width, f.ff, &L.ff));
             continue;
         }
         std::vector<std::string> names;
         for (int e = 0; e < f.experts; e++) names.push_back(mlp + "e" + std::to_string(e) + ".");
-        A81W41_TRY(load_feed_forward(src, names, f.ff, &L.ff));
-        if (f.shared_ff) A81W41_TRY(load_feed_forward(src, {mlp + "shared."}, f.shared_ff, &L.shared));
+        A81W41_TRY(load_feed_forward(src, names, width, f.ff, &L.ff));
+        if (f.shared_ff) A81W41_TRY(load_feed_forward(src, {mlp + "shared."}, width, f.shared_ff, &L.shared));
         std::vector<int> table;
         A81W41_TRY(src.table(mlp + "table", cfg_.vocab, f.top, f.experts, table));
         A81W41_TRY(upload_array(table, &L.table));
@@ -456,10 +340,10 @@ LatentRows TakosunModel<T>::latent_rows(const Layer& L) const {
 
 // Query rows q_lat_ (like cache rows) against the layer's cache.
 template <typename T>
-AttendArgs TakosunModel<T>::shared_attend(const Layer& L, const LatentShape& sh, int M) const {
-    AttendArgs a;
-    a.q = reinterpret_cast<const bf16*>(q_lat_), a.ld_q = sh.ld_cache, a.rows = M * sh.heads, a.rows_per_token = sh.heads;
-    a.k_own = reinterpret_cast<const bf16*>(L.cache), a.ld_k_own = sh.ld_cache, a.k_own_width = (sh.rank + sh.rot + 7) / 8 * 8;
+AttendArgs<T> TakosunModel<T>::shared_attend(const Layer& L, const LatentShape& sh, int M) const {
+    AttendArgs<T> a;
+    a.q = q_lat_, a.ld_q = sh.ld_cache, a.q_token = sh.heads * sh.ld_cache, a.rows = M * sh.heads, a.rows_per_token = sh.heads;
+    a.k_own = L.cache, a.ld_k_own = sh.ld_cache, a.k_own_width = (sh.rank + sh.rot + 7) / 8 * 8;
     a.dv = sh.rank, a.scale = sh.scale, a.pos_dev = pos, a.max_seq = max_seq();
     a.part = part_, a.part_stats = part_stats_, a.ld_part = (sh.rank + 3) / 4 * 4;
     // enough workgroups for the chip, at least 64 keys for each
@@ -482,14 +366,18 @@ int TakosunModel<T>::attend_latent(const Layer& L, const LatentShape& sh, int M,
     bool done = false;
     if constexpr (kMatrixAttention) {
         if (opt_attention_ != 1 && attend_shared_fits(sh.rank + sh.rot, sh.rank)) {
-            AttendArgs a = shared_attend(L, sh, M);
-            a.out = o_lat_, a.ld_out = ld_rank;
+            AttendArgs<T> a = shared_attend(L, sh, M);
+            a.out = o_lat_, a.ld_out = ld_rank, a.out_token = sh.heads * ld_rank;
             A81W41_HIP_TRY(launch_attend_shared(a, s));
-            if (a.splits > 1) A81W41_HIP_TRY(launch_merge_shares(a, s));
+            if (a.splits > 1) A81W41_HIP_TRY(launch_merge_shares(a, 1, s));
             done = true;
         }
     }
-    if (!done) A81W41_HIP_TRY((launch_latent_attention_vector<T, T>(q_lat_, L.cache, sh, pos, max_seq(), M, o_lat_, ld_rank, s)));
+    if (!done) {
+        AttendArgs<T> a = shared_attend(L, sh, M);
+        a.ld_out = ld_rank, a.out_token = sh.heads * ld_rank;
+        A81W41_HIP_TRY((launch_attend_vector<T, T>(a, 1, o_lat_, s)));
+    }
     return 0;
 }
 
@@ -505,13 +393,13 @@ int TakosunModel<T>::attend_formed(const Layer& L, const LatentShape& sh, int M,
         g.C = v_formed_, g.ldc = ld_v_;
         A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kElement, s));
         A81W41_HIP_TRY(launch_rotate_queries<T>(q_, ld_q_, latent_rows(L), sh, M, nope_, dk, nope_ + sh.dim, dk, s));
-        AttendArgs a;
-        a.q = nope_, a.q_head = dk, a.ld_q = sh.heads * dk, a.rows = M;
+        AttendArgs<T> a;
+        a.q = nope_, a.q_head = dk, a.q_token = sh.heads * dk, a.rows = M;
         a.k_own = k_formed_, a.k_own_head = sh.dim, a.ld_k_own = sh.heads * sh.dim, a.k_own_width = sh.dim;
         a.k_shared = L.cache + sh.rank, a.ld_k_shared = sh.ld_cache, a.k_shared_width = sh.rot;
         a.v_t = v_formed_, a.ld_v = ld_v_, a.dv = sh.vdim;
         a.head_gate = gates, a.ld_gate = ld_down_;
-        a.out = attn_, a.out_head = sh.vdim, a.ld_out = ld_attn_;
+        a.out = attn_, a.out_head = sh.vdim, a.out_token = ld_attn_;
         a.scale = sh.scale, a.pos_dev = pos, a.max_seq = max_seq();
         A81W41_HIP_TRY(launch_attend_expanded(a, sh.heads, s));
     }
@@ -550,7 +438,7 @@ int TakosunModel<T>::feed_forward(const Layer& L, const LayerConfig& lc, int M, 
     const int W = cfg_.width;
     auto two_products = [&](const FeedForward& w, int ff, float* y) -> int {
         const int ld = pad_k<T>(ff);
-        A81W41_HIP_TRY(launch_dense_gemm<T>(product(h_, ld_h_, w.gate_up, act_, ld, M), Epilogue::kSiluPair, s));
+        A81W41_HIP_TRY(launch_dense_gemm<T>(product(h_, ld_h_, w.gate_up, act_, ld, M), Epilogue::kGatedPair, s));
         A81W41_HIP_TRY(launch_dense_gemm<T>(product(act_, ld, w.down, y, W, M), Epilogue::kFloat, s));
         return 0;
     };
@@ -561,12 +449,12 @@ int TakosunModel<T>::feed_forward(const Layer& L, const LayerConfig& lc, int M, 
         A81W41_TRY(two_products(L.shared, f.shared_ff, y_shared_));
         out->shared = y_shared_;
     }
-    A81W41_HIP_TRY(launch_table_route(ids, L.table, cfg_.vocab, f.top, f.experts, M, src_rows_, slot_rows_, tiles_, n_tiles_, s));
+    A81W41_HIP_TRY(launch_expert_rows(ids, L.table, cfg_.vocab, f.top, f.experts, M, src_rows_, slot_rows_, tiles_, n_tiles_, s));
     const int ld = pad_k<T>(f.ff), cols = pair_columns(f.ff);
     GemmArgs g = product(h_, ld_h_, L.ff.gate_up, act_, ld, M * f.top);
     g.N = cols, g.w_step = (long long)cols * L.ff.gate_up.ld, g.a_rows = src_rows_;
     g.tiles = tiles_, g.n_tiles = n_tiles_, g.max_tiles = M * f.top / kGroupTileRows + std::min(f.experts, M * f.top);
-    A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kSiluPair, s));
+    A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kGatedPair, s));
     g.A = act_, g.lda = ld, g.a_rows = nullptr, g.W = L.ff.down.data, g.ldw = g.K = L.ff.down.ld;
     g.N = W, g.w_step = (long long)W * L.ff.down.ld, g.C = y2_, g.ldc = W;
     A81W41_HIP_TRY(launch_dense_gemm<T>(g, Epilogue::kFloat, s));
@@ -586,7 +474,7 @@ int TakosunModel<T>::feed_forward_one_token(const Layer& L, const LayerConfig& l
         e.ids = ids, e.table = L.table, e.vocab = cfg_.vocab, e.top = f.top, e.experts = f.experts, e.ff = f.ff;
         e.pair_rows = pair_columns(f.ff);
     }
-    A81W41_HIP_TRY(launch_gemv_gate_up<T>(step, e, L.ff.gate_up.data, every.gate_up.data, L.ff.gate_up.ld, act_row_, s));
+    A81W41_HIP_TRY(launch_gemv_gate_up<T>(step, nullptr, e, L.ff.gate_up.data, every.gate_up.data, L.ff.gate_up.ld, act_row_, s));
     A81W41_HIP_TRY(launch_gemv_ff_down<T>(e, act_row_, L.ff.down.data, L.ff.down.ld, every.down.data, every.down.ld, cfg_.width, y_ff_, s));
     return 0;
 }
@@ -597,7 +485,7 @@ int TakosunModel<T>::feed_forward_one_token(const Layer& L, const LayerConfig& l
 template <typename T>
 int TakosunModel<T>::enqueue_one_token(int n_want, hipStream_t s) {
     const int W = cfg_.width, n = n_layers();
-    A81W41_HIP_TRY(launch_embed_rows(ids, embed_.data, sizeof(T) == 2 ? TableType::kBf16 : TableType::kFp32, embed_.ld, states_, 1, W,
+    A81W41_HIP_TRY(launch_embed_rows(ids, embed_.data, kTable, embed_.ld, states_, 1, W,
                                      cfg_.vocab, s));
     RowStep step;  // what the next product's prologue does
     step.x = states_, step.width = W, step.norm_h = norm(layers_[0].norm1);
@@ -617,14 +505,17 @@ int TakosunModel<T>::enqueue_one_token(int n_want, hipStream_t s) {
         LatentShares shares;
         if constexpr (kMatrixAttention) {
             if (opt_attention_ != 1 && attend_shared_fits(sh.rank + sh.rot, sh.rank)) {
-                AttendArgs a = shared_attend(L, sh, 1);
+                AttendArgs<T> a = shared_attend(L, sh, 1);
                 a.splits = std::max(a.splits, 2);  // shares stay fp32; the product with W_uv merges them
                 A81W41_HIP_TRY(launch_attend_shared(a, s));
                 shares = LatentShares{a.part, a.part_stats, a.splits, a.ld_part};
             }
         }
-        if (!shares.part)
-            A81W41_HIP_TRY((launch_latent_attention_vector<T, float>(q_lat_, L.cache, sh, pos, max_seq(), 1, o_lat_row_, ld_rank, s)));
+        if (!shares.part) {
+            AttendArgs<T> a = shared_attend(L, sh, 1);
+            a.ld_out = ld_rank, a.out_token = sh.heads * ld_rank;
+            A81W41_HIP_TRY((launch_attend_vector<T, float>(a, 1, o_lat_row_, s)));
+        }
         A81W41_HIP_TRY(launch_gemv_values<T>(o_lat_row_, ld_rank, shares, sh, L.uv.data, L.uv.ld, down_ + sh.q_rank + (own ? sh.rank + sh.rot : 0),
                                              attn_row_, s));
         A81W41_HIP_TRY(launch_gemv_plain<T>(attn_row_, sh.heads * sh.vdim, L.o.data, L.o.ld, W, y_, s));
@@ -649,7 +540,7 @@ int TakosunModel<T>::enqueue_pass(int M, const int* want, int n_want, hipStream_
     (void)want;  // the head product reads want_dev
     if (M == 1 && one_token_fits_ && !opt_unfused_) return enqueue_one_token(n_want, s);
     const int W = cfg_.width, n = n_layers();
-    A81W41_HIP_TRY(launch_embed_rows(ids, embed_.data, sizeof(T) == 2 ? TableType::kBf16 : TableType::kFp32, embed_.ld, states_, M, W,
+    A81W41_HIP_TRY(launch_embed_rows(ids, embed_.data, kTable, embed_.ld, states_, M, W,
                                      cfg_.vocab, s));
     A81W41_HIP_TRY(launch_group_norm<T>(states_, M, W, norm(layers_[0].norm1), h_, ld_h_, s));
     const float* x = states_;
@@ -683,22 +574,8 @@ int TakosunModel<T>::enqueue_pass(int M, const int* want, int n_want, hipStream_
 
 namespace {
 
-template <typename T>
-int create_model(const Config& c, const LoadRequest& req, TensorSource& src, a81w41_model** out) {
-    auto m = std::make_unique<TakosunModel<T>>(c);
-    A81W41_TRY(m->create(req.max_seq, src));
-    *out = m.release();
-    return 0;
-}
-
 int load_registered(const LoadRequest& req, a81w41_model** out) {
-    const Config c = read_config(*req.config);
-    std::unique_ptr<TensorSource> src;
-    if (req.random_weights)
-        src = random_tensors(req.seed);
-    else
-        A81W41_TRY(open_safetensors(req.dir + "/model.safetensors", &src));
-    return req.dtype == "float32" ? create_model<float>(c, req, *src, out) : create_model<bf16>(c, req, *src, out);
+    return create_dense_model<TakosunModel>(read_config(*req.config), req, out);
 }
 const RegisterModel registered("Takosun", load_registered);
 

@@ -20,6 +20,7 @@ from . import capi
 ARCHITECTURES = {
     "Qwen3": (capi.lib, capi.LIB_PATH, "liba81w41.so"),
     "Takosun": (capi.dense, capi.DENSE_PATH, "dense"),
+    "Dimesun": (capi.dense, capi.DENSE_PATH, "dense"),
 }
 
 
