@@ -22,7 +22,8 @@ Also reported in the same JSON line:
   m_sweep       forward at M in {1, 8, 32, 128, 512, 2048} on gate and down
   e2e           random-init Qwen3-8B: 322-token prefill + 128 greedy decode steps, resident bytes
   a80w40        the A80W40 variant's GEMV sweep and M=322 GEMM
-  (--takosun [SIZE] runs the Takosun model beside Qwen3 at equal size instead and prints that object)
+  (--takosun [SIZE] runs the Takosun model beside Qwen3 at equal size instead and prints that object; --dimesun [SIZE]
+   the Dimesun model beside Takosun)
 Every figure is the median of five timed windows (the minimum is reported beside it).
   cpu_baseline  the AVX2+OpenMP port of the reference's CPU path on this host
 """
@@ -63,6 +64,13 @@ TAKOSUN_SIZES = {
     "4k": dict(width=4096, heads=32, q_rank=1536, ff=12288, layers=8),
     "2k-moe": dict(width=2048, heads=16, q_rank=768, ff=6144, layers=12, experts=64, top=6, expert_ff=1024, shared_ff=1024),
 }
+# Layers of the Dimesun leg: attention and matrix memory in turn, `layers` of them run twice.
+DIMESUN_SIZES = {
+    "2k": dict(width=2048, heads=16, kv_heads=4, chunk=1024, memory_heads=8, memory_dim=128, memory_vdim=256, experts=32, top=4, ff=1024,
+               layers=6),
+    "4k": dict(width=4096, heads=32, kv_heads=8, chunk=2048, memory_heads=8, memory_dim=256, memory_vdim=512, experts=16, top=4, ff=2048,
+               layers=4),
+}
 
 
 def gemv_bytes(K, N):
@@ -93,6 +101,11 @@ def parse():
                          "(prints its JSON object)")
     ap.add_argument("--takosun-prompt", type=int, default=2048)
     ap.add_argument("--takosun-no-qwen", action="store_true", help="leave the Qwen3 runs of --takosun out (for profiles)")
+    ap.add_argument("--dimesun", nargs="?", const="all", choices=["all"] + sorted(DIMESUN_SIZES), metavar="SIZE",
+                    help="run only the Dimesun model at sizes like a real model's layers, beside Takosun at equal size "
+                         "(prints its JSON object)")
+    ap.add_argument("--dimesun-prompt", type=int, default=2048)
+    ap.add_argument("--dimesun-no-takosun", action="store_true", help="leave the Takosun runs of --dimesun out (for profiles)")
     ap.add_argument("--no-m-sweep", action="store_true", help="skip the M sweep on the gate and down shapes")
     ap.add_argument("--no-e2e", action="store_true",
                     help="skip the random-init Qwen3-8B forward pass (322-token prefill + 128 greedy decode steps; "
@@ -162,6 +175,10 @@ def main():
 
     if args.takosun:
         print(json.dumps(takosun_leg(pkg, args.takosun, args.takosun_prompt, with_qwen=not args.takosun_no_qwen)), flush=True)
+        return
+
+    if args.dimesun:
+        print(json.dumps(dimesun_leg(pkg, args.dimesun, args.dimesun_prompt, with_takosun=not args.dimesun_no_takosun)), flush=True)
         return
 
     if args.e2e_only:
@@ -666,9 +683,78 @@ def takosun_work(cfg, n_prompt):
         kv = 0 if "kv_from" in m else m["kv_rank"] + m["rot_dim"]
         weights += W * (m["q_rank"] + kv + m["heads"]) + m["q_rank"] * m["heads"] * (m["dim"] + m["rot_dim"])
         weights += m["heads"] * (m["dim"] + m["vdim"]) * m["kv_rank"] + W * m["heads"] * m["vdim"]
-        weights += 3 * W * (f["ff"] if f["kind"] == "dense" else f["router"]["top"] * f["expert"]["ff"] + f["shared"]["ff"])
+        weights += 3 * W * (f["ff"] if f["kind"] == "dense" else f["router"]["top"] * f["expert"]["ff"] + f.get("shared", {"ff": 0})["ff"])
         attn += n_prompt * (n_prompt + 1) // 2 * m["heads"] * (m["dim"] + m["rot_dim"] + m["vdim"]) * 2
     return 2 * weights, 2 * (weights - cfg["vocab"] * W) * n_prompt, attn
+
+
+def rates(n_prompt, ms_pre, n_decode, ms_dec, nbytes, flops, attn):
+    return {"prefill_tokens": n_prompt, "prefill_ms": round(ms_pre, 3), "prefill_tokens_per_s": round(n_prompt / ms_pre * 1e3, 1),
+            "prefill_TFLOPS": round((flops + attn) / ms_pre / 1e9, 1), "prefill_attention_share_of_flops": round(attn / (flops + attn), 3),
+            "decode_ms_per_token": round(ms_dec / n_decode, 4), "decode_tokens_per_s": round(n_decode / ms_dec * 1e3, 1),
+            "decode_weight_MB_per_token": round(nbytes / 1e6, 1), "decode_GBps": round(nbytes / (ms_dec / n_decode) / 1e6, 1),
+            "decode_hbm_frac": round(nbytes / (ms_dec / n_decode) / 1e6 / HBM_PEAK_GBS, 4)}
+
+
+def random_model_rates(pkg, cfg, work, n_prompt, n_decode, label):
+    t0 = time.time()
+    model = pkg.Model.random(cfg, n_prompt + n_decode + 2, "bfloat16", seed=1)
+    print(f"[bench] {label} resident after {time.time() - t0:.1f}s", file=sys.stderr, flush=True)
+    prompt = np.random.default_rng(7).integers(0, cfg["vocab"], n_prompt).astype(np.int32)
+    _, ms_pre, ms_dec = time_generation(model, prompt, n_decode)
+    print(f"[bench] {label} prefill {ms_pre:.3f} ms, decode {ms_dec / n_decode:.4f} ms per token", file=sys.stderr, flush=True)
+    model.close()
+    return rates(n_prompt, ms_pre, n_decode, ms_dec, *work(cfg, n_prompt))
+
+
+def dimesun_config(size):
+    d = DIMESUN_SIZES[size]
+    mlp = {"kind": "moe", "router": {"experts": d["experts"], "top": d["top"]}, "expert": {"ff": d["ff"], "limit": 7.0}}
+    attention = {"heads": d["heads"], "kv_heads": d["kv_heads"], "dim": 128, "vdim": 128, "rot": {"base": 10000.0, "dims": 64},
+                 "mask": {"size": d["chunk"]}, "scale": 128.0 ** -0.5}
+    memory = {"heads": d["memory_heads"], "dim": d["memory_dim"], "vdim": d["memory_vdim"], "gate_cap": 15.0}
+    layers = [{"type": "mlstm", "mixer": memory, "mlp": mlp} if i % 2 else {"type": "attention", "mixer": attention, "mlp": mlp}
+              for i in range(d["layers"])]
+    return {"architecture": "Dimesun", "vocab": 32768, "width": d["width"], "norm": {"eps": 1e-6}, "residual_mult": 0.5, "layers": layers,
+            "loop": {"start": 0, "stop": d["layers"], "times": 2}}
+
+
+def dimesun_work(cfg, n_prompt):
+    """Like takosun_work; the bytes hold the matrix memories' states too, the operations outside attention their updates and
+    reads (not the products inside a chunk of a prompt)."""
+    W, head = cfg["width"], cfg["vocab"] * cfg["width"]
+    weights, states, attn = 0, 0, 0
+    for l in cfg["layers"]:
+        m, f = l["mixer"], l["mlp"]
+        if l["type"] == "mlstm":
+            weights += W * m["heads"] * (2 * m["dim"] + 2 * m["vdim"] + 2) + W * m["heads"] * m["vdim"]
+            states += m["heads"] * m["dim"] * m["vdim"]
+        else:
+            weights += W * (m["heads"] * m["dim"] + m["kv_heads"] * (m["dim"] + m["vdim"])) + W * m["heads"] * m["vdim"]
+            pairs = sum(p % m["mask"]["size"] + 1 for p in range(n_prompt))
+            attn += pairs * m["heads"] * (m["dim"] + m["vdim"]) * 2
+        weights += W * f["router"]["experts"] + 3 * W * f["router"]["top"] * f["expert"]["ff"]
+    times = cfg["loop"]["times"]   # every layer is in the loop
+    weights, states, attn = weights * times, states * times, attn * times
+    return 2 * (weights + head) + 8 * states, 2 * (weights + 2 * states) * n_prompt, attn
+
+
+def dimesun_leg(pkg, which, n_prompt=2048, n_decode=128, with_takosun=True):
+    """Prefill and decode rates of Dimesun (seeded random weights) and, at equal width, heads, experts, vocabulary and as many
+    layers as Dimesun has layer runs, of Takosun.  A repeated layer's weights are read once per run in both counts."""
+    out = {}
+    for size in sorted(DIMESUN_SIZES) if which == "all" else [which]:
+        d = DIMESUN_SIZES[size]
+        out[size] = dict(random_model_rates(pkg, dimesun_config(size), dimesun_work, n_prompt, n_decode, f"Dimesun {size}"), config=d)
+        if with_takosun:
+            mixer = {"heads": d["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": d["width"] * 3 // 8, "kv_rank": 512,
+                     "scale": 192.0 ** -0.5, "rot": {"base": 10000.0, "dims": 64}}
+            mlp = {"kind": "moe", "router": {"experts": d["experts"], "top": d["top"]}, "expert": {"ff": d["ff"]}}
+            cfg = {"architecture": "Takosun", "vocab": 32768, "width": d["width"], "norm": {"eps": 1e-6, "groups": 1},
+                   "layers": [{"type": "latent_attention", "mixer": dict(mixer, kv_from=i - 1) if i % 2 else mixer, "mlp": mlp}
+                              for i in range(2 * d["layers"])]}
+            out[size]["takosun_equal_size"] = random_model_rates(pkg, cfg, takosun_work, n_prompt, n_decode, f"Takosun like {size}")
+    return out
 
 
 def takosun_leg(pkg, which, n_prompt=2048, n_decode=128, with_qwen=True):
@@ -677,23 +763,12 @@ def takosun_leg(pkg, which, n_prompt=2048, n_decode=128, with_qwen=True):
     out = {}
     for size in sorted(TAKOSUN_SIZES) if which == "all" else [which]:
         cfg = takosun_config(size)
-        max_seq = n_prompt + n_decode + 2
-        t0 = time.time()
-        model = pkg.Model.random(cfg, max_seq, "bfloat16", seed=1)
-        print(f"[bench] Takosun {size} resident after {time.time() - t0:.1f}s", file=sys.stderr, flush=True)
-        prompt = np.random.default_rng(7).integers(0, cfg["vocab"], n_prompt).astype(np.int32)
-        toks, ms_pre, ms_dec = time_generation(model, prompt, n_decode)
-        nbytes, flops, attn = takosun_work(cfg, n_prompt)
-        row = {"prefill_tokens": n_prompt, "prefill_ms": round(ms_pre, 3), "prefill_tokens_per_s": round(n_prompt / ms_pre * 1e3, 1),
-               "prefill_TFLOPS": round((flops + attn) / ms_pre / 1e9, 1), "prefill_attention_share_of_flops": round(attn / (flops + attn), 3),
-               "decode_ms_per_token": round(ms_dec / n_decode, 4), "decode_tokens_per_s": round(n_decode / ms_dec * 1e3, 1),
-               "decode_weight_MB_per_token": round(nbytes / 1e6, 1), "decode_GBps": round(nbytes / (ms_dec / n_decode) / 1e6, 1),
-               "decode_hbm_frac": round(nbytes / (ms_dec / n_decode) / 1e6 / HBM_PEAK_GBS, 4), "config": TAKOSUN_SIZES[size]}
-        model.close()
+        row = dict(random_model_rates(pkg, cfg, takosun_work, n_prompt, n_decode, f"Takosun {size}"), config=TAKOSUN_SIZES[size])
         if with_qwen and "experts" not in TAKOSUN_SIZES[size]:
             d = TAKOSUN_SIZES[size]
             q = dict(n_layers=d["layers"], hidden=d["width"], n_q_heads=d["heads"], n_kv_heads=d["heads"] // 4, intermediate=d["ff"],
-                     vocab=cfg["vocab"], max_seq=max_seq)
+                     vocab=cfg["vocab"], max_seq=n_prompt + n_decode + 2)
+            prompt = np.random.default_rng(7).integers(0, cfg["vocab"], n_prompt).astype(np.int32)
             qwen, _, n_w = build_e2e_model(pkg, n_prompt, q)
             _, ms_pre, ms_dec = time_generation(qwen, prompt, n_decode)
             qbytes = 0.625 * n_w

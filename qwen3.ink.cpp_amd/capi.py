@@ -107,6 +107,11 @@ DENSE_SIGNATURES = {
     "a81w41_dense_gemm": (_i, [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _vp]),
     "a81w41_latent_attention": (_i, [_vp, _vp, _i, _i, _i, _i, _vp, _i, _i, C.c_float, _vp, _i, _i, _i, _vp, _vp, _vp]),
     "a81w41_formed_attention": (_i, [_vp, _vp, _vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _vp, _i, _i, C.c_float, _vp, _vp]),
+    "a81w41_grouped_attention": (_i, [_vp, _vp, _i, _i, _i, _i, _i, _i, _vp, _i, _i, C.c_float, _i, _i, _vp, _i, _i, _i, _vp, _vp, _vp]),
+    "a81w41_matrix_memory_state": (_sz, [_i, _i, _i]),
+    "a81w41_matrix_memory_scratch": (_sz, [_i, _i, _i, _i]),
+    "a81w41_matrix_memory": (_i, [_vp, _i, _i, _i, _i, _i, C.c_float, C.c_float, _vp, _vp, _vp, _vp, _vp, _i, _vp, _vp, _vp]),
+    "a81w41_router": (_i, [_vp, _i, _vp, _i, _i, _i, _vp, _vp, _vp]),
 }
 
 

@@ -215,6 +215,12 @@ struct MemoryShape {
     int heads = 0, dim = 0, vdim = 0;
     float cap = 1.f, q_scale = 1.f, eps = 0.f;
     int at_q = 0, at_k = 0, at_v = 0, at_g = 0, at_i = 0, at_f = 0;
+    // columns in this order; the first one behind them
+    int place_columns() {
+        at_q = 0, at_k = at_q + heads * dim, at_v = at_k + heads * dim, at_g = at_v + heads * vdim, at_i = at_g + heads * vdim;
+        at_f = at_i + heads;
+        return at_f + heads;
+    }
     // floats of a sequence's state: S of all heads, then two copies of [n dim | m] per head: the one of parity p is valid at
     // positions of that parity, so that workgroups can read one while another is written
     __host__ __device__ size_t s_size() const { return (size_t)heads * dim * vdim; }
@@ -297,8 +303,9 @@ hipError_t launch_gemv_gate_up(const RowStep& p, const float* h, const ExpertRow
 template <typename T>
 hipError_t launch_gemv_ff_down(const ExpertRows& e, const float* act, const T* experts, int ld, const T* dense, int ld_dense, int N,
                                float* y, hipStream_t s);
-// What a mixer leaves for its output product, one row of `width`: attention's (merged from its shares if there are any:
-// `heads` rows of `vdim`), or a matrix memory's before its norm and gate.
+// What a mixer leaves for its output product, one row of `width`: attention's (merged from its shares if there are any, at
+// most kMixerShares: `heads` rows of `vdim`; every workgroup of the product repeats the merge), or a matrix memory's before its norm and gate.
+constexpr int kMixerShares = 8;
 struct MixerRow {
     const float* row = nullptr;
     int width = 0;

@@ -538,85 +538,194 @@ __global__ __launch_bounds__(kThreads) void gemv_ff_down_kernel(ExpertRows e, co
     }
 }
 
-// The mixer's row into xs (LDS, zero-padded).  inv: a float for every head, or for every head and share.
-__device__ __forceinline__ void form_mixer_row(const MixerRow& m, float* xs, int padded, float* inv, float* red) {
-    const int t = threadIdx.x;
-    if (m.shares.part) {  // per head sum_k w_k share_k / sum_k w_k sum_k, w_k = 2^(maximum_k - largest)
-        const int n = m.shares.splits, H = m.heads;
-        for (int h = t; h < H; h += kThreads) {
-            float top = -3.402823466e38f;
-            for (int k = 0; k < n; k++) top = fmaxf(top, m.shares.stats[2 * ((size_t)k * H + h)]);
-            float all = 0.f;
-            for (int k = 0; k < n; k++) {
-                const float w = exp2f(m.shares.stats[2 * ((size_t)k * H + h)] - top);
-                inv[h * n + k] = w;
-                all = fmaf(w, m.shares.stats[2 * ((size_t)k * H + h) + 1], all);
+// The mixer's row: load() requests what a thread will need of it, finish() puts it into xs (LDS, zero-padded; ends without
+// a barrier).  inv: LDS, a float for every head, or for every head and share.
+class MixerPrologue {
+   public:
+    __device__ __forceinline__ explicit MixerPrologue(const MixerRow& m)
+        : m_(m), parts_(m.width, m.norm ? m.heads : 1), quads_(m.shares.part && m.vdim % 4 == 0), normed_(m.norm && parts_.fits()) {}
+    __device__ __forceinline__ void load() {
+        const int t = threadIdx.x;
+        if (quads_) {
+            if (t < m_.heads) {
+#pragma unroll
+                for (int k = 0; k < kShares; k++) stats_[k] = stat(min(k, m_.shares.splits - 1), t);
             }
-            for (int k = 0; k < n; k++) inv[h * n + k] /= all;
+            request_shares(0);
+        } else if (normed_) {
+#pragma unroll
+            for (int k = 0; k < RowParts<kThreads>::kParts; k++) {
+                const int i = parts_.place(k);
+                const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+                row_[k] = i >= 0 ? load4(m_.row + i) : zero;
+                norm_[k] = i >= 0 ? load4(m_.norm + i) : zero;
+                gate_[k] = i >= 0 ? load4(m_.gates + i) : zero;
+            }
         }
-        __syncthreads();
-        fill_row(xs, m.width, padded, [&](int i) {
-            const int h = i / m.vdim, d = i - h * m.vdim;
-            float s = 0.f;
-            for (int k = 0; k < n; k++) s = fmaf(inv[h * n + k], m.shares.part[((size_t)k * H + h) * m.shares.ld + d], s);
-            return s;
-        });
-    } else if (m.norm) {
-        group_inverse_rms<kThreads>([&](int i) { return m.row[i]; }, m.width, m.heads, m.eps, inv, red);
-        fill_row(xs, m.width, padded, [&](int i) { return m.row[i] * inv[i / m.vdim] * m.norm[i] * sigmoid(m.gates[i]); });
-    } else {
-        copy_row(xs, m.row, m.width, padded);
     }
-}
+    __device__ __forceinline__ void finish(float* xs, int padded, float* inv, float* red) {
+        const int t = threadIdx.x, n = m_.shares.splits, H = m_.heads;
+        if (m_.shares.part) {
+            for (int h = t; h < H; h += kThreads) {  // weights w_k / sum_k w_k sum_k, w_k = 2^(maximum_k - largest)
+                if (!quads_ || h != t) {
+#pragma unroll
+                    for (int k = 0; k < kShares; k++) stats_[k] = stat(min(k, n - 1), h);
+                }
+                float largest = stats_[0].x, all = 0.f, w[kShares];
+#pragma unroll
+                for (int k = 1; k < kShares; k++) largest = fmaxf(largest, stats_[k].x);
+#pragma unroll
+                for (int k = 0; k < kShares; k++) {
+                    w[k] = k < n ? exp2f(stats_[k].x - largest) : 0.f;
+                    all = fmaf(w[k], stats_[k].y, all);
+                }
+                const float share = 1.0f / all;
+#pragma unroll
+                for (int k = 0; k < kShares; k++) inv[h * kShares + k] = w[k] * share;
+            }
+            dense_lds_barrier();
+            if (quads_) {
+                for (int q0 = 0; 4 * q0 < m_.width; q0 += kQuads * kThreads) {
+                    if (q0) request_shares(q0);
+#pragma unroll
+                    for (int u = 0; u < kQuads; u++) {
+                        const int i = 4 * (q0 + u * kThreads + t), h = i / m_.vdim;
+                        if (i >= m_.width) continue;
+                        float4 s = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+                        for (int k = 0; k < kShares; k++) s = fma4(inv[h * kShares + k], shares_[u][k], s);
+                        store4(xs + i, s);
+                    }
+                }
+                for (int i = m_.width + t; i < padded; i += kThreads) xs[i] = 0.f;
+            } else {
+                fill_row(xs, m_.width, padded, [&](int i) {
+                    const int h = i / m_.vdim, d = i - h * m_.vdim;
+                    float s = 0.f;
+                    for (int k = 0; k < n; k++) s = fmaf(inv[h * kShares + k], share_row(k, h)[d], s);
+                    return s;
+                });
+            }
+        } else if (normed_) {
+            const float scale = parts_.inverse_rms(row_, m_.eps, red);
+#pragma unroll
+            for (int k = 0; k < RowParts<kThreads>::kParts; k++) {
+                const int i = parts_.place(k);
+                if (i < 0) continue;
+                const float4 r = row_[k], w = norm_[k], g = gate_[k], v = scale4(r, scale, w);
+                store4(xs + i, make_float4(v.x * sigmoid(g.x), v.y * sigmoid(g.y), v.z * sigmoid(g.z), v.w * sigmoid(g.w)));
+            }
+            for (int i = m_.width + t; i < padded; i += kThreads) xs[i] = 0.f;
+        } else if (m_.norm) {
+            group_inverse_rms<kThreads>([&](int i) { return m_.row[i]; }, m_.width, H, m_.eps, inv, red);
+            fill_row(xs, m_.width, padded, [&](int i) { return m_.row[i] * inv[i / m_.vdim] * m_.norm[i] * sigmoid(m_.gates[i]); });
+        } else {
+            copy_row(xs, m_.row, m_.width, padded);
+        }
+    }
 
-// y[n] = W_o[n] . mixer row + sum_k weights[k] W_e(k)[n] . act_k: a pair of rows of every expert in turn, then of W_o; the
-// loads run one step ahead.
+   private:
+    static constexpr int kShares = kMixerShares, kQuads = 2;
+    __device__ __forceinline__ float2 stat(int k, int h) const {
+        return *reinterpret_cast<const float2*>(m_.shares.stats + 2 * ((size_t)k * m_.heads + h));
+    }
+    __device__ __forceinline__ const float* share_row(int k, int h) const {
+        return m_.shares.part + ((size_t)k * m_.heads + h) * m_.shares.ld;
+    }
+    __device__ __forceinline__ void request_shares(int q0) {
+#pragma unroll
+        for (int u = 0; u < kQuads; u++) {
+            const int i = min(4 * (q0 + u * kThreads + (int)threadIdx.x), m_.width - 4), h = i / m_.vdim;
+#pragma unroll
+            for (int k = 0; k < kShares; k++) shares_[u][k] = load4(share_row(min(k, m_.shares.splits - 1), h) + (i - h * m_.vdim));
+        }
+    }
+    const MixerRow& m_;
+    RowParts<kThreads> parts_;
+    bool quads_, normed_;
+    float2 stats_[kShares];
+    float4 shares_[kQuads][kShares], row_[RowParts<kThreads>::kParts], norm_[RowParts<kThreads>::kParts], gate_[RowParts<kThreads>::kParts];
+};
+
+// y[n] = W_o[n] . mixer row + sum_k weights[k] W_e(k)[n] . act_k, as one row of W_o's and the chosen experts' chunks in turn;
+// the experts' weights are in the activations.
 template <typename T>
 __global__ __launch_bounds__(kThreads) void gemv_mixer_down_kernel(MixerRow m, const T* __restrict__ wo, int ld_wo, ExpertRows e,
                                                                   const float* __restrict__ act, const T* __restrict__ experts, int ld,
                                                                   int N, float* __restrict__ y) {
     extern __shared__ __attribute__((aligned(16))) float smem[];
     __shared__ int chosen[kMaxTop];
-    __shared__ float weights[kMaxTop];
-    const int chunks = ld * (int)sizeof(T) / 16, chunks_wo = ld_wo * (int)sizeof(T) / 16, pairs = (N + 1) / 2;
-    float *xs_mixer = smem, *xs = xs_mixer + ld_wo, *red = xs + e.top * ld, *inv = red + kThreads / 64;
-    const Deal d = deal_rows<T>(chunks_wo, gridDim.x);
-    if ((int)threadIdx.x < e.top) {
-        chosen[threadIdx.x] = min(max(e.chosen[threadIdx.x], 0), e.experts - 1);
-        weights[threadIdx.x] = e.weights[threadIdx.x];
-    }
-    const int parts = e.top + 1, per_step = kAhead * d.lanes;
-    auto rows_of = [&](int n, int k) {
-        return k == 0 ? PlainRows<T>{wo, ld_wo, N}(n) : PlainRows<T>{experts + (size_t)chosen[k - 1] * N * ld, ld, N}(n);
+    const int t = threadIdx.x;
+    const int chunks = ld * (int)sizeof(T) / 16, chunks_wo = ld_wo * (int)sizeof(T) / 16, all = chunks_wo + e.top * chunks;
+    const int pairs = (N + 1) / 2;
+    float *xs = smem, *xs_experts = xs + ld_wo, *red = xs_experts + e.top * ld, *inv = red + kThreads / 64;
+    const Deal d = deal_rows<T>(all, gridDim.x);
+    const float per_chunk = 1.0f / (float)max(chunks, 1);
+    auto load = [&](Pair& p, int n, int c) __attribute__((always_inline)) {
+        const int second = 2 * n + 1 < N ? 1 : 0;
+#pragma unroll
+        for (int u = 0; u < kAhead; u++) {
+            int at = min(c + u * d.lanes, all - 1);
+            size_t row = 2 * (size_t)n;
+            const T* w = wo;
+            int stride = ld_wo;
+            if (at >= chunks_wo) {
+                at -= chunks_wo;
+                const int k = (int)(((float)at + 0.5f) * per_chunk);
+                at -= k * chunks;
+                row += (size_t)chosen[k] * N;
+                w = experts;
+                stride = ld;
+            }
+            const uint4* src = reinterpret_cast<const uint4*>(w + row * stride) + at;
+            p.a[u] = *src;
+            p.b[u] = *reinterpret_cast<const uint4*>(reinterpret_cast<const T*>(src) + (second ? stride : 0));
+        }
     };
     Pair ahead;
-    if (d.group < pairs) load_pair(ahead, rows_of(d.group, 0), d.at, d.lanes, chunks_wo);
-    for (int k = 0; k < e.top; k++) copy_row(xs + k * ld, act + (size_t)k * e.ld_act, e.ff, ld);
-    form_mixer_row(m, xs_mixer, ld_wo, inv, red);
-    __syncthreads();
-    for (int n = d.group; n < pairs; n += d.groups) {
-        float a0 = 0.f, a1 = 0.f;
-        for (int k = 0; k < parts; k++) {
-            const int all = k ? chunks : chunks_wo, steps = (all + per_step - 1) / per_step;
-            const float* row = k ? xs + (k - 1) * ld : xs_mixer;
-            float s0 = 0.f, s1 = 0.f;
-            for (int step = 0; step < steps; step++) {
-                const int c = d.at + step * per_step;
-                const Pair now = ahead;
-                if (step + 1 < steps)
-                    load_pair(ahead, rows_of(n, k), c + per_step, d.lanes, all);
-                else if (k + 1 < parts)
-                    load_pair(ahead, rows_of(n, k + 1), d.at, d.lanes, chunks);
-                else if (n + d.groups < pairs)
-                    load_pair(ahead, rows_of(n + d.groups, 0), d.at, d.lanes, chunks_wo);
-                use_pair<T>(now, row, c, d.lanes, all, s0, s1);
-            }
-            a0 = fmaf(k ? weights[k - 1] : 1.f, s0, a0);
-            a1 = fmaf(k ? weights[k - 1] : 1.f, s1, a1);
+    MixerPrologue row(m);
+    row.load();
+    const bool early = kAhead * d.lanes <= chunks_wo;  // the first step is W_o's alone
+    if (early && d.group < pairs) load(ahead, d.group, d.at);
+    if (t < e.top) chosen[t] = min(max(e.chosen[t], 0), e.experts - 1);
+    if ((e.ff & 3) == 0) {
+        for (int i = t; i < e.top * (e.ff >> 2); i += kThreads) {
+            const int k = i / (e.ff >> 2), c = 4 * (i - k * (e.ff >> 2));
+            const float w = e.weights[k];
+            const float4 v = load4(act + (size_t)k * e.ld_act + c);
+            store4(xs_experts + k * ld + c, make_float4(w * v.x, w * v.y, w * v.z, w * v.w));
         }
-        a0 = dense_wave_sum(a0, d.lanes);
-        a1 = dense_wave_sum(a1, d.lanes);
-        if (d.at == 0) PlainEmit{y, N, 1.f}(n, a0, a1);
+        for (int i = t; i < e.top * (ld - e.ff); i += kThreads) {
+            const int k = i / (ld - e.ff);
+            xs_experts[k * ld + e.ff + (i - k * (ld - e.ff))] = 0.f;
+        }
+    } else {
+        for (int k = 0; k < e.top; k++) {
+            const float w = e.weights[k];
+            fill_row(xs_experts + k * ld, e.ff, ld, [&](int i) { return w * act[(size_t)k * e.ld_act + i]; });
+        }
+    }
+    if (!early) {
+        dense_lds_barrier();
+        if (d.group < pairs) load(ahead, d.group, d.at);
+    }
+    row.finish(xs, ld_wo, inv, red);
+    dense_lds_barrier();
+    const int per_step = kAhead * d.lanes, steps = (all + per_step - 1) / per_step;
+    for (int n = d.group; n < pairs; n += d.groups) {
+        float s0 = 0.f, s1 = 0.f;
+        for (int step = 0; step < steps; step++) {
+            const int c = d.at + step * per_step;
+            const Pair now = ahead;
+            if (step + 1 < steps)
+                load(ahead, n, c + per_step);
+            else if (n + d.groups < pairs)
+                load(ahead, n + d.groups, d.at);
+            use_pair<T>(now, xs, c, d.lanes, all, s0, s1);
+        }
+        s0 = dense_wave_sum(s0, d.lanes);
+        s1 = dense_wave_sum(s1, d.lanes);
+        if (d.at == 0) PlainEmit{y, N, 1.f}(n, s0, s1);
     }
 }
 
@@ -699,9 +808,9 @@ hipError_t launch_gemv_ff_down(const ExpertRows& e, const float* act, const T* e
 template <typename T>
 hipError_t launch_gemv_mixer_down(const MixerRow& m, const T* wo, int ld_wo, const ExpertRows& e, const float* act, const T* experts,
                                   int ld, int N, float* y, hipStream_t s) {
-    const int inv = m.shares.part ? m.heads * m.shares.splits : m.heads;
-    const size_t lds = (ld_wo + (size_t)e.top * ld + kThreads / 64 + inv) * sizeof(float);
-    hipLaunchKernelGGL(gemv_mixer_down_kernel<T>, dim3(workgroups<T>(N, ld_wo, kMaxGrid)), dim3(kThreads), lds, s, m, wo, ld_wo, e, act,
+    const int row = ld_wo + e.top * ld, inv = m.shares.part ? m.heads * kMixerShares : m.heads;
+    const size_t lds = (row + kThreads / 64 + inv) * sizeof(float);
+    hipLaunchKernelGGL(gemv_mixer_down_kernel<T>, dim3(workgroups<T>(N, row, kMaxGrid)), dim3(kThreads), lds, s, m, wo, ld_wo, e, act,
                        experts, ld, N, y);
     return hipGetLastError();
 }

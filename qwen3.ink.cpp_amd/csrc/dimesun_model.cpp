@@ -18,8 +18,6 @@
 namespace a81w41 {
 namespace {
 
-constexpr int kRowShares = 8;  // most shares of a one-token attention: every workgroup of the output product merges them
-
 struct AttentionConfig {
     int heads = 0, kv_heads = 0, dim = 0, vdim = 0, rot_dims = 0, chunk = 0;
     double rot_base = 0;
@@ -43,6 +41,8 @@ struct LayerConfig {
     int mixer_width() const { return memory ? mem.heads * mem.vdim : att.heads * att.vdim; }
     int mixer_columns() const { return memory ? mem.at_f + mem.heads : att.columns(); }
     int columns() const { return mixer_columns() + (routed ? moe.experts : 0); }
+    // floats of a row that leaves the product: all columns, or those that no head takes
+    int row_stride() const { return ((memory ? columns() : columns() - mixer_columns()) + 3) / 4 * 4; }
 };
 struct Config {
     int vocab = 0, width = 0, loop_times = 0;
@@ -81,12 +81,7 @@ MemoryShape read_memory(const Json& m, float eps, const std::string& where) {
     require(s.dim <= 4096 && s.vdim <= 16384 && s.heads <= 4096, where + "matrix memory too large");
     s.q_scale = 1.0f / std::sqrt((float)s.dim);
     s.eps = eps;
-    s.at_q = 0;
-    s.at_k = s.heads * s.dim;
-    s.at_v = s.at_k + s.heads * s.dim;
-    s.at_g = s.at_v + s.heads * s.vdim;
-    s.at_i = s.at_g + s.heads * s.vdim;
-    s.at_f = s.at_i + s.heads;
+    s.place_columns();
     return s;
 }
 
@@ -347,7 +342,7 @@ int DimesunModel<T>::allocate(int max_seq) {
     int top = 0, heads = 0, memory_heads = 0, vdim = 0;
     one_token_fits_ = ld_h_ + 1 <= kGemvMaxRow;
     for (const LayerConfig& lc : cfg_.layers) {
-        ld_in_ = std::max(ld_in_, lc.memory ? lc.columns() : lc.columns() - lc.mixer_columns());
+        ld_in_ = std::max(ld_in_, lc.row_stride());
         ld_attn_ = std::max(ld_attn_, pad_k<T>(lc.mixer_width()));
         int row = pad_k<T>(lc.mixer_width());
         if (lc.memory) {
@@ -359,7 +354,7 @@ int DimesunModel<T>::allocate(int max_seq) {
             q = std::max(q, (size_t)lc.att.heads * lc.att.key_width());
             heads = std::max(heads, lc.att.heads);
             vdim = std::max(vdim, (lc.att.vdim + 3) / 4 * 4);
-            row += lc.att.heads * kRowShares;
+            row += lc.att.heads * kMixerShares;
         }
         if (lc.routed) {
             top = std::max(top, lc.moe.top);
@@ -443,7 +438,7 @@ MemoryArgs DimesunModel<T>::memory_args(const Layer& L, const MemoryShape& sh, c
 template <typename T>
 int DimesunModel<T>::attention(const Layer& L, const LayerConfig& lc, const RunCache& kept, int M, hipStream_t s) {
     const AttentionConfig& c = lc.att;
-    A81W41_HIP_TRY(launch_dense_gemm_heads<T>(product(h_, ld_h_, L.in, nullptr, 0, M), head_rows(L, c, kept, in_, lc.moe.experts), s));
+    A81W41_HIP_TRY(launch_dense_gemm_heads<T>(product(h_, ld_h_, L.in, nullptr, 0, M), head_rows(L, c, kept, in_, lc.row_stride()), s));
     AttendArgs<T> a = attend_args(c, kept, M);
     a.out = attn_;
     if constexpr (kMatrixAttention) {
@@ -460,7 +455,7 @@ int DimesunModel<T>::attention(const Layer& L, const LayerConfig& lc, const RunC
 // The matrix memory on h_: leaves the normed and gated rows in attn_, the router's logits in in_.
 template <typename T>
 int DimesunModel<T>::memory(const Layer& L, const LayerConfig& lc, const RunCache& kept, int M, hipStream_t s) {
-    const int ld = lc.columns();
+    const int ld = lc.row_stride();
     A81W41_HIP_TRY(launch_dense_gemm<T>(product(h_, ld_h_, L.in, in_, ld, M), Epilogue::kFloat, s));
     const MemoryArgs a = memory_args(L, lc.mem, kept, ld, M);
     if (memory_in_chunks(lc.mem, M)) {
@@ -478,7 +473,7 @@ int DimesunModel<T>::routed_experts(const Layer& L, const LayerConfig& lc, int M
     const ExpertsConfig& f = lc.moe;
     const int W = cfg_.width, ld = pad_k<T>(f.ff), cols = pair_columns(f.ff);
     const float* logits = lc.memory ? in_ + lc.mixer_columns() : in_;
-    A81W41_HIP_TRY(launch_router(logits, lc.memory ? lc.columns() : f.experts, L.router_bias, f.experts, f.top, M, chosen_, expert_weights_, s));
+    A81W41_HIP_TRY(launch_router(logits, lc.row_stride(), L.router_bias, f.experts, f.top, M, chosen_, expert_weights_, s));
     A81W41_HIP_TRY(launch_expert_rows(nullptr, chosen_, M, f.top, f.experts, M, src_rows_, slot_rows_, tiles_, n_tiles_, s));
     GemmArgs g = product(h_, ld_h_, L.experts.gate_up, act_, ld, M * f.top);
     g.N = cols, g.w_step = (long long)cols * L.experts.gate_up.ld, g.a_rows = src_rows_;
@@ -501,17 +496,17 @@ int DimesunModel<T>::mixer_one_token(const Layer& L, const LayerConfig& lc, cons
     if (lc.memory) {
         const MemoryShape& sh = lc.mem;
         A81W41_HIP_TRY(launch_gemv_step<T>(step, L.in.data, L.in.ld, L.in.rows, in_, s));
-        A81W41_HIP_TRY(launch_memory_steps(memory_args(L, sh, kept, lc.columns(), 1), mixer_row_, s));
+        A81W41_HIP_TRY(launch_memory_steps(memory_args(L, sh, kept, lc.row_stride(), 1), mixer_row_, s));
         out->heads = sh.heads, out->vdim = sh.vdim, out->norm = L.memory_norm, out->gates = in_ + sh.at_g, out->eps = sh.eps;
         return 0;
     }
     const AttentionConfig& c = lc.att;
-    A81W41_HIP_TRY(launch_gemv_step_heads<T>(step, L.in.data, L.in.ld, L.in.rows, head_rows(L, c, kept, in_, lc.moe.experts), s));
+    A81W41_HIP_TRY(launch_gemv_step_heads<T>(step, L.in.data, L.in.ld, L.in.rows, head_rows(L, c, kept, in_, lc.row_stride()), s));
     AttendArgs<T> a = attend_args(c, kept, 1);
     out->heads = c.heads, out->vdim = c.vdim;
     if constexpr (kMatrixAttention) {
         if (opt_attention_ != 1 && attend_rows_fits(c.key_width(), c.value_width())) {
-            a.splits = std::max(2, std::min(a.splits, kRowShares));  // shares stay fp32; the output product merges them
+            a.splits = std::max(2, std::min(a.splits, kMixerShares));  // shares stay fp32; the output product merges them
             A81W41_HIP_TRY(launch_attend_rows(a, c.kv_heads, s));
             out->shares = LatentShares{a.part, a.part_stats, a.splits, a.ld_part};
             return 0;

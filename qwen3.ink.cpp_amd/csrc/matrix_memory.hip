@@ -151,17 +151,50 @@ __global__ __launch_bounds__(kThreads) void memory_norm_kernel(MemoryArgs a, con
 
 __device__ __forceinline__ f32x16 mfma32(float a, float b, f32x16 c) { return __builtin_amdgcn_mfma_f32_32x32x2f32(a, b, c, 0, 0, 0); }
 
+// W floats (4: aligned to 16 bytes), zeros where there are none
+template <int W>
+__device__ __forceinline__ void read_part(float* part, const float* src, bool real) {
+    if constexpr (W == 4) {
+        const float4 v = real ? load4(src) : make_float4(0.f, 0.f, 0.f, 0.f);
+        part[0] = v.x, part[1] = v.y, part[2] = v.z, part[3] = v.w;
+    } else {
+        part[0] = real ? src[0] : 0.f;
+    }
+}
+template <int W>
+__device__ __forceinline__ void write_part(float* dst, const float* part) {
+    if constexpr (W == 4)
+        store4(dst, make_float4(part[0], part[1], part[2], part[3]));
+    else
+        dst[0] = part[0];
+}
+
 // A chunk's own sums for its last token: sum_s w_s k_s v_s^T and sum_s w_s k_s with w_s = e^(a_s - max a).  A workgroup has
 // a 128 x 128 tile of a head's S; its waves take the 32 x 32 pieces in turn.  K and V sit in LDS as [token][column], column
 // c of token s at place c ^ 32 (s & 1): the two tokens a matrix operand takes at a time lie in different banks.
 constexpr int kOuter = 128;
+template <int W>
 __global__ __launch_bounds__(kThreads) void memory_outer_kernel(MemoryArgs a) {
-    __shared__ float ks[C * kOuter], vs[C * kOuter], weight[C];
+    constexpr int kPer = kOuter / W, kLoads = C * kPer / kThreads, kBatch = W == 4 ? kLoads : 8;
+    __shared__ __attribute__((aligned(16))) float ks[C * kOuter], vs[C * kOuter], weight[C];
     const MemoryShape sh = a.sh;
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6, l31 = lane & 31, half = lane >> 5;
     const int chunk = blockIdx.x, h = blockIdx.y, m0 = chunk * C, count = min(C, a.M - m0);
     const int v_tiles = (sh.vdim + kOuter - 1) / kOuter, d0 = blockIdx.z / v_tiles * kOuter, v0 = blockIdx.z % v_tiles * kOuter;
     const int nd = min(kOuter, sh.dim - d0), nv = min(kOuter, sh.vdim - v0);
+    const int cols_k = (nd + 31) / 32 * 32, cols_v = (nv + 31) / 32 * 32;
+    // the rows are requested before the gates are formed
+    float k_part[kBatch][W], v_part[kBatch][W];
+    auto request = [&](int first) {
+#pragma unroll
+        for (int u = 0; u < kBatch; u++) {
+            const int i = t + (first + u) * kThreads, s = i / kPer, c = i % kPer * W;
+            const float* row = a.in + (size_t)(m0 + min(s, count - 1)) * a.ld_in;
+            read_part<W>(k_part[u], row + sh.at_k + h * sh.dim + d0 + c, s < count && c < nd);
+            read_part<W>(v_part[u], row + sh.at_v + h * sh.vdim + v0 + c, s < count && c < nv);
+        }
+    };
+    request(0);
     if (wave == 0) {
         const ChunkGates g = chunk_gates(a, m0, count, h);
         const double most = __shfl(g.most, 63, 64);
@@ -172,19 +205,18 @@ __global__ __launch_bounds__(kThreads) void memory_outer_kernel(MemoryArgs a) {
             st[1] = (float)g.b;
         }
     }
-    const int cols_k = (nd + 31) / 32 * 32, cols_v = (nv + 31) / 32 * 32;
-#pragma unroll 4
-    for (int i = t; i < C * kOuter; i += kThreads) {
-        const int s = i / kOuter, c = i % kOuter, at = s * kOuter + (c ^ ((s & 1) << 5));
-        const float* row = a.in + (size_t)(m0 + min(s, count - 1)) * a.ld_in;
-        const bool real = s < count;
-        if (c < cols_k) ks[at] = real && c < nd ? row[sh.at_k + h * sh.dim + d0 + c] : 0.f;
-        if (c < cols_v) vs[at] = real && c < nv ? row[sh.at_v + h * sh.vdim + v0 + c] : 0.f;
-    }
-    __syncthreads();
-    for (int i = t; i < C * kOuter; i += kThreads) {
-        const int s = i / kOuter;
-        if (((i % kOuter) ^ ((s & 1) << 5)) < cols_k) ks[i] *= weight[s];
+    dense_lds_barrier();
+    for (int first = 0; first < kLoads; first += kBatch) {
+        if (first) request(first);
+#pragma unroll
+        for (int u = 0; u < kBatch; u++) {
+            const int i = t + (first + u) * kThreads, s = i / kPer, c = i % kPer * W, at = s * kOuter + (c ^ ((s & 1) << 5));
+            const float w = weight[s];
+#pragma unroll
+            for (int e = 0; e < W; e++) k_part[u][e] *= w;
+            write_part<W>(ks + at, k_part[u]);
+            write_part<W>(vs + at, v_part[u]);
+        }
     }
     __syncthreads();
     float* out = a.chunk_states + ((size_t)chunk * sh.heads + h) * sh.chunk_size();
@@ -274,18 +306,48 @@ __global__ __launch_bounds__(kThreads) void memory_chain_kernel(MemoryArgs a, in
     if (scale_writer) a.chunk_m[(size_t)chunks * sh.heads + h] = m;
 }
 
-// Outputs of a chunk for one head, 64 tokens x vdim columns in the accumulators: 64 x 32 VF per wave.
+// Outputs of a chunk for one head, 64 tokens x vdim columns in the accumulators: 64 x 32 VF per wave.  q and k come through
+// LDS, 64 columns at a time; rows of S and v go from memory to the matrix operands, requested ahead of the barriers.
 constexpr int kStep = 64;          // columns of q and k in LDS at a time
 constexpr int kLd = kStep + 4;     // floats of an LDS row: sixteen-byte reads of neighbouring rows spread over the banks
-template <typename T, int VF>
-__global__ __launch_bounds__(kThreads) void memory_outputs_kernel(MemoryArgs a, int chunks, T* __restrict__ out, int ld_out) {
+template <typename T, int W, int WAVES, int VF>
+__global__ __launch_bounds__(64 * WAVES) void memory_outputs_kernel(MemoryArgs a, int chunks, T* __restrict__ out, int ld_out) {
+    constexpr int kT = 64 * WAVES, kPer = kStep / W, kLoads = C * kPer / kT;
+    constexpr int kTeam = kT / C;  // threads that share a token's sums
     __shared__ __attribute__((aligned(16))) float qs[C * kLd], ks[C * kLd];  // ks holds the weighted scores afterwards
     __shared__ double log_a[C], log_most[C];                                // a_s, M_t
-    __shared__ float start[C], floor_t[C], den[C], inv[C], squares[C][kThreads / 64], n_part[kStep];
+    __shared__ float start[C], floor_t[C], den[C], inv[C], squares[C][WAVES], n_part[kStep];
     const MemoryShape sh = a.sh;
     const int t = threadIdx.x, lane = t & 63, wave = t >> 6, l31 = lane & 31, half = lane >> 5;
     const int chunk = blockIdx.x, h = blockIdx.y, m0 = chunk * C, count = min(C, a.M - m0);
     const float m_start = a.chunk_m[(size_t)chunk * sh.heads + h];
+    const float* S = a.chunk_states + ((size_t)chunk * sh.heads + h) * sh.chunk_size();
+    const float* n = S + (size_t)sh.dim * sh.vdim;
+    const int col0 = wave * 32 * VF + l31;
+    float q_part[kLoads][W], k_part[kLoads][W], n_own = 0.f;
+    auto request = [&](int d0) {
+#pragma unroll
+        for (int u = 0; u < kLoads; u++) {
+            const int i = t + u * kT, s = i / kPer, d = d0 + i % kPer * W;
+            const float* row = a.in + (size_t)(m0 + min(s, count - 1)) * a.ld_in + h * sh.dim + d;
+            const bool real = s < count && d < sh.dim;
+            read_part<W>(q_part[u], row + sh.at_q, real);
+            read_part<W>(k_part[u], row + sh.at_k, real);
+        }
+        if (t < kStep) n_own = d0 + t < sh.dim ? n[d0 + t] : 0.f;
+    };
+    constexpr int kHalf = kStep / 16;  // operand steps of eight columns: half of those of a pass
+    float b[kHalf][VF][4];
+    auto request_states = [&](int d0) {
+#pragma unroll
+        for (int kk = 0; kk < kHalf; kk++)
+#pragma unroll
+            for (int f = 0; f < VF; f++)
+#pragma unroll
+                for (int j = 0; j < 4; j++)
+                    b[kk][f][j] = S[(size_t)min(d0 + 4 * (2 * kk + half) + j, sh.dim - 1) * sh.vdim + min(col0 + 32 * f, sh.vdim - 1)];
+    };
+    request(0);
     if (wave == 0) {
         const ChunkGates g = chunk_gates(a, m0, count, h);
         const double most = fmax((double)m_start, g.most);
@@ -297,9 +359,6 @@ __global__ __launch_bounds__(kThreads) void memory_outputs_kernel(MemoryArgs a, 
     // the scale after the last chunk goes to the state only now: the chain's workgroups all read the old one
     if (chunk == chunks - 1 && t == 0)
         state_nm(a, max(a.pos_dev[0], 0) + a.M)[(size_t)h * (sh.dim + 1) + sh.dim] = a.chunk_m[(size_t)chunks * sh.heads + h];
-    const float* S = a.chunk_states + ((size_t)chunk * sh.heads + h) * sh.chunk_size();
-    const float* n = S + (size_t)sh.dim * sh.vdim;
-    const int col0 = wave * 32 * VF + l31;
     f32x16 acc[2][VF], score;
 #pragma unroll
     for (int i = 0; i < 16; i++) {
@@ -307,105 +366,127 @@ __global__ __launch_bounds__(kThreads) void memory_outputs_kernel(MemoryArgs a, 
 #pragma unroll
         for (int f = 0; f < VF; f++) acc[0][f][i] = acc[1][f][i] = 0.f;
     }
-    const int st = (wave & 1) * 32, ss = (wave >> 1) * 32;  // this wave's piece of the scores: tokens st.., keys ss..
-    float nq = 0.f;                                          // of token t / 4, a quarter of the columns
+    // this wave's piece of the scores, tokens st.. and keys ss..; the waves from 4 on take every second operand step
+    const int st = (wave & 1) * 32, ss = (wave >> 1 & 1) * 32;
+    float nq = 0.f;  // of token t / kTeam, a share of the columns
     for (int d0 = 0; d0 < sh.dim; d0 += kStep) {
-        __syncthreads();
-#pragma unroll 4
-        for (int i = t; i < C * kStep; i += kThreads) {
-            const int s = i / kStep, c = i % kStep, d = d0 + c;
-            const float* row = a.in + (size_t)(m0 + min(s, count - 1)) * a.ld_in + h * sh.dim + min(d, sh.dim - 1);
-            const bool real = s < count && d < sh.dim;
-            qs[s * kLd + c] = real ? row[sh.at_q] * sh.q_scale : 0.f;
-            ks[s * kLd + c] = real ? row[sh.at_k] : 0.f;
+        request_states(d0);
+        if (d0) dense_lds_barrier();  // nobody still reads the columns before
+#pragma unroll
+        for (int u = 0; u < kLoads; u++) {
+            const int i = t + u * kT, at = i / kPer * kLd + i % kPer * W;
+#pragma unroll
+            for (int e = 0; e < W; e++) q_part[u][e] *= sh.q_scale;
+            write_part<W>(qs + at, q_part[u]);
+            write_part<W>(ks + at, k_part[u]);
         }
-        if (t < kStep) n_part[t] = d0 + t < sh.dim ? n[d0 + t] : 0.f;
-        __syncthreads();
-        const int steps = (min(kStep, sh.dim - d0) + 7) / 8;
-        for (int kk = 0; kk < steps; kk++) {
-            const int at = 4 * (2 * kk + half);
-            alignas(16) float q[2][4], k[4];
+        if (t < kStep) n_part[t] = n_own;
+        dense_lds_barrier();
+        if (d0 + kStep < sh.dim) request(d0 + kStep);
 #pragma unroll
-            for (int i = 0; i < 2; i++) *reinterpret_cast<float4*>(q[i]) = load4(qs + (i * 32 + l31) * kLd + at);
-            *reinterpret_cast<float4*>(k) = load4(ks + (ss + l31) * kLd + at);
+        for (int part = 0; part < 2; part++) {
+            if (part) request_states(d0 + kStep / 2);
+            if (d0 + part * (kStep / 2) >= sh.dim) break;
 #pragma unroll
-            for (int f = 0; f < VF; f++) {
-                const int col = min(col0 + 32 * f, sh.vdim - 1);
-                float b[4];
+            for (int kk = 0; kk < kHalf; kk++) {
+                const int step = part * kHalf + kk, at = 4 * (2 * step + half);
+                alignas(16) float q[2][4], k[4];
 #pragma unroll
-                for (int j = 0; j < 4; j++) b[j] = S[(size_t)min(d0 + at + j, sh.dim - 1) * sh.vdim + col];
+                for (int i = 0; i < 2; i++) *reinterpret_cast<float4*>(q[i]) = load4(qs + (i * 32 + l31) * kLd + at);
+#pragma unroll
+                for (int f = 0; f < VF; f++)
+#pragma unroll
+                    for (int j = 0; j < 4; j++)
+#pragma unroll
+                        for (int i = 0; i < 2; i++) acc[i][f] = mfma32(q[i][j], b[kk][f][j], acc[i][f]);
+                // a piece whose keys all come later counts nothing
+                if (ss <= st && (WAVES == 4 || (step & 1) == wave >> 2)) {
+                    *reinterpret_cast<float4*>(k) = load4(ks + (ss + l31) * kLd + at);
+#pragma unroll
+                    for (int j = 0; j < 4; j++) score = mfma32(st ? q[1][j] : q[0][j], k[j], score);
+                }
+            }
+        }
+#pragma unroll
+        for (int c = 0; c < kStep / kTeam; c++) {
+            const int d = t % kTeam + kTeam * c;
+            nq = fmaf(qs[t / kTeam * kLd + d], n_part[d], nq);
+        }
+    }
+    // the first rows of v, while the scores are weighted
+    constexpr int kRowsAhead = 4;
+    const float* v_rows = a.in + sh.at_v + h * sh.vdim;
+    float v[kRowsAhead][VF][4];
+    auto request_values = [&](int kk0) {
+#pragma unroll
+        for (int kk = 0; kk < kRowsAhead; kk++)
+#pragma unroll
+            for (int f = 0; f < VF; f++)
 #pragma unroll
                 for (int j = 0; j < 4; j++)
-#pragma unroll
-                    for (int i = 0; i < 2; i++) acc[i][f] = mfma32(q[i][j], b[j], acc[i][f]);
-            }
-            if (ss <= st) {  // a piece whose keys all come later counts nothing
-#pragma unroll
-                for (int j = 0; j < 4; j++) score = mfma32(st ? q[1][j] : q[0][j], k[j], score);
-            }
-        }
-#pragma unroll
-        for (int c = 0; c < kStep / 4; c++) {
-            const int d = (t & 3) + 4 * c;
-            nq = fmaf(qs[(t >> 2) * kLd + d], n_part[d], nq);
-        }
-    }
-    __syncthreads();
+                    v[kk][f][j] = v_rows[(size_t)(m0 + min(4 * (2 * (kk0 + kk) + half) + j, count - 1)) * a.ld_in + min(col0 + 32 * f, sh.vdim - 1)];
+    };
+    request_values(0);
+    dense_lds_barrier();
     float* weighted = ks;  // [token][key]
+    for (int turn = 0; turn < WAVES / 4; turn++) {
+        if (wave >> 2 == turn) {
 #pragma unroll
-    for (int i = 0; i < 16; i++) {
-        const int token = st + 8 * (i >> 2) + 4 * half + (i & 3), key = ss + l31;
-        weighted[token * kLd + key] = key <= token ? score[i] * expf((float)(log_a[key] - log_most[token])) : 0.f;
+            for (int i = 0; i < 16; i++) {
+                const int token = st + 8 * (i >> 2) + 4 * half + (i & 3), key = ss + l31;
+                float& w = weighted[token * kLd + key];
+                const float own = key <= token ? score[i] * expf((float)(log_a[key] - log_most[token])) : 0.f;
+                w = turn ? w + own : own;
+            }
+        }
+        dense_lds_barrier();
     }
 #pragma unroll
     for (int i = 0; i < 2; i++)
 #pragma unroll
-        for (int v = 0; v < 16; v++) {
-            const float w = start[i * 32 + 8 * (v >> 2) + 4 * half + (v & 3)];
+        for (int r = 0; r < 16; r++) {
+            const float w = start[i * 32 + 8 * (r >> 2) + 4 * half + (r & 3)];
 #pragma unroll
-            for (int f = 0; f < VF; f++) acc[i][f][v] *= w;
+            for (int f = 0; f < VF; f++) acc[i][f][r] *= w;
         }
-    __syncthreads();
     {
-        const int token = t >> 2;
+        const int token = t / kTeam;
         float sum = nq * start[token];
 #pragma unroll
-        for (int c = 0; c < C / 4; c++) sum += weighted[token * kLd + (t & 3) + 4 * c];
-        sum = dense_wave_sum(sum, 4);
-        if ((t & 3) == 0) den[token] = 1.0f / (fmaxf(fabsf(sum), floor_t[token]) + kMemoryFloor);
+        for (int c = 0; c < C / kTeam; c++) sum += weighted[token * kLd + t % kTeam + kTeam * c];
+        sum = dense_wave_sum(sum, kTeam);
+        if (t % kTeam == 0) den[token] = 1.0f / (fmaxf(fabsf(sum), floor_t[token]) + kMemoryFloor);
     }
-    const float* v_rows = a.in + sh.at_v + h * sh.vdim;
-#pragma unroll 2
-    for (int kk = 0; kk < C / 8; kk++) {
-        const int at = 4 * (2 * kk + half);
-        alignas(16) float p[2][4];
 #pragma unroll
-        for (int i = 0; i < 2; i++) *reinterpret_cast<float4*>(p[i]) = load4(weighted + (i * 32 + l31) * kLd + at);
+    for (int kk0 = 0; kk0 < C / 8; kk0 += kRowsAhead) {
+        if (kk0) request_values(kk0);
 #pragma unroll
-        for (int f = 0; f < VF; f++) {
-            const int col = min(col0 + 32 * f, sh.vdim - 1);
-            float b[4];
+        for (int kk = 0; kk < kRowsAhead; kk++) {
+            const int at = 4 * (2 * (kk0 + kk) + half);
+            alignas(16) float p[2][4];
 #pragma unroll
-            for (int j = 0; j < 4; j++) b[j] = v_rows[(size_t)(m0 + min(at + j, count - 1)) * a.ld_in + col];
+            for (int i = 0; i < 2; i++) *reinterpret_cast<float4*>(p[i]) = load4(weighted + (i * 32 + l31) * kLd + at);
 #pragma unroll
-            for (int j = 0; j < 4; j++) {
-                if (kk < C / 16) acc[0][f] = mfma32(p[0][j], b[j], acc[0][f]);
-                acc[1][f] = mfma32(p[1][j], b[j], acc[1][f]);
-            }
+            for (int f = 0; f < VF; f++)
+#pragma unroll
+                for (int j = 0; j < 4; j++) {
+                    if (kk0 + kk < C / 16) acc[0][f] = mfma32(p[0][j], v[kk][f][j], acc[0][f]);
+                    acc[1][f] = mfma32(p[1][j], v[kk][f][j], acc[1][f]);
+                }
         }
     }
-    __syncthreads();
+    dense_lds_barrier();
 #pragma unroll
     for (int i = 0; i < 2; i++)
 #pragma unroll
-        for (int v = 0; v < 16; v++) {
-            const int token = i * 32 + 8 * (v >> 2) + 4 * half + (v & 3);
+        for (int r = 0; r < 16; r++) {
+            const int token = i * 32 + 8 * (r >> 2) + 4 * half + (r & 3);
             const float d = den[token];
             float sum = 0.f;
 #pragma unroll
             for (int f = 0; f < VF; f++) {
-                acc[i][f][v] *= d;
-                if (col0 + 32 * f < sh.vdim) sum = fmaf(acc[i][f][v], acc[i][f][v], sum);
+                acc[i][f][r] *= d;
+                if (col0 + 32 * f < sh.vdim) sum = fmaf(acc[i][f][r], acc[i][f][r], sum);
             }
             sum = dense_wave_sum(sum, 32);
             if (l31 == 0) squares[token][wave] = sum;
@@ -413,7 +494,7 @@ __global__ __launch_bounds__(kThreads) void memory_outputs_kernel(MemoryArgs a, 
     __syncthreads();
     if (t < C) {
         float sum = 0.f;
-        for (int w = 0; w < kThreads / 64; w++) sum += squares[t][w];
+        for (int w = 0; w < WAVES; w++) sum += squares[t][w];
         inv[t] = 1.0f / sqrtf(sum / (float)sh.vdim + sh.eps);
     }
     __syncthreads();
@@ -423,18 +504,45 @@ __global__ __launch_bounds__(kThreads) void memory_outputs_kernel(MemoryArgs a, 
         if (col >= sh.vdim) continue;
         const float w = a.norm[h * sh.vdim + col];
 #pragma unroll
-        for (int i = 0; i < 2; i++)
+        for (int i = 0; i < 2; i++) {
+            float gate[16];
 #pragma unroll
-            for (int v = 0; v < 16; v++) {
-                const int token = i * 32 + 8 * (v >> 2) + 4 * half + (v & 3);
-                if (token >= count) continue;
-                const float gate = a.in[(size_t)(m0 + token) * a.ld_in + sh.at_g + h * sh.vdim + col];
-                out[(size_t)(m0 + token) * ld_out + h * sh.vdim + col] = (T)(acc[i][f][v] * inv[token] * w * sigmoid(gate));
+            for (int r = 0; r < 16; r++) {
+                const int token = min(i * 32 + 8 * (r >> 2) + 4 * half + (r & 3), count - 1);
+                gate[r] = a.in[(size_t)(m0 + token) * a.ld_in + sh.at_g + h * sh.vdim + col];
             }
+#pragma unroll
+            for (int r = 0; r < 16; r++) {
+                const int token = i * 32 + 8 * (r >> 2) + 4 * half + (r & 3);
+                if (token < count)
+                    out[(size_t)(m0 + token) * ld_out + h * sh.vdim + col] = (T)(acc[i][f][r] * inv[token] * w * sigmoid(gate[r]));
+            }
+        }
     }
 }
 
-bool whole_quads(const MemoryShape& sh) { return sh.dim % 4 == 0 && sh.vdim % 4 == 0; }
+// whether heads, rows and what is read of them are whole float4s
+bool whole_quads(const MemoryArgs& a) {
+    const MemoryShape& sh = a.sh;
+    return (sh.dim | sh.vdim | a.ld_in | sh.at_q | sh.at_k | sh.at_v) % 4 == 0;
+}
+
+template <typename T, int W>
+hipError_t launch_chunks(const MemoryArgs& a, T* out, int ld_out, hipStream_t s) {
+    const MemoryShape& sh = a.sh;
+    const int chunks = (a.M + C - 1) / C, tiles = ((sh.dim + kOuter - 1) / kOuter) * ((sh.vdim + kOuter - 1) / kOuter);
+    const int parts = (int)(sh.chunk_size() / W);
+    hipLaunchKernelGGL(memory_outer_kernel<W>, dim3(chunks, sh.heads, tiles), dim3(kThreads), 0, s, a);
+    hipLaunchKernelGGL(memory_chain_kernel<W>, dim3((parts + kThreads - 1) / kThreads, sh.heads), dim3(kThreads), 0, s, a, chunks);
+    const dim3 grid(chunks, sh.heads);
+    if (sh.vdim <= 128)
+        hipLaunchKernelGGL((memory_outputs_kernel<T, W, 4, 1>), grid, dim3(256), 0, s, a, chunks, out, ld_out);
+    else if (sh.vdim <= 256)
+        hipLaunchKernelGGL((memory_outputs_kernel<T, W, 8, 1>), grid, dim3(512), 0, s, a, chunks, out, ld_out);
+    else
+        hipLaunchKernelGGL((memory_outputs_kernel<T, W, 8, 2>), grid, dim3(512), 0, s, a, chunks, out, ld_out);
+    return hipGetLastError();
+}
 
 }  // namespace
 
@@ -458,23 +566,7 @@ bool memory_chunks_fit(const MemoryShape& sh) { return sh.vdim <= 512; }
 
 template <typename T>
 hipError_t launch_memory_chunks(const MemoryArgs& a, T* out, int ld_out, hipStream_t s) {
-    const MemoryShape& sh = a.sh;
-    const int chunks = (a.M + C - 1) / C, tiles = ((sh.dim + kOuter - 1) / kOuter) * ((sh.vdim + kOuter - 1) / kOuter);
-    hipLaunchKernelGGL(memory_outer_kernel, dim3(chunks, sh.heads, tiles), dim3(kThreads), 0, s, a);
-    const int size = (int)sh.chunk_size();
-    // four elements at a time where all parts are whole quads; n's copies start behind odd numbers of floats otherwise
-    if (whole_quads(sh))
-        hipLaunchKernelGGL(memory_chain_kernel<4>, dim3((size / 4 + kThreads - 1) / kThreads, sh.heads), dim3(kThreads), 0, s, a, chunks);
-    else
-        hipLaunchKernelGGL(memory_chain_kernel<1>, dim3((size + kThreads - 1) / kThreads, sh.heads), dim3(kThreads), 0, s, a, chunks);
-    const dim3 grid(chunks, sh.heads), block(kThreads);
-    if (sh.vdim <= 128)
-        hipLaunchKernelGGL((memory_outputs_kernel<T, 1>), grid, block, 0, s, a, chunks, out, ld_out);
-    else if (sh.vdim <= 256)
-        hipLaunchKernelGGL((memory_outputs_kernel<T, 2>), grid, block, 0, s, a, chunks, out, ld_out);
-    else
-        hipLaunchKernelGGL((memory_outputs_kernel<T, 4>), grid, block, 0, s, a, chunks, out, ld_out);
-    return hipGetLastError();
+    return whole_quads(a) ? launch_chunks<T, 4>(a, out, ld_out, s) : launch_chunks<T, 1>(a, out, ld_out, s);
 }
 
 #define INSTANTIATE(T)                                                                                   \

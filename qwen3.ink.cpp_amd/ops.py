@@ -239,6 +239,53 @@ def formed_attention(q, k, k_rot, v_t, gates, pos: int, vdim: int, scale: float)
     return out
 
 
+def grouped_attention(q, rows, pos: int, kv_heads: int, key_width: int, vdim: int, scale: float, chunk: int = 0, sink: bool = False,
+                      variant: int = 0, splits: int = 1):
+    """Parity hook a81w41_grouped_attention: q [M][heads][key_width], rows [max_seq][ld] of kv_heads x [value | key]
+    -> [M][heads][vdim] of q's type."""
+    torch = _torch()
+    M, heads, _ = q.shape
+    value_width = (vdim + 7) // 8 * 8
+    out = torch.empty((M, heads, vdim), dtype=q.dtype, device=q.device)
+    pos_dev = torch.tensor([pos], dtype=torch.int32, device=q.device)
+    part = torch.empty((splits * M * heads, (vdim + 3) // 4 * 4), dtype=torch.float32, device=q.device)
+    stats = torch.empty((splits * M * heads, 2), dtype=torch.float32, device=q.device)
+    capi.check(capi.dense().a81w41_grouped_attention(
+        _dev_ptr(q), _dev_ptr(rows), rows.shape[1], heads, kv_heads, key_width, value_width, vdim, _dev_ptr(pos_dev), rows.shape[0], M,
+        scale, chunk, int(sink), _dev_ptr(out), _element(q), variant, splits, _dev_ptr(part), _dev_ptr(stats), _stream()))
+    return out
+
+
+def matrix_memory_state(heads: int, dim: int, vdim: int):
+    """The state of a new sequence for ``matrix_memory``."""
+    torch = _torch()
+    return torch.zeros(capi.dense().a81w41_matrix_memory_state(heads, dim, vdim), dtype=torch.float32, device="cuda")
+
+
+def matrix_memory(rows, heads: int, dim: int, vdim: int, cap: float, eps: float, bias_i, bias_f, norm, state, pos: int, variant: int = 0):
+    """Parity hook a81w41_matrix_memory: rows [M][ld] fp32 at positions pos .. -> fp32 [M][heads*vdim]; state is carried on."""
+    torch = _torch()
+    M = rows.shape[0]
+    out = torch.empty((M, heads * vdim), dtype=torch.float32, device=rows.device)
+    scratch = torch.empty(capi.dense().a81w41_matrix_memory_scratch(heads, dim, vdim, M), dtype=torch.float32, device=rows.device)
+    pos_dev = torch.tensor([pos], dtype=torch.int32, device=rows.device)
+    capi.check(capi.dense().a81w41_matrix_memory(
+        _dev_ptr(rows), rows.shape[1], M, heads, dim, vdim, cap, eps, _dev_ptr(bias_i), _dev_ptr(bias_f), _dev_ptr(norm),
+        _dev_ptr(state), _dev_ptr(pos_dev), variant, _dev_ptr(scratch), _dev_ptr(out), _stream()))
+    return out
+
+
+def router(logits, bias, top: int):
+    """Parity hook a81w41_router: logits [M][experts] fp32, bias [experts] -> (chosen int32 [M][top], weights fp32 [M][top])."""
+    torch = _torch()
+    M, experts = logits.shape
+    chosen = torch.empty((M, top), dtype=torch.int32, device=logits.device)
+    weights = torch.empty((M, top), dtype=torch.float32, device=logits.device)
+    capi.check(capi.dense().a81w41_router(_dev_ptr(logits), experts, _dev_ptr(bias), experts, top, M, _dev_ptr(chosen), _dev_ptr(weights),
+                                          _stream()))
+    return chosen, weights
+
+
 # ---------------------------------------------------------------- layer objects
 
 class Context:
