@@ -123,11 +123,15 @@ def clamped_expert(h, tensor, prefix, limit):
     return (g * sigmoid(1.702 * g) * (u + 1.0)) @ tensor(prefix + "down").T
 
 
-def routed_experts(h, mlp, tensor):
-    logits = h @ tensor("router").T + tensor("router.b")
+def routed_experts(h, mlp, tensor, margins=None):
+    """margins [T], if given, falls to the distance between the last chosen and the first other logit of a token."""
+    logits, top = h @ tensor("router").T + tensor("router.b"), mlp["router"]["top"]
     out = np.zeros_like(h)
     for t in range(h.shape[0]):
-        for e, w in zip(*choose(logits[t], mlp["router"]["top"])):
+        if margins is not None and top < logits.shape[1]:
+            rising = np.sort(logits[t])
+            margins[t] = min(margins[t], rising[-top] - rising[-top - 1])
+        for e, w in zip(*choose(logits[t], top)):
             out[t] += w * clamped_expert(h[t], tensor, f"e{e}.", mlp["expert"]["limit"])
     return out
 
@@ -144,12 +148,16 @@ def layer_runs(config):
 
 
 class DimesunOracle:
-    def __init__(self, config: dict, weights: dict):
+    """normed_as: applied to every normed row, for instance round_bf16, to see what rounding alone does to a sequence."""
+
+    def __init__(self, config: dict, weights: dict, normed_as=None):
         self.cfg = config
+        self.normed_as = normed_as or (lambda h: h)
         self.w = {k: np.asarray(v, np.float64) for k, v in weights.items()}
 
-    def forward(self, ids, layer_states: list | None = None):
-        """token ids of one sequence -> logits [T, vocab]; appends the stream after every layer run to layer_states."""
+    def forward(self, ids, layer_states: list | None = None, margins: np.ndarray | None = None):
+        """token ids of one sequence -> logits [T, vocab]; appends the stream after every layer run to layer_states; margins
+        [T] falls to the closest call of a router for each token."""
         cfg, w, eps = self.cfg, self.w, self.cfg["norm"]["eps"]
         ids = [int(i) for i in ids]
         positions = np.arange(len(ids))
@@ -158,18 +166,18 @@ class DimesunOracle:
             layer = cfg["layers"][i]
             if opens is not None:
                 x = x + w["loop.step"][opens]
-            h = norm_around_zero(x, w[f"l{i}.norm1"], eps)
+            h = self.normed_as(norm_around_zero(x, w[f"l{i}.norm1"], eps))
             mix = lambda name, i=i: w[f"l{i}.mix.{name}"]  # noqa: E731
             if layer["type"] == "mlstm":
                 y = mlstm(h, layer["mixer"], mix, eps)
             else:
                 y = attention(h, layer["mixer"], mix, positions)
             if layer.get("mlp"):
-                y = y + routed_experts(h, layer["mlp"], lambda name, i=i: w[f"l{i}.mlp.{name}"])
+                y = y + routed_experts(h, layer["mlp"], lambda name, i=i: w[f"l{i}.mlp.{name}"], margins)
             x = x + cfg["residual_mult"] * y
             if layer_states is not None:
                 layer_states.append(x)
-        return norm_around_zero(x, w["final.norm"], eps) @ w["embed"].T
+        return self.normed_as(norm_around_zero(x, w["final.norm"], eps)) @ w["embed"].T
 
 
 def greedy(oracle: DimesunOracle, prompt, n_new):
@@ -200,6 +208,8 @@ def random_weights(config: dict, seed: int, bf16=True) -> dict:
         if layer["type"] == "mlstm":
             lin(mix + "q", H * D, W, 1.5)
             lin(mix + "k", H * D, W)
+            # a token's key resembles its query, so that a head's output, which is scaled to size one, is seldom near zero
+            out[mix + "k"] = 0.7 * out[mix + "k"] + 0.5 * out[mix + "q"]
             lin(mix + "v", H * V, W)
             lin(mix + "g", H * V, W)
             lin(mix + "o", W, H * V)

@@ -8,6 +8,7 @@ import numpy as np
 import pytest
 
 from oracle import takosun_forward as tf
+from tests import dimesun_fixture
 from tests.takosun_fixture import SMALL, write_model
 
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
@@ -18,8 +19,8 @@ def refused(pkg, cfg, match):
         pkg.Model.random(cfg, 16)
 
 
-def edit(path, value):
-    cfg = copy.deepcopy(SMALL)
+def edit(path, value, of=SMALL):
+    cfg = copy.deepcopy(of)
     at = cfg
     for k in path[:-1]:
         at = at[k]
@@ -46,6 +47,29 @@ def edit(path, value):
 ])
 def test_bad_configurations_are_refused(pkg, path, value, match):
     refused(pkg, edit(path, value), match)
+
+
+@pytest.mark.parametrize("path,value,match", [
+    (["residual_mult"], None, "missing key 'residual_mult'"),
+    (["norm", "eps"], -1.0, "norm.eps"),
+    (["layers", 1, "type"], "latent_attention", "layer 1: unknown type"),
+    (["layers", 1, "mixer", "kv_heads"], 4, "multiple of kv_heads"),
+    (["layers", 1, "mixer", "rot", "dims"], 26, "rot.dims"),
+    (["layers", 1, "mixer", "rot", "dims"], 3, "rot.dims"),
+    (["layers", 1, "mixer", "mask"], None, "missing key 'mask'"),
+    (["layers", 1, "mixer", "mask", "size"], 0, "'size' is out of range"),
+    (["layers", 0, "mixer", "gate_cap"], 0.0, "gate_cap"),
+    (["layers", 0, "mixer", "vdim"], None, "missing key 'vdim'"),
+    (["layers", 0, "mlp", "kind"], "dense", "unknown feed-forward"),
+    (["layers", 0, "mlp", "router", "top"], 6, "router out of range"),
+    (["layers", 0, "mlp", "expert", "limit"], None, "missing key 'limit'"),
+    (["loop", "stop"], 6, "loop.start"),
+    (["loop", "start"], 4, "loop.start"),
+    (["loop", "times"], 0, "'times' is out of range"),
+    (["layers"], [], "no layers"),
+])
+def test_bad_dimesun_configurations_are_refused(pkg, path, value, match):
+    refused(pkg, edit(path, value, dimesun_fixture.SMALL), match)
 
 
 def test_unknown_architecture(pkg):
