@@ -792,8 +792,10 @@ hipError_t launch_gemv_gate_up(const RowStep& p, const float* h, const ExpertRow
     const int most = e.top && e.ff > e.dense_ff ? e.ff : e.dense_ff;
     const int slots = e.top + (e.dense_ff ? 1 : 0);
     const size_t router = e.logits ? (ld + e.experts) * sizeof(float) : 0, lds = step_lds(ld, p);
-    hipLaunchKernelGGL(gemv_gate_up_kernel<T>, dim3(workgroups<T>(2 * most, ld, kMaxGrid), slots), dim3(kThreads), lds > router ? lds : router,
-                       s, p, h, e, experts, dense, ld, act);
+    // behind a router a workgroup first has to learn its expert: two rounds of rows for each of the 512 that fit the chip at once
+    const int limit = e.logits && slots < 16 ? 512 / slots : e.logits ? 32 : kMaxGrid;
+    hipLaunchKernelGGL(gemv_gate_up_kernel<T>, dim3(workgroups<T>(2 * most, ld, limit), slots), dim3(kThreads), lds > router ? lds : router, s,
+                       p, h, e, experts, dense, ld, act);
     return hipGetLastError();
 }
 template <typename T>
