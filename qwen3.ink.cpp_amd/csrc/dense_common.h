@@ -18,7 +18,6 @@ __device__ __forceinline__ float dense_wave_max(float v, int width = 64) {
     return v;
 }
 __device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float silu(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float gated_unit(const GatedUnit& p, float gate, float up) {
     const float g = fminf(gate, p.limit), u = fminf(fmaxf(up, -p.limit), p.limit);
     return g / (1.0f + expf(-p.slope * g)) * (u + p.shift);
